@@ -43,6 +43,8 @@ extra = {
         "-std=c++17",
         "--offload-arch=gfx950",
         "-fno-gpu-rdc",
+        # no packed fp32 arithmetic in device code
+        "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
     ],
 }
 
