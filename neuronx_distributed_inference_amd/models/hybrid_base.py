@@ -10,7 +10,8 @@ attention layers with recurrent layers on an fp32 residual stream).
 - one :class:`BlockKVCacheManager` whose per-run page shapes, lenders and
   recurrent-state tensors are collected from the layers: a layer exposes
   ``kv_shape()`` (None when it owns no pages), ``kv_source()`` (layer index
-  it borrows pages from, or None) and ``state_shapes()``;
+  it borrows pages from, or None) and ``state_shapes()``; state that belongs
+  to no layer comes from :meth:`HybridDecoderModel.model_state`;
 - the fp32 residual stream (embedding widened, optionally scaled).
 
 A subclass builds its layers and may override :meth:`run_order` (layers that
@@ -55,6 +56,10 @@ class HybridDecoderModel(DecoderModel):
         """Layer index of every layer run, in execution order."""
         return list(range(len(self.layers)))
 
+    def model_state(self) -> Dict[str, tuple]:
+        """Per-sequence state outside the layers: name -> (shape, dtype)."""
+        return {}
+
     def build_kv_manager(self, config) -> nn.Module:
         from neuronx_distributed_inference_amd.modules.kvcache.block_kv_cache_manager import (
             BlockKVCacheManager,
@@ -83,6 +88,8 @@ class HybridDecoderModel(DecoderModel):
         for ri, li in enumerate(self._order):
             for name, shape in self.layers[li].state_shapes().items():
                 mgr.state.register(f"run{ri}.{name}", shape)
+        for name, (shape, dtype) in self.model_state().items():
+            mgr.state.register(name, shape, dtype)
         return mgr
 
     # -- engine hooks ---------------------------------------------------

@@ -172,6 +172,10 @@ class DecoderModel(nn.Module):
         context on the cache manager and returns the block table to use."""
         return block_table
 
+    def embed(self, input_ids: torch.Tensor) -> torch.Tensor:
+        """Embedding rows of the step's tokens (after :meth:`begin_step`)."""
+        return self.embed_tokens(input_ids)
+
     def prepare_hidden(self, h: torch.Tensor) -> torch.Tensor:
         """Embedding output -> residual stream (e.g. a widening cast)."""
         return h
@@ -234,7 +238,7 @@ class DecoderModel(nn.Module):
             and phase == PHASE_CTE and tp > 1 and S % tp == 0 and S >= tp
         )
         h = self.embed_tokens(input_ids, sequence_parallel=sp_active) \
-            if sp_active else self.embed_tokens(input_ids)
+            if sp_active else self.embed(input_ids)
         # multimodal splice (llava/pixtral pattern): projected vision
         # features replace the image-placeholder token embeddings. The mask
         # derives from input_ids, so bucket padding is handled for free.

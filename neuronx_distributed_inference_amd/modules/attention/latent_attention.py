@@ -10,7 +10,10 @@ part. With ``sink`` the softmax denominator carries one extra term
 ``exp(sink_h)`` per head: a key without a value, unscaled. With ``window``
 query ``i`` sees keys ``i - window < j <= i`` only. A ``gate`` handed to
 the call multiplies the concatenated heads by ``sigmoid(gate)`` element by
-element.
+element, or head by head with ``gate_per_head``. ``half_split`` pairs rotated
+channel ``i`` with ``i + rot_dims/2`` instead of neighbours. A module built
+with ``owns_kv=False`` stores nothing and reads the rows of the layer its
+cache index is mapped to (``dkv`` is None then), with its own up-projections.
 
 Steps that continue a sequence (decoded tokens, later prompt portions, mixed
 batches) are computed in the *absorbed* form, which never expands the cache:
@@ -46,7 +49,8 @@ from neuronx_distributed_inference_amd.ops import seqmix
 class LatentSinkAttention(nn.Module):
     def __init__(self, num_heads: int, dim: int, rot_dim: int, v_dim: int, kv_rank: int,
                  scale: float, eps: float, rope_base: float, rot_dims: int,
-                 dtype: torch.dtype, sink: bool = True, window: Optional[int] = None):
+                 dtype: torch.dtype, sink: bool = True, window: Optional[int] = None,
+                 half_split: bool = False, gate_per_head: bool = False, owns_kv: bool = True):
         super().__init__()
         assert rot_dims <= rot_dim and rot_dims % 2 == 0
         self.num_heads = num_heads
@@ -57,7 +61,11 @@ class LatentSinkAttention(nn.Module):
         self.scale = float(scale)
         self.window = None if window is None else int(window)
         self.row = kv_rank + rot_dim                      # one cache row
-        self.latent_norm = StreamRMSNorm(kv_rank, eps=eps, one_plus=False)
+        self.half_split = bool(half_split)
+        self.gate_per_head = bool(gate_per_head)
+        self.owns_kv = bool(owns_kv)
+        self.latent_norm = StreamRMSNorm(kv_rank, eps=eps, one_plus=False) if owns_kv else None
+        # (interleaved and half-split pairs turn at the same frequencies)
         self.register_buffer("inv_freq", interleaved_inv_freq(rope_base, rot_dims),
                              persistent=False)
         # per-head up-projections in checkpoint layout: uk (H, dim, kv_rank),
@@ -72,13 +80,14 @@ class LatentSinkAttention(nn.Module):
 
     def kv_shape(self):
         """One key 'head' of kv_rank + rot_dim channels, no value pages."""
-        return (1, self.row, 0)
+        return (1, self.row, 0) if self.owns_kv else None
 
     @torch.no_grad()           # inference only: the batched products write into views
     def forward(self, q: torch.Tensor, dkv: torch.Tensor, kv_mgr, cache_idx: int,
                 step: seqmix.StepLayout, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
-        """q (B,S,H*(dim+rot_dim)), dkv (B,S,kv_rank+rot_dim), gate
-        (B,S,H*v_dim) or None: column slices of a fused projection are fine.
+        """q (B,S,H*(dim+rot_dim)), dkv (B,S,kv_rank+rot_dim) (None for a
+        borrowing layer), gate (B,S,H*v_dim), (B,S,H) with ``gate_per_head``,
+        or None: column slices of a fused projection are fine.
         Returns (B,S,H*v_dim)."""
         B, S = q.shape[0], q.shape[1]
         H, D, R, C = self.num_heads, self.dim, self.rot_dim, self.kv_rank
@@ -90,24 +99,32 @@ class LatentSinkAttention(nn.Module):
         kc, _ = kv_mgr.get_cache(cache_idx)
         q4 = q.unflatten(-1, (H, D + R))
         fresh = bool(getattr(step, "fresh", False))
-        row = torch.empty(B, S, self.row, dtype=dt, device=q.device) if fresh else None
-        seqmix.latent_row_write(dkv, self.latent_norm.weight, self.latent_norm.eps,
-                                self.inv_freq, step, kc.data, kv_mgr.slot_mapping, C, row=row)
+        if self.owns_kv:
+            row = torch.empty(B, S, self.row, dtype=dt, device=q.device) if fresh else None
+            seqmix.latent_row_write(dkv, self.latent_norm.weight, self.latent_norm.eps,
+                                    self.inv_freq, step, kc.data, kv_mgr.slot_mapping, C, row=row,
+                                    half_split=self.half_split)
+            if fresh and cache_idx in kv_mgr.layer_kv_source:
+                step.latent_rows[cache_idx] = row           # a later layer reads this cache
+        elif fresh:
+            row = step.latent_rows[kv_mgr.layer_kv_source[cache_idx]]
         if fresh:
             return self._expanded(q4, row, step, gate)
         # query in latent space: [uk_h^T q_plain | rotated q_rot] per head
         qa = torch.empty(B, S, H, self.row, dtype=dt, device=q.device)
         torch.bmm(q4[..., :D].flatten(0, 1).transpose(0, 1), self.uk,
                   out=qa.view(T, H, self.row)[..., :C].transpose(0, 1))
-        seqmix.rotate_interleaved(q4[..., D:], step, self.inv_freq, out=qa[..., C:])
+        seqmix.rotate_interleaved(q4[..., D:], step, self.inv_freq, out=qa[..., C:],
+                                  half_split=self.half_split)
         k_cache = kc.data
         lat = seqmix.paged_attention(
             qa.view(B, S, H * self.row), k_cache, k_cache[..., :C], step, kv_mgr.block_table,
-            self.scale, H, window=self.window, sink=self.sink, out_dtype=dt)   # (B,S,H*C)
-        out = torch.empty(B, S, H * self.v_dim, dtype=dt, device=q.device)
-        torch.bmm(lat.view(T, H, C).transpose(0, 1), self.uv.transpose(1, 2),
-                  out=out.view(T, H, self.v_dim).transpose(0, 1))
-        if gate is not None:
+            self.scale, H, window=self.window, sink=self.sink, out_dtype=dt,
+            # a head's gate commutes with its W_uv
+            gate=gate if self.gate_per_head else None,
+            gate_per_head=self.gate_per_head)                                  # (B,S,H*C)
+        out = seqmix.head_product(lat.view(T, H, C), self.uv).view(B, S, H * self.v_dim)
+        if gate is not None and not self.gate_per_head:
             seqmix.sigmoid_gate_(out, gate)
         return out
 
@@ -124,8 +141,10 @@ class LatentSinkAttention(nn.Module):
         kx[..., D:] = row[..., C:].unsqueeze(2)
         vx = torch.nn.functional.linear(c, self.uv.view(H * Dv, C)).view(B, S, H, Dv)
         qx = q4.clone(memory_format=torch.contiguous_format)
-        seqmix.rotate_interleaved(qx[..., D:], step, self.inv_freq, out=qx[..., D:])
+        seqmix.rotate_interleaved(qx[..., D:], step, self.inv_freq, out=qx[..., D:],
+                                  half_split=self.half_split)
         pages = torch.arange(B, device=q4.device, dtype=torch.int32).view(B, 1)
         return seqmix.paged_attention(
             qx.view(B, S, H * (D + R)), kx, vx, step, pages, self.scale, H,
-            window=self.window, sink=self.sink, gate=gate, out_dtype=dt)
+            window=self.window, sink=self.sink, gate=gate, out_dtype=dt,
+            gate_per_head=self.gate_per_head)

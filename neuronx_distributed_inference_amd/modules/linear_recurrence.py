@@ -1,6 +1,7 @@
 """Linear-recurrence token mixer cores with matrix state: the gated delta
-rule (below), selective state spaces (:class:`StateSpaceDuality`) and
-retention (:class:`Retention`).
+rule (below), selective state spaces (:class:`StateSpaceDuality`),
+retention (:class:`Retention`) and gated linear attention
+(:class:`GatedLinearAttention`).
 
 Gated delta rule.
 
@@ -196,4 +197,52 @@ class Retention(nn.Module):
         o = seqmix.decay_scan(q, k, v, states.get(key + ".mem"), step, self.dim, self.vdim,
                               head_decay=self.decay, k_scale=self.dim ** -0.5)
         return seqmix.group_gated_norm(o, gate, None, self.eps, self.num_heads,
+                                       gate_first=False, out_dtype=gate.dtype)
+
+
+class GatedLinearAttention(nn.Module):
+    """Linear attention with a data-dependent decay per key channel: per head a
+    (dim x vdim) fp32 state
+
+        S_t = diag(a_t) S_{t-1} + (dim^-1/2 k_t) v_t^T ,   o_t = S_t^T q_t ,
+        a_t = sigmoid(A2 r_t + bias)^(1/tau)
+
+    with ``r_t`` (``decay_rank`` wide) the first stage of a low-rank decay
+    projection. (The dim^-1/2 belongs to the query; the read-out is linear in
+    both, so it rides on the keys as they enter the state.) Each head's
+    read-out is RMS-normed with one weight shared by the heads and multiplied
+    by silu of a gate projection.
+
+    The caller owns the q/k/v/gate/first-stage and the output projections; the
+    second stage ``A2`` lives here, its bias enters in fp32. The state lives
+    in the cache manager's :class:`RecurrentStateManager`.
+    """
+
+    def __init__(self, num_heads: int, dim: int, vdim: int, tau: float, decay_rank: int,
+                 eps: float, dtype: torch.dtype):
+        super().__init__()
+        self.num_heads = num_heads
+        self.dim = dim
+        self.vdim = vdim
+        self.tau = float(tau)
+        self.eps = float(eps)
+        self.decay_up = ColumnParallelLinear(decay_rank, num_heads * dim, dtype=dtype, tp_degree=1)
+        f32 = dict(dtype=torch.float32)
+        self.decay_bias = nn.Parameter(torch.zeros(num_heads * dim, **f32), requires_grad=False)
+        self.norm_weight = nn.Parameter(torch.ones(vdim, **f32), requires_grad=False)
+
+    def state_shapes(self):
+        return {"mem": (self.num_heads, self.vdim, self.dim)}      # stored transposed
+
+    def forward(self, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torch.Tensor,
+                decay_low: torch.Tensor, states, key: str,
+                step: seqmix.StepLayout) -> torch.Tensor:
+        """q, k (B,S,H*dim), v, gate (B,S,H*vdim), decay_low (B,S,rank): raw
+        projections, column slices of one GEMM output are fine. Returns
+        (B,S,H*vdim) in the gate's dtype."""
+        o = seqmix.decay_scan(q, k, v, states.get(key + ".mem"), step, self.dim, self.vdim,
+                              channel_logits=self.decay_up(decay_low),
+                              channel_bias=self.decay_bias, tau=self.tau,
+                              k_scale=self.dim ** -0.5)
+        return seqmix.group_gated_norm(o, gate, self.norm_weight, self.eps, self.num_heads,
                                        gate_first=False, out_dtype=gate.dtype)

@@ -405,11 +405,13 @@ class GroupLimitedRouter(nn.Module):
     fp32. ``extra_gates`` further rows of the weight are per-token sigmoid
     gates computed by the same fp32 product (a shared expert's gate). With
     ``correction`` a stored per-expert offset is added to the scores for the
-    choice only; the weights stay the uncorrected scores."""
+    choice only; the weights stay the uncorrected scores. With ``bias`` a
+    stored offset is part of the logits. ``normalize`` without groups is a
+    softmax over the chosen logits only."""
 
     def __init__(self, hidden_size: int, num_experts: int, top_k: int, n_groups: int = 1,
                  keep_groups: int = 1, scale: float = 1.0, normalize: bool = False,
-                 extra_gates: int = 0, correction: bool = False):
+                 extra_gates: int = 0, correction: bool = False, bias: bool = False):
         super().__init__()
         assert num_experts % max(n_groups, 1) == 0 and top_k <= num_experts
         self.num_experts = num_experts
@@ -424,6 +426,8 @@ class GroupLimitedRouter(nn.Module):
             torch.empty(num_experts + extra_gates, hidden_size, dtype=torch.float32))
         self.correction = nn.Parameter(torch.zeros(num_experts, dtype=torch.float32),
                                        requires_grad=False) if correction else None
+        self.bias = nn.Parameter(torch.zeros(num_experts + extra_gates, dtype=torch.float32),
+                                 requires_grad=False) if bias else None
 
     def forward(self, x: torch.Tensor):
         """x (T, hidden) -> (dense (T, E + extra) fp32, idx (T, top_k) int32,
@@ -432,12 +436,12 @@ class GroupLimitedRouter(nn.Module):
 
         return seqmix.route_tokens(x, self.weight, self.num_experts, self.top_k, self.n_groups,
                                    self.keep_groups, self.scale, self.normalize,
-                                   correction=self.correction)
+                                   correction=self.correction, bias=self.bias)
 
 
 class FusedUngatedExperts(nn.Module):
-    """Two-matrix experts ``W_down act(W_up x)`` with act = relu squared,
-    stacked so that ALL experts (and an optional always-on shared expert) are
+    """Two-matrix experts ``W_down act(W_up x)`` with act = relu squared or
+    the exact gelu (``act``: relu2 / gelu), stacked so that ALL experts (and an optional always-on shared expert) are
     two GEMMs: ``up`` (E*ff + shared_ff, hidden) and ``down`` (hidden, E*ff +
     shared_ff). The routing weight (zero for an unchosen expert) multiplies
     the activation before the second product, whose fp32 accumulator then
@@ -446,7 +450,7 @@ class FusedUngatedExperts(nn.Module):
     the step has no data-dependent shapes and no host synchronisation."""
 
     def __init__(self, num_experts: int, hidden_size: int, expert_ff: int, shared_ff: int,
-                 dtype: torch.dtype, tp_degree: int = 1):
+                 dtype: torch.dtype, tp_degree: int = 1, act: str = "relu2"):
         super().__init__()
         from neuronx_distributed_inference_amd.parallel.layers import (
             ColumnParallelLinear,
@@ -457,6 +461,7 @@ class FusedUngatedExperts(nn.Module):
         self.num_experts = num_experts
         self.expert_ff = expert_ff
         self.shared_ff = shared_ff
+        self.act = act
         inner = num_experts * expert_ff + shared_ff
         self.up = ColumnParallelLinear(hidden_size, inner, dtype=dtype, tp_degree=1)
         self.down = RowParallelLinear(inner, hidden_size, dtype=dtype, tp_degree=1)
@@ -473,26 +478,31 @@ class FusedUngatedExperts(nn.Module):
 
     def forward(self, x: torch.Tensor, gates: torch.Tensor) -> torch.Tensor:
         """x (T, hidden); gates (T, E [+ 1]) fp32 dense routing weights, the
-        last column the shared expert's gate when there is one."""
+        last column the shared expert's gate when it has one."""
         from neuronx_distributed_inference_amd.ops import seqmix
 
         hid = self.up(x)
-        return self.down(seqmix.relu2_scale(hid, gates, self.expert_ff, self.num_experts,
-                                             out_dtype=hid.dtype))
+        return self.down(seqmix.act_scale(hid, gates, self.expert_ff, self.num_experts,
+                                          act=self.act, out_dtype=hid.dtype))
 
 
 class GroupRoutedFeedForward(nn.Module):
-    """Mixture of relu-squared experts behind a :class:`GroupLimitedRouter`,
-    with an optional shared expert that runs for every token and is scaled by
-    a per-token sigmoid gate (``shared_ff`` = 0: none)."""
+    """Mixture of two-matrix experts (``act``) behind a
+    :class:`GroupLimitedRouter`, with an optional shared expert that runs for
+    every token (``shared_ff`` = 0: none), scaled by a per-token sigmoid gate
+    or, without ``shared_gate``, by one."""
 
     def __init__(self, hidden_size: int, num_experts: int, top_k: int, expert_ff: int,
                  dtype: torch.dtype, n_groups: int = 1, keep_groups: int = 1,
-                 scale: float = 1.0, normalize: bool = False, shared_ff: int = 0):
+                 scale: float = 1.0, normalize: bool = False, shared_ff: int = 0,
+                 shared_gate: bool = True, act: str = "relu2", router_bias: bool = False):
         super().__init__()
         self.router = GroupLimitedRouter(hidden_size, num_experts, top_k, n_groups, keep_groups,
-                                         scale, normalize, extra_gates=1 if shared_ff else 0)
-        self.experts = FusedUngatedExperts(num_experts, hidden_size, expert_ff, shared_ff, dtype)
+                                         scale, normalize,
+                                         extra_gates=1 if shared_ff and shared_gate else 0,
+                                         bias=router_bias)
+        self.experts = FusedUngatedExperts(num_experts, hidden_size, expert_ff, shared_ff, dtype,
+                                           act=act)
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         shape = h.shape

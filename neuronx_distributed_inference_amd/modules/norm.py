@@ -61,6 +61,35 @@ class LayerNorm(nn.Module):
         return xf, new_res
 
 
+class StreamLayerNorm(nn.Module):
+    """LayerNorm with bias for models whose residual stream is fp32. Besides
+    the plain call, :meth:`sum_into` does the residual step of designs that
+    norm after the sum, ``stream = norm(alpha * stream + y)``, in one kernel
+    and hands back the new stream in the next GEMM's input dtype."""
+
+    def __init__(self, hidden_size: int, eps: float = 1e-5,
+                 out_dtype: torch.dtype = torch.float32):
+        super().__init__()
+        self.weight = nn.Parameter(torch.ones(hidden_size, dtype=torch.float32),
+                                   requires_grad=False)
+        self.bias = nn.Parameter(torch.zeros(hidden_size, dtype=torch.float32),
+                                 requires_grad=False)
+        self.eps = float(eps)
+        self.out_dtype = out_dtype
+
+    def forward(self, x: torch.Tensor, residual: torch.Tensor = None):
+        from neuronx_distributed_inference_amd.ops import seqmix
+
+        assert residual is None
+        return seqmix.layer_norm(x, self.weight, self.eps, self.out_dtype, bias=self.bias)
+
+    def sum_into(self, stream: torch.Tensor, y: torch.Tensor, alpha: float, copy_dtype=None):
+        from neuronx_distributed_inference_amd.ops import seqmix
+
+        return seqmix.add_layer_norm(stream, y, alpha, self.weight, self.bias, self.eps,
+                                     copy_dtype)
+
+
 class StreamRMSNorm(nn.Module):
     """RMS norm for models whose residual stream is fp32: statistics and the
     weight product in fp32, output in the dtype the consumer asks for.

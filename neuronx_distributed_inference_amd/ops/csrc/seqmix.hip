@@ -1,5 +1,5 @@
-// Sequence-mixing kernels for hybrid models (gfx950): bias-free LayerNorm and
-// RMS norms on an fp32 residual stream (with the post-norm residual step fused),
+// Sequence-mixing kernels for hybrid models (gfx950): LayerNorm and RMS norms on
+// an fp32 residual stream (with the post-norm residual step fused),
 // short causal convolutions with a carried tail, paged KV scatter with distinct
 // K/V head sizes, interleaved rotary positions, paged softmax attention with
 // optional sliding window / always-visible first tokens / log-distance penalty /
@@ -86,7 +86,8 @@ DEV float block_sum(float v, float* red) {
 template <typename TOut>
 __global__ void __launch_bounds__(LN_THREADS)
 layer_norm_kernel(const float* __restrict__ x, const float* __restrict__ w,
-                  TOut* __restrict__ out, long rows, int C, float eps) {
+                  const float* __restrict__ bias, TOut* __restrict__ out, long rows, int C,
+                  float eps) {
     __shared__ float red[LN_THREADS / WAVE];
     const long row = blockIdx.x;
     const float* xr = x + row * C;
@@ -97,7 +98,8 @@ layer_norm_kernel(const float* __restrict__ x, const float* __restrict__ w,
     for (int c = threadIdx.x; c < C; c += LN_THREADS) { float d = xr[c] - mean; v += d * d; }
     const float inv = 1.f / sqrtf(block_sum(v, red) / C + eps);
     TOut* o = out + row * C;
-    for (int c = threadIdx.x; c < C; c += LN_THREADS) stf<TOut>(o + c, (xr[c] - mean) * inv * w[c]);
+    for (int c = threadIdx.x; c < C; c += LN_THREADS)
+        stf<TOut>(o + c, (xr[c] - mean) * inv * w[c] + (bias ? bias[c] : 0.f));
 }
 
 // ------------------------------------------------------------- short conv
@@ -285,13 +287,14 @@ __global__ void paged_kv_write_kernel(T* __restrict__ kc, T* __restrict__ vc,
 
 // --------------------------------------------- latent cache row, one launch
 // A latent layer's cache row of a token: [rms_norm(x[:C]) * w | x[C:C+R] with its
-// first 2*half channels turned in interleaved pairs by pos * inv_freq[i]], written
-// straight into the token's page slot (and, when `row` is given, into a dense row
+// first 2*half channels turned in interleaved (split = 0: 2i, 2i+1) or half-split
+// (split = 1: i, i+half) pairs by pos * inv_freq[i]], written straight into the token's page slot (and, when `row` is given, into a dense row
 // buffer as well). One wave per token; statistics and angles in fp32. Pad tokens
 // (slot or position < 0) write nothing to the cache.
 template <typename T>
 __global__ void latent_row_kernel(const T* __restrict__ x, long xs, const float* __restrict__ w,
                                   float eps, const float* __restrict__ inv_freq, int half,
+                                  int split,
                                   const int* __restrict__ pos, const int* __restrict__ slots,
                                   T* __restrict__ cache, long nslots, T* __restrict__ row, long rs,
                                   long ntok, int C, int R) {
@@ -313,12 +316,13 @@ __global__ void latent_row_kernel(const T* __restrict__ x, long xs, const float*
     }
     for (int e = lane; e < half + (R - 2 * half); e += WAVE) {
         if (e < half) {
-            const float a = ldf<T>(xr + C + 2 * e), b = ldf<T>(xr + C + 2 * e + 1);
+            const int c0 = C + (split ? e : 2 * e), c1 = C + (split ? e + half : 2 * e + 1);
+            const float a = ldf<T>(xr + c0), b = ldf<T>(xr + c1);
             float sn, cs;
             sincosf((float)(p < 0 ? 0 : p) * inv_freq[e], &sn, &cs);
             const float u = a * cs - b * sn, v = b * cs + a * sn;
-            if (cp) { stf<T>(cp + C + 2 * e, u); stf<T>(cp + C + 2 * e + 1, v); }
-            if (rp) { stf<T>(rp + C + 2 * e, u); stf<T>(rp + C + 2 * e + 1, v); }
+            if (cp) { stf<T>(cp + c0, u); stf<T>(cp + c1, v); }
+            if (rp) { stf<T>(rp + c0, u); stf<T>(rp + c1, v); }
         } else {
             const int c = C + 2 * half + (e - half);
             const float v = ldf<T>(xr + c);
@@ -995,7 +999,8 @@ paged_attn_mfma_kernel(const bf16* __restrict__ q, long qstride, const bf16* __r
 // channels [128w, 128w+128), so a workgroup covers 512 of them and the key row
 // is fetched from memory once: global -> registers (next tile prefetched) -> LDS
 // row-major, then V^T is cut out of that LDS tile. Causal, optionally inside a
-// sliding window or the token's block of positions; optional sink.
+// sliding window or the token's block of positions; optional sink and sigmoid gate
+// per head.
 // Grid: (tokens x key splits, head chunks of 16 x value splits of 512, batch
 // rows). With nks > 1 key splits a workgroup scans every nks-th run of tiles and
 // leaves an unnormalised partial (fp32 values, running max, sum) in `ws`;
@@ -1010,7 +1015,8 @@ latent_decode_mfma_kernel(const bf16* __restrict__ q, long qstride, const bf16* 
                           const int* __restrict__ btab, int max_blocks,
                           const float* __restrict__ sink, bf16* __restrict__ out, int H, int Dk,
                           int Dv, int bsz, int S, float scale, int nsplit, int nks,
-                          float* __restrict__ ws, int window, int cmask) {
+                          float* __restrict__ ws, int window, int cmask,
+                          const bf16* __restrict__ gate, long gstride) {
     constexpr int KS = DKP + 8;
     constexpr int VS = LD_KT + 8;
     constexpr int VCH = 4 * LD_VW;
@@ -1179,6 +1185,8 @@ latent_decode_mfma_kernel(const bf16* __restrict__ q, long qstride, const bf16* 
         const float ca = m_run > -INFINITY ? __expf(m_run - mf) : 0.f;
         fin = ca / (l_run * ca + __expf(sk - mf));
     }
+    // one gate number per head
+    if (gate && hv) fin *= sigmoidf_(__bfloat162float(gate[((long)b * S + t) * gstride + h]));
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
         const int hh = h0 + lg * 4 + r;
@@ -1199,7 +1207,7 @@ __global__ void latent_decode_merge_kernel(const float* __restrict__ ws,
                                            const float* __restrict__ sink,
                                            const int* __restrict__ pos, const int* __restrict__ seq,
                                            bf16* __restrict__ out, long ntok, int S, int H, int Dv,
-                                           int nks) {
+                                           int nks, const bf16* __restrict__ gate, long gstride) {
     const int lane = threadIdx.x & (WAVE - 1);
     const long wid = (long)blockIdx.x * (blockDim.x / WAVE) + threadIdx.x / WAVE;
     if (wid >= ntok * H) return;
@@ -1215,7 +1223,8 @@ __global__ void latent_decode_merge_kernel(const float* __restrict__ ws,
         const float mi = wp[i * (long)(Dv + 2) + Dv];
         if (mi > -INFINITY) L += wp[i * (long)(Dv + 2) + Dv + 1] * expf(mi - M);
     }
-    const float inv = L > 0.f ? 1.f / L : 0.f;
+    float inv = L > 0.f ? 1.f / L : 0.f;
+    if (gate) inv *= sigmoidf_(__bfloat162float(gate[tok * gstride + h]));
     float wgt[8];                                        // nks <= 8
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
@@ -1493,7 +1502,13 @@ __global__ void residual_add_kernel(float* __restrict__ x, const T* __restrict__
 }
 
 // out[r, c] = gelu_tanh(gu[r, c]) * gu[r, I + c]
-template <typename T>
+// gated units: act(gate) * up, act = the tanh form of gelu (0) or silu (1)
+DEV float gelu_tanh_(float z) {
+    return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
+template <int ACT> DEV float unit_act_(float z) { return ACT == 0 ? gelu_tanh_(z) : z * sigmoidf_(z); }
+
+template <typename T, int ACT>
 __global__ void gelu_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, long rows, int I) {
     const long total = rows * I;
     for (long idx = (long)blockIdx.x * blockDim.x + threadIdx.x; idx < total;
@@ -1502,13 +1517,12 @@ __global__ void gelu_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, l
         const int c = idx % I;
         const float z = ldf<T>(gu + r * 2 * I + c);
         const float u = ldf<T>(gu + r * 2 * I + I + c);
-        const float ge = 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-        stf<T>(out + idx, ge * u);
+        stf<T>(out + idx, unit_act_<ACT>(z) * u);
     }
 }
 
 // 8 channels per thread, 16-byte accesses; rows on blockIdx.y (strided)
-template <typename T>
+template <typename T, int ACT>
 __global__ void gelu_mul_vec_kernel(const T* __restrict__ gu, T* __restrict__ out, long rows,
                                     int I) {
     const int c = (blockIdx.x * blockDim.x + threadIdx.x) * 8;
@@ -1518,9 +1532,7 @@ __global__ void gelu_mul_vec_kernel(const T* __restrict__ gu, T* __restrict__ ou
         load8<T>(gu + r * 2 * I + c, z);
         load8<T>(gu + r * 2 * I + I + c, u);
 #pragma unroll
-        for (int e = 0; e < 8; ++e)
-            o[e] = 0.5f * z[e] * (1.f + tanhf(0.7978845608028654f *
-                                              (z[e] + 0.044715f * z[e] * z[e] * z[e]))) * u[e];
+        for (int e = 0; e < 8; ++e) o[e] = unit_act_<ACT>(z[e]) * u[e];
         T* op = out + r * I + c;
         if constexpr (sizeof(T) == 2) {
             uint32_t pk[4];
@@ -1700,15 +1712,90 @@ add_rms_norm_kernel(float* __restrict__ stream, const TY* __restrict__ y,
         stf<TC>(copy + row * C + c, xr[c] * inv2 * next_w[c]);
 }
 
+// ----------------------------------------- residual step with the norm after the sum
+// stream[row] = layer_norm(alpha * stream[row] + y[row]) * w + bias, fp32; `copy`
+// (optional) receives the new row in the next GEMM's input type. One workgroup per
+// row. The vector form keeps the row in registers between mean, variance (of the
+// deviations) and output: one read of each operand, one write of each result.
+template <typename TY, typename TC, int NV>
+__global__ void __launch_bounds__(LN_THREADS)
+add_layer_norm_vec_kernel(float* __restrict__ stream, const TY* __restrict__ y, float alpha,
+                          const float* __restrict__ w, const float* __restrict__ bias, float eps,
+                          TC* __restrict__ copy, int C) {
+    __shared__ float red[LN_THREADS / WAVE];
+    const long row = blockIdx.x;
+    float* xr = stream + row * C;
+    float v[NV][8];
+    float s = 0.f;
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+        const int c = (j * LN_THREADS + threadIdx.x) * 8;
+        if (c < C) {
+            float yv[8];
+            load8<float>(xr + c, v[j]);
+            load8<TY>(y + row * C + c, yv);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) { v[j][e] = alpha * v[j][e] + yv[e]; s += v[j][e]; }
+        }
+    }
+    const float mean = block_sum(s, red) / C;
+    float q = 0.f;
+#pragma unroll
+    for (int j = 0; j < NV; ++j)
+        if ((j * LN_THREADS + threadIdx.x) * 8 < C)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) { v[j][e] -= mean; q += v[j][e] * v[j][e]; }
+    const float inv = 1.f / sqrtf(block_sum(q, red) / C + eps);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+        const int c = (j * LN_THREADS + threadIdx.x) * 8;
+        if (c >= C) continue;
+        float wv[8], bv[8];
+        load8<float>(w + c, wv);
+        load8<float>(bias + c, bv);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[j][e] = v[j][e] * inv * wv[e] + bv[e];
+        store8<float>(xr + c, v[j]);
+        if (copy) store8<TC>(copy + row * C + c, v[j]);
+    }
+}
+
+// scalar form: any width and alignment (the sum is parked in the stream row)
+template <typename TY, typename TC>
+__global__ void __launch_bounds__(LN_THREADS)
+add_layer_norm_kernel(float* __restrict__ stream, const TY* __restrict__ y, float alpha,
+                      const float* __restrict__ w, const float* __restrict__ bias, float eps,
+                      TC* __restrict__ copy, int C) {
+    __shared__ float red[LN_THREADS / WAVE];
+    const long row = blockIdx.x;
+    float* xr = stream + row * C;
+    float s = 0.f;
+    for (int c = threadIdx.x; c < C; c += LN_THREADS) {
+        const float v = alpha * xr[c] + ldf<TY>(y + row * C + c);
+        xr[c] = v;                                       // re-read by this thread only
+        s += v;
+    }
+    const float mean = block_sum(s, red) / C;
+    float q = 0.f;
+    for (int c = threadIdx.x; c < C; c += LN_THREADS) { const float d = xr[c] - mean; q += d * d; }
+    const float inv = 1.f / sqrtf(block_sum(q, red) / C + eps);
+    for (int c = threadIdx.x; c < C; c += LN_THREADS) {
+        const float v = (xr[c] - mean) * inv * w[c] + bias[c];
+        xr[c] = v;
+        if (copy) stf<TC>(copy + row * C + c, v);
+    }
+}
+
 // ---------------------------------------------------------- rotary positions
-// pairs (2i, 2i+1) of the first 2*half channels of every head turn by
-// p * inv_freq[i] (fp32 angle, full-range sincosf); the rest is copied.
+// pairs (2i, 2i+1) of the first 2*half channels of every head (split = 0), or
+// pairs (i, i + half) (split = 1), turn by p * inv_freq[i] (fp32 angle, full-range
+// sincosf); the rest is copied.
 // One thread per (token, head, channel pair or trailing channel).
 template <typename TIn, typename TOut>
 __global__ void rope_pairs_kernel(const TIn* __restrict__ x, long xt, long xh,
                                   TOut* __restrict__ out, long ot, long oh,
                                   const int* __restrict__ pos, const float* __restrict__ inv_freq,
-                                  int half, long ntok, int N, int C) {
+                                  int half, int split, long ntok, int N, int C) {
     const int per = half + (C - 2 * half);            // work items per head
     const long total = ntok * N * per;
     for (long idx = (long)blockIdx.x * blockDim.x + threadIdx.x; idx < total;
@@ -1721,11 +1808,12 @@ __global__ void rope_pairs_kernel(const TIn* __restrict__ x, long xt, long xh,
         const TIn* xp = x + tok * xt + (long)h * xh;
         TOut* op = out + tok * ot + (long)h * oh;
         if (e < half) {
-            float a = ldf<TIn>(xp + 2 * e), b = ldf<TIn>(xp + 2 * e + 1);
+            const int c0 = split ? e : 2 * e, c1 = split ? e + half : 2 * e + 1;
+            float a = ldf<TIn>(xp + c0), b = ldf<TIn>(xp + c1);
             float sn, cs;
             sincosf((float)(p < 0 ? 0 : p) * inv_freq[e], &sn, &cs);
-            stf<TOut>(op + 2 * e, a * cs - b * sn);
-            stf<TOut>(op + 2 * e + 1, b * cs + a * sn);
+            stf<TOut>(op + c0, a * cs - b * sn);
+            stf<TOut>(op + c1, b * cs + a * sn);
         } else {
             const int c = 2 * half + (e - half);
             stf<TOut>(op + c, ldf<TIn>(xp + c));
@@ -1832,20 +1920,25 @@ head_norm_rope_kernel(const TIn* __restrict__ x, long xt, long xh, TOut* __restr
     for (int c = 2 * half + lane; c < C; c += WAVE) stf<TOut>(op + c, row[c]);
 }
 
-// ----------------------------------------------- scalar-decay linear recurrence
+// ----------------------------------------------------- decayed linear recurrence
 // S_t = a_t S_{t-1} + k_t (w_t v_t)^T, o_t = S_t^T q_t (+ skip_h v_t), one scalar
-// decay per head and token. Workgroup = (row, head, 16 value channels); the 16
+// decay per head and token, or (CH) one per key channel: S_t = diag(a_t) S_{t-1} +
+// k_t v_t^T. Workgroup = (row, head, 16 value channels); the 16
 // lanes of a channel split its key rows (lane p owns rows p*R .. p*R+R-1), the
 // state sits in registers for the whole step and is read/written once. Tokens
 // are staged through LDS in chunks of DS_TC (q, k, v, decay, step size), so
 // global loads are coalesced and the serial loop reads only LDS.
 // Decay: selective (dt projection + dt_bias, a_log: w = softplus(dt + bias),
-// a = exp(-exp(a_log) w)) or fixed per head (head_decay: a = decay, w = 1).
+// a = exp(-exp(a_log) w)) or fixed per head (head_decay: a = decay, w = 1). CH takes
+// `dt` (H*D wide) as decay logits, a = sigmoid(dt + dt_bias)^inv_tau (steps of few
+// tokens), or, with dt_bias = null, as the decays themselves, computed once per
+// token by channel_decay_kernel instead of once per value-channel block.
 //
 // Long rows with few workgroups are cut into `nseg` segments of `seglen`
 // tokens that run side by side; the recurrence is linear in the state, so
 //   MODE 1: every segment scans from a ZERO state and leaves its end state E_c
-//           and the product P_c of its decays in the workspace (no outputs);
+//           and the product P_c of its decays (a scalar, or one per key channel) in
+//           the workspace (no outputs);
 //   decay_scan_link_kernel: start state of segment c, serially over the few
 //           segments: S_c = P_{c-1} S_{c-1} + E_{c-1} (S_0 = the carried state);
 //   MODE 2: every segment scans again from its true start state and writes
@@ -1853,7 +1946,25 @@ head_norm_rope_kernel(const TIn* __restrict__ x, long xt, long xh, TOut* __restr
 // MODE 0 is the plain single pass (decode steps, short portions, full batches).
 #define DS_TC 16
 
-template <typename T, typename TD, int R, int MODE>
+// sigmoid(z)^inv_tau, through the logarithm: no underflow for very negative z
+DEV float channel_decay_(float z, float inv_tau) {
+    return expf((fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau);
+}
+
+template <typename T>
+__global__ void channel_decay_kernel(const T* __restrict__ z, long zs,
+                                     const float* __restrict__ bias, float inv_tau,
+                                     float* __restrict__ out, long rows, int C) {
+    const long total = rows * C;
+    for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < total;
+         i += (long)gridDim.x * blockDim.x) {
+        const long t = i / C;
+        const int c = i % C;
+        out[i] = channel_decay_(ldf<T>(z + t * zs + c) + bias[c], inv_tau);
+    }
+}
+
+template <typename T, typename TD, int R, int MODE, bool CH>
 __global__ void __launch_bounds__(256)
 decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, long ks,
                   const T* __restrict__ v, long vs, const TD* __restrict__ dt, long dts,
@@ -1863,8 +1974,9 @@ decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, lon
                   const int* __restrict__ pos, const int* __restrict__ seq,
                   const int* __restrict__ nvalid, float* __restrict__ out, int S, int H, int G,
                   int D, int Dv, float* __restrict__ ws, float* __restrict__ wdec, int nseg,
-                  int seglen) {
+                  int seglen, float inv_tau) {
     constexpr int DP = 16 * R;
+    __shared__ __attribute__((aligned(16))) float sd[CH ? DS_TC : 1][CH ? DP : 4];
     __shared__ __attribute__((aligned(16))) float sq[MODE == 1 ? 1 : DS_TC][DP], sk[DS_TC][DP];
     __shared__ float sv[DS_TC][16], sa[DS_TC], sw[DS_TC];
     const int b = blockIdx.z, h = blockIdx.y;
@@ -1905,7 +2017,9 @@ decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, lon
         }
     }
     const float skp = skip ? skip[h] : 0.f;
-    float aprod = 1.f;
+    float aprod[CH ? R : 1];
+#pragma unroll
+    for (int r = 0; r < (CH ? R : 1); ++r) aprod[r] = 1.f;
     for (int t0 = tbeg; t0 < tend; t0 += DS_TC) {
         const int cnt = min(DS_TC, tend - t0);
         __syncthreads();                                  // the previous chunk is consumed
@@ -1919,6 +2033,14 @@ decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, lon
             }
             if (MODE != 1) sq[tt][d] = qv;
             sk[tt][d] = kv;
+            if constexpr (CH) {
+                float a = 0.f;
+                if (tt < cnt && d < D) {
+                    a = ldf<TD>(dt + ((long)b * S + t0 + tt) * dts + (long)h * D + d);
+                    if (dt_bias) a = channel_decay_(a + dt_bias[(long)h * D + d], inv_tau);
+                }
+                sd[tt][d] = a;
+            }
         }
         {
             const int tt = tid >> 4, cc = tid & 15;       // 256 = DS_TC * 16
@@ -1927,7 +2049,7 @@ decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, lon
                 vv = ldf<T>(v + ((long)b * S + t0 + tt) * vs + (long)h * Dv + c0 + cc);
             sv[tt][cc] = vv;
         }
-        if (tid < cnt) {
+        if (!CH && tid < cnt) {
             float a, w = 1.f;
             if (dt) {
                 w = softplusf_(ldf<TD>(dt + ((long)b * S + t0 + tid) * dts + h) + dt_bias[h]);
@@ -1940,8 +2062,23 @@ decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, lon
         }
         __syncthreads();
         for (int tt = 0; tt < cnt; ++tt) {
-            const float a = sa[tt], xv = sv[tt][cl];
-            const float wv = sw[tt] * xv;
+            const float xv = sv[tt][cl];
+            const float wv = CH ? xv : sw[tt] * xv;
+            float ar[R];                                  // this lane's decays
+            if constexpr (!CH) {
+                const float a = sa[tt];
+#pragma unroll
+                for (int r = 0; r < R; ++r) ar[r] = a;
+            } else if constexpr (R % 4 == 0) {
+#pragma unroll
+                for (int r = 0; r < R; r += 4) {
+                    const float4 a4 = *reinterpret_cast<const float4*>(&sd[tt][part * R + r]);
+                    ar[r] = a4.x; ar[r + 1] = a4.y; ar[r + 2] = a4.z; ar[r + 3] = a4.w;
+                }
+            } else {
+#pragma unroll
+                for (int r = 0; r < R; ++r) ar[r] = sd[tt][part * R + r];
+            }
             // a lane's key rows are contiguous: 16-byte LDS reads
             float kr[R], qr[R];
             if constexpr (R % 4 == 0) {
@@ -1962,14 +2099,15 @@ decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, lon
                 }
             }
             if (MODE == 1) {
-                aprod *= a;
 #pragma unroll
-                for (int r = 0; r < R; ++r) st[r] = a * st[r] + kr[r] * wv;
+                for (int r = 0; r < (CH ? R : 1); ++r) aprod[r] *= ar[r];
+#pragma unroll
+                for (int r = 0; r < R; ++r) st[r] = ar[r] * st[r] + kr[r] * wv;
             } else {
                 float acc = 0.f;
 #pragma unroll
                 for (int r = 0; r < R; ++r) {
-                    st[r] = a * st[r] + kr[r] * wv;
+                    st[r] = ar[r] * st[r] + kr[r] * wv;
                     acc += st[r] * qr[r];
                 }
                 acc += __shfl_xor(acc, 8, WAVE);
@@ -1981,7 +2119,18 @@ decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, lon
             }
         }
     }
-    if (MODE == 1 && c0 == 0 && tid == 0) wdec[((long)b * nseg + sgi) * H + h] = aprod;
+    if (MODE == 1 && c0 == 0) {
+        const long wi = ((long)b * nseg + sgi) * H + h;
+        if constexpr (CH) {
+            if (cl == 0) {
+#pragma unroll
+                for (int r = 0; r < R; ++r)
+                    if (part * R + r < D) wdec[wi * D + part * R + r] = aprod[r];
+            }
+        } else if (tid == 0) {
+            wdec[wi] = aprod[0];
+        }
+    }
     float* dst = MODE == 1 ? wp : ((MODE == 0 || sgi == nseg - 1) ? sp : nullptr);
     if (cok && dst) {
         if (v4) {
@@ -2008,7 +2157,8 @@ __global__ void decay_scan_link_kernel(float* __restrict__ ws, const float* __re
                                        const float* __restrict__ state,
                                        const int* __restrict__ pos, const int* __restrict__ seq,
                                        const int* __restrict__ nvalid, int B, int S, int H,
-                                       long per_head, int nseg) {
+                                       long per_head, int nseg, int dch) {
+    // dch: decay channels (1: a scalar per head, else the key dimension)
     const long total = (long)B * H * per_head;
     for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < total;
          i += (long)gridDim.x * blockDim.x) {
@@ -2022,19 +2172,20 @@ __global__ void decay_scan_link_kernel(float* __restrict__ ws, const float* __re
             float* p = ws + (((long)b * nseg + c) * H + h) * per_head + e;
             const float end = *p;
             *p = s;
-            s = wdec[((long)b * nseg + c) * H + h] * s + end;
+            s = wdec[(((long)b * nseg + c) * H + h) * dch + (dch > 1 ? e % dch : 0)] * s + end;
         }
     }
 }
 
 // ------------------------------------------------ grouped RMS norm with silu gate
 // One wave per (row, group of C/groups channels): y (fp32) is multiplied by
-// silu(gate) before the norm (gate_first) or after it; optional weight.
+// silu(gate) before the norm (gate_first) or after it; optional weight (C, or, wshared,
+// C / groups for every group).
 template <typename TG, typename TOut>
 __global__ void group_gated_norm_kernel(const float* __restrict__ y, const TG* __restrict__ gate,
                                         long gs, const float* __restrict__ w, float eps,
-                                        int groups, int gate_first, TOut* __restrict__ out,
-                                        long rows, int C) {
+                                        int groups, int gate_first, int wshared,
+                                        TOut* __restrict__ out, long rows, int C) {
     const int lane = threadIdx.x & (WAVE - 1);
     const long id = (long)blockIdx.x * (blockDim.x / WAVE) + threadIdx.x / WAVE;
     if (id >= rows * groups) return;
@@ -2042,7 +2193,7 @@ __global__ void group_gated_norm_kernel(const float* __restrict__ y, const TG* _
     const int gi = id % groups, Cg = C / groups;
     const float* yp = y + row * C + (long)gi * Cg;
     const TG* gp = gate + row * gs + (long)gi * Cg;
-    const float* wp = w ? w + (long)gi * Cg : nullptr;
+    const float* wp = w ? w + (wshared ? 0 : (long)gi * Cg) : nullptr;
     TOut* op = out + row * C + (long)gi * Cg;
     float ss = 0.f;
     for (int c = lane; c < Cg; c += WAVE) {
@@ -2184,8 +2335,8 @@ template <typename T>
 __global__ void __launch_bounds__(RT_WAVES * WAVE)
 router_fused_kernel(const T* __restrict__ x, long xs, const float* __restrict__ w, int W, int vec,
                     int E, int extra, int top, int ngroups, int keep, float scale, int normalize,
-                    const float* __restrict__ corr, float* __restrict__ dense,
-                    int* __restrict__ idx, float* __restrict__ wts) {
+                    const float* __restrict__ corr, const float* __restrict__ bias,
+                    float* __restrict__ dense, int* __restrict__ idx, float* __restrict__ wts) {
     extern __shared__ float rsm[];                // E + extra logits, then the selection scratch
     __shared__ float part[RT_WAVES][8];
     const int tid = threadIdx.x, lane = tid & (WAVE - 1), wv = tid / WAVE;
@@ -2224,7 +2375,7 @@ router_fused_kernel(const T* __restrict__ x, long xs, const float* __restrict__ 
         }
         __syncthreads();
         if (tid < 8 && e0 + tid < rows) {
-            float v = 0.f;
+            float v = bias ? bias[e0 + tid] : 0.f;
 #pragma unroll
             for (int q = 0; q < RT_WAVES; ++q) v += part[q][tid];
             rsm[e0 + tid] = v;
@@ -2236,38 +2387,52 @@ router_fused_kernel(const T* __restrict__ x, long xs, const float* __restrict__ 
                   dense + t * (long)(E + extra), idx + t * top, wts + t * top, lane);
 }
 
-// -------------------------------------------------- relu^2 times routing weight
-// out[t, c] = relu(x[t, c])^2 * gates[t, min(c / ff, E)] (gates = null: times one)
-template <typename T>
-__global__ void relu2_scale_kernel(const T* __restrict__ x, const float* __restrict__ gates,
-                                   int gcols, int ff, int E, T* __restrict__ out, long rows,
-                                   int C) {
+// ------------------------------------------- activation times routing weight
+// out[t, c] = act(x[t, c]) * gates[t, e], e = c / ff for an expert's columns (c <
+// E*ff); the rest (a shared expert) takes gate column E, or one when there is no
+// such column (gcols = E). gates = null: times one. act = relu^2 (0) or the exact
+// gelu (1).
+template <int ACT> DEV float expert_act_(float v) {
+    if (ACT == 0) { const float r = fmaxf(v, 0.f); return r * r; }
+    return 0.5f * v * (1.f + erff(v * 0.7071067811865476f));
+}
+DEV float expert_gate_(const float* __restrict__ gates, long t, int gcols, int c, int ff, int E) {
+    const int e = min(c / ff, E);
+    return (gates && e < gcols) ? gates[t * gcols + e] : 1.f;
+}
+
+template <typename T, int ACT>
+__global__ void act_scale_kernel(const T* __restrict__ x, const float* __restrict__ gates,
+                                 int gcols, int ff, int E, T* __restrict__ out, long rows, int C) {
     const long total = rows * C;
     for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < total;
          i += (long)gridDim.x * blockDim.x) {
         const long t = i / C;
-        const int c = i % C;
-        const int e = min(c / ff, E);
-        const float v = fmaxf(ldf<T>(x + i), 0.f);
-        stf<T>(out + i, v * v * (gates ? gates[t * gcols + e] : 1.f));
+        stf<T>(out + i, expert_act_<ACT>(ldf<T>(x + i)) *
+                            expert_gate_(gates, t, gcols, i % C, ff, E));
     }
 }
 
-template <typename T>
-__global__ void relu2_scale_vec_kernel(const T* __restrict__ x, const float* __restrict__ gates,
-                                       int gcols, int ff, int E, T* __restrict__ out, long rows,
-                                       int C) {
+template <typename T, int ACT>
+__global__ void act_scale_vec_kernel(const T* __restrict__ x, const float* __restrict__ gates,
+                                     int gcols, int ff, int E, T* __restrict__ out, long rows,
+                                     int C) {
     const int C8 = C / 8;
     const long total = rows * C8;
     for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < total;
          i += (long)gridDim.x * blockDim.x) {
         const long t = i / C8;
         const int c = (i % C8) * 8;
-        const float gw = gates ? gates[t * gcols + min(c / ff, E)] : 1.f;
+        const float gw = expert_gate_(gates, t, gcols, c, ff, E);
         float v[8];
-        load8<T>(x + t * C + c, v);
+        if (gw == 0.f) {                                  // an expert the token did not choose
 #pragma unroll
-        for (int e = 0; e < 8; ++e) { const float r = fmaxf(v[e], 0.f); v[e] = r * r * gw; }
+            for (int e = 0; e < 8; ++e) v[e] = 0.f;
+        } else {
+            load8<T>(x + t * C + c, v);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) v[e] = expert_act_<ACT>(v[e]) * gw;
+        }
         store8<T>(out + t * C + c, v);
     }
 }
@@ -2435,6 +2600,71 @@ __global__ void embed_pos_kernel(const T* __restrict__ emb, const T* __restrict_
     }
 }
 
+// ------------------------------------------------ token + bigram embedding rows
+// stream[t, :] = emb[tok] + table[row], row = (prev * mul_prev + tok * mul_cur) mod
+// buckets, or `buckets` (the last row) at position 0. `prev` is the token before it in
+// the row; for a row's first column it is carried per state slot in `last`, which the
+// workgroup of that column (its only reader) then sets to the row's last real token.
+// One workgroup per token; pad tokens give zero rows.
+template <typename T>
+__global__ void __launch_bounds__(256)
+bigram_embed_kernel(const long long* __restrict__ ids, const int* __restrict__ pos,
+                    const int* __restrict__ seq, const int* __restrict__ nvalid,
+                    const T* __restrict__ emb, const T* __restrict__ table,
+                    int* __restrict__ last, long long mul_prev, long long mul_cur,
+                    long long buckets, int vocab, float* __restrict__ out, int S, int C, int vec) {
+    const long tok = blockIdx.x;
+    const int b = tok / S, t = tok % S, slot = seq[b], p = pos[tok];
+    float* op = out + tok * C;
+    if (p < 0 || slot < 0) {                              // uniform
+        for (int c = threadIdx.x; c < C; c += 256) op[c] = 0.f;
+        return;
+    }
+    const long long cur = min(max(ids[tok], 0ll), (long long)vocab - 1);
+    long long row = buckets;
+    if (p > 0) {
+        const long long prev = t > 0 ? ids[tok - 1] : (long long)last[slot];
+        row = (prev * mul_prev + cur * mul_cur) % buckets;
+        if (row < 0) row += buckets;
+    }
+    if (t == 0) {
+        __syncthreads();                                  // `last` has been read
+        if (threadIdx.x == 0) last[slot] = (int)ids[tok + nvalid[b] - 1];
+    }
+    const T* ep = emb + cur * C;
+    const T* tp = table + row * C;
+    if (vec) {
+        for (int c = threadIdx.x * 8; c < C; c += 256 * 8) {
+            float a[8], g[8];
+            load8<T>(ep + c, a);
+            load8<T>(tp + c, g);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) a[e] += g[e];
+            st8<float>(op + c, a);
+        }
+    } else {
+        for (int c = threadIdx.x; c < C; c += 256) op[c] = ldf<T>(ep + c) + ldf<T>(tp + c);
+    }
+}
+
+// -------------------------------------------------- per-layer token input, gated
+// out[t, c] = gelu_tanh(z[t, c]) * table[tok, off + c]: a layer's slice of the token's
+// row in a (vocab, layers * C) table, gated by a projection of the stream
+template <typename T>
+__global__ void token_gate_kernel(const T* __restrict__ z, long zs,
+                                  const long long* __restrict__ ids, const T* __restrict__ table,
+                                  long ts, int off, int vocab, T* __restrict__ out, long rows,
+                                  int C) {
+    const long total = rows * C;
+    for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < total;
+         i += (long)gridDim.x * blockDim.x) {
+        const long t = i / C;
+        const int c = i % C;
+        const long long tok = min(max(ids[t], 0ll), (long long)vocab - 1);
+        stf<T>(out + i, gelu_tanh_(ldf<T>(z + t * zs + c)) * ldf<T>(table + tok * ts + off + c));
+    }
+}
+
 // ------------------------------------- residual sum of weighted, optionally normed terms
 // x[row] += sum_i f_i(y_i[row]) * w_i, f_i = RMS norm over the row or identity.
 // One workgroup per row; statistics fp32.
@@ -2478,12 +2708,39 @@ static inline int grid_for(long total, int block, int cap = 8192) {
 
 extern "C" {
 
-int nx_layer_norm(const float* x, const float* w, void* out, int out_bf16, long rows, int C,
-                  float eps, hipStream_t st) {
+int nx_layer_norm(const float* x, const float* w, const float* bias, void* out, int out_bf16,
+                  long rows, int C, float eps, hipStream_t st) {
     if (rows <= 0) return 0;
     dim3 grid((unsigned)rows), block(LN_THREADS);
-    if (out_bf16) layer_norm_kernel<bf16><<<grid, block, 0, st>>>(x, w, (bf16*)out, rows, C, eps);
-    else layer_norm_kernel<float><<<grid, block, 0, st>>>(x, w, (float*)out, rows, C, eps);
+    if (out_bf16)
+        layer_norm_kernel<bf16><<<grid, block, 0, st>>>(x, w, bias, (bf16*)out, rows, C, eps);
+    else layer_norm_kernel<float><<<grid, block, 0, st>>>(x, w, bias, (float*)out, rows, C, eps);
+    return (int)hipGetLastError();
+}
+
+int nx_add_layer_norm(float* stream, const void* y, int y_bf16, float alpha, const float* w,
+                      const float* bias, float eps, void* copy, int copy_bf16, long rows, int C,
+                      hipStream_t st) {
+    if (rows <= 0) return 0;
+    if (C <= 0) return -1;
+    dim3 grid((unsigned)rows), block(LN_THREADS);
+    const bool vec = (C % 8) == 0 && C <= LN_THREADS * 8 * 4 && ((uintptr_t)stream % 16) == 0 &&
+                     ((uintptr_t)y % 16) == 0 && ((uintptr_t)copy % 16) == 0 &&
+                     ((uintptr_t)w % 16) == 0 && ((uintptr_t)bias % 16) == 0;
+#define ALA(TY, TC) stream, (const TY*)y, alpha, w, bias, eps, (TC*)copy, C
+#define ALN(TY, TC) do { \
+        if (!vec) add_layer_norm_kernel<TY, TC><<<grid, block, 0, st>>>(ALA(TY, TC)); \
+        else if (C <= LN_THREADS * 8) \
+            add_layer_norm_vec_kernel<TY, TC, 1><<<grid, block, 0, st>>>(ALA(TY, TC)); \
+        else if (C <= LN_THREADS * 16) \
+            add_layer_norm_vec_kernel<TY, TC, 2><<<grid, block, 0, st>>>(ALA(TY, TC)); \
+        else add_layer_norm_vec_kernel<TY, TC, 4><<<grid, block, 0, st>>>(ALA(TY, TC)); } while (0)
+    if (y_bf16 && copy_bf16) ALN(bf16, bf16);
+    else if (y_bf16) ALN(bf16, float);
+    else if (copy_bf16) ALN(float, bf16);
+    else ALN(float, float);
+#undef ALN
+#undef ALA
     return (int)hipGetLastError();
 }
 
@@ -2573,7 +2830,7 @@ int nx_paged_attn(const void* q, long qstride, const void* kc, long ktok, long k
     const bool v_al = (Dv % 8) == 0 && (vtok % vecn) == 0 && (vhead % vecn) == 0 &&
                       ((uintptr_t)vc % 16) == 0;
     if (io_bf16 && out_bf16 && S == 1 && G == 1 && vc == kc && vtok == ktok && k_al && v_al &&
-        !r1 && !gate && cap <= 0.f && qt_every <= 0 && keep == 0 && H >= 8 &&
+        !r1 && (!gate || ghead) && cap <= 0.f && qt_every <= 0 && keep == 0 && H >= 8 &&
         Dk <= 640 && (qstride % 8) == 0 && ((uintptr_t)q % 16) == 0) {
         // latent caches, single-token steps: one workgroup per token reads each
         // key row once and covers 512 value channels
@@ -2592,7 +2849,8 @@ int nx_paged_attn(const void* q, long qstride, const void* kc, long ktok, long k
             } \
             latent_decode_mfma_kernel<DKV><<<gl, bl, lsh, st>>>( \
                 (const bf16*)q, qstride, (const bf16*)kc, ktok, pos, seq, btab, max_blocks, sink, \
-                (bf16*)out, H, Dk, Dv, bsz, S, scale, nsplit, nks, ws, window, cmask); } while (0)
+                (bf16*)out, H, Dk, Dv, bsz, S, scale, nsplit, nks, ws, window, cmask, \
+                (const bf16*)gate, gstride); } while (0)
         if (dkp <= 128) LD(128);
         else if (dkp <= 256) LD(256);
         else if (dkp <= 384) LD(384);
@@ -2602,7 +2860,8 @@ int nx_paged_attn(const void* q, long qstride, const void* kc, long ktok, long k
         if (nks > 1) {
             const long waves = (long)B * S * H;
             latent_decode_merge_kernel<<<(unsigned)((waves + 3) / 4), 4 * WAVE, 0, st>>>(
-                ws, sink, pos, seq, (bf16*)out, (long)B * S, S, H, Dv, nks);
+                ws, sink, pos, seq, (bf16*)out, (long)B * S, S, H, Dv, nks, (const bf16*)gate,
+                gstride);
         }
         return (int)hipGetLastError();
     }
@@ -2756,17 +3015,18 @@ int nx_residual_add(float* x, const void* a, float sa, const void* b, float sb, 
     return (int)hipGetLastError();
 }
 
-int nx_gelu_mul(const void* gu, void* out, int is_bf16, long rows, int I, hipStream_t st) {
+int nx_gelu_mul(const void* gu, void* out, int is_bf16, long rows, int I, int silu,
+                hipStream_t st) {
     if (rows <= 0) return 0;
-    if ((I % 8) == 0 && ((uintptr_t)gu % 16) == 0 && ((uintptr_t)out % 16) == 0) {
-        dim3 gv((I / 8 + 255) / 256, (unsigned)(rows > 32768 ? 32768 : rows)), bv(256);
-        if (is_bf16) gelu_mul_vec_kernel<bf16><<<gv, bv, 0, st>>>((const bf16*)gu, (bf16*)out, rows, I);
-        else gelu_mul_vec_kernel<float><<<gv, bv, 0, st>>>((const float*)gu, (float*)out, rows, I);
-        return (int)hipGetLastError();
-    }
+    const bool vec = (I % 8) == 0 && ((uintptr_t)gu % 16) == 0 && ((uintptr_t)out % 16) == 0;
+    dim3 gv((I / 8 + 255) / 256, (unsigned)(rows > 32768 ? 32768 : rows));
     dim3 grid(grid_for(rows * I, 256)), block(256);
-    if (is_bf16) gelu_mul_kernel<bf16><<<grid, block, 0, st>>>((const bf16*)gu, (bf16*)out, rows, I);
-    else gelu_mul_kernel<float><<<grid, block, 0, st>>>((const float*)gu, (float*)out, rows, I);
+#define GM(T, A) do { if (vec) gelu_mul_vec_kernel<T, A><<<gv, block, 0, st>>>( \
+        (const T*)gu, (T*)out, rows, I); \
+    else gelu_mul_kernel<T, A><<<grid, block, 0, st>>>((const T*)gu, (T*)out, rows, I); } while (0)
+    if (is_bf16) { if (silu) GM(bf16, 1); else GM(bf16, 0); }
+    else { if (silu) GM(float, 1); else GM(float, 0); }
+#undef GM
     return (int)hipGetLastError();
 }
 
@@ -2810,14 +3070,14 @@ int nx_add_rms_norm(float* stream, const void* y, int y_bf16, const float* w, in
 }
 
 int nx_rope_pairs(const void* x, long xt, long xh, int x_bf16, void* out, long ot, long oh,
-                  int out_bf16, const int* pos, const float* inv_freq, int half, long ntok,
-                  int N, int C, hipStream_t st) {
+                  int out_bf16, const int* pos, const float* inv_freq, int half, int split,
+                  long ntok, int N, int C, hipStream_t st) {
     const long total = ntok * N * (C - half);
     if (total <= 0) return 0;
     if (2 * half > C) return -1;
     dim3 grid(grid_for(total, 256)), block(256);
 #define RP(TI, TO) rope_pairs_kernel<TI, TO><<<grid, block, 0, st>>>( \
-        (const TI*)x, xt, xh, (TO*)out, ot, oh, pos, inv_freq, half, ntok, N, C)
+        (const TI*)x, xt, xh, (TO*)out, ot, oh, pos, inv_freq, half, split, ntok, N, C)
     if (x_bf16 && out_bf16) RP(bf16, bf16);
     else if (x_bf16) RP(bf16, float);
     else if (out_bf16) RP(float, bf16);
@@ -2867,11 +3127,12 @@ int nx_decay_scan(const void* q, long qs, const void* k, long ks, const void* v,
                   const float* a_log, const float* head_decay, float k_scale, const float* skip,
                   float* state, const int* pos, const int* seq, const int* nvalid, float* out,
                   int B, int S, int H, int G, int D, int Dv, float* ws, float* wdec, int nseg,
-                  int seglen, hipStream_t st) {
+                  int seglen, int channel, float inv_tau, hipStream_t st) {
     if ((long)B * S <= 0) return 0;
     if (D <= 0 || Dv <= 0 || G <= 0 || H % G != 0 || D > 256) return -1;
     if ((dt == nullptr) == (head_decay == nullptr)) return -2;
-    if (dt && (!dt_bias || !a_log)) return -2;
+    if (dt && !channel && (!dt_bias || !a_log)) return -2;
+    if (channel && (!dt || a_log || skip)) return -2;
     if (H > 65535 || B > 65535) return -3;
     // the kernel reads state rows 16 bytes at a time when dim % 4 == 0
     if (((uintptr_t)state % 16) != 0 || ((uintptr_t)ws % 16) != 0) return -5;
@@ -2879,40 +3140,55 @@ int nx_decay_scan(const void* q, long qs, const void* k, long ks, const void* v,
         return -4;
     const int cb = (Dv + 15) / 16;
     dim3 grid(cb * nseg, H, B), block(256);
-#define DSK(T, TD, RV, MD) decay_scan_kernel<T, TD, RV, MD><<<grid, block, 0, st>>>( \
+#define DSK(T, TD, RV, MD, CHV) decay_scan_kernel<T, TD, RV, MD, CHV><<<grid, block, 0, st>>>( \
         (const T*)q, qs, (const T*)k, ks, (const T*)v, vs, (const TD*)dt, dts, dt_bias, a_log, \
         head_decay, k_scale, skip, state, pos, seq, nvalid, out, S, H, G, D, Dv, ws, wdec, nseg, \
-        seglen)
-#define DSR(T, TD, MD) do { if (D <= 16) DSK(T, TD, 1, MD); else if (D <= 32) DSK(T, TD, 2, MD); \
-        else if (D <= 64) DSK(T, TD, 4, MD); else if (D <= 128) DSK(T, TD, 8, MD); \
-        else DSK(T, TD, 16, MD); } while (0)
-#define DST(MD) do { \
-        if (in_bf16) { if (dt_bf16) DSR(bf16, bf16, MD); else DSR(bf16, float, MD); } \
-        else { if (dt_bf16) DSR(float, bf16, MD); else DSR(float, float, MD); } } while (0)
+        seglen, inv_tau)
+#define DSR(T, TD, MD, CHV) do { if (D <= 16) DSK(T, TD, 1, MD, CHV); \
+        else if (D <= 32) DSK(T, TD, 2, MD, CHV); \
+        else if (D <= 64) DSK(T, TD, 4, MD, CHV); else if (D <= 128) DSK(T, TD, 8, MD, CHV); \
+        else DSK(T, TD, 16, MD, CHV); } while (0)
+#define DST(MD, CHV) do { \
+        if (in_bf16) { if (dt_bf16) DSR(bf16, bf16, MD, CHV); else DSR(bf16, float, MD, CHV); } \
+        else { if (dt_bf16) DSR(float, bf16, MD, CHV); else DSR(float, float, MD, CHV); } } while (0)
+#define DSC(MD) do { if (channel) DST(MD, true); else DST(MD, false); } while (0)
     if (nseg == 1) {
-        DST(0);
+        DSC(0);
     } else {
-        DST(1);
+        DSC(1);
         const long per_head = (long)Dv * D;
         decay_scan_link_kernel<<<grid_for((long)B * H * per_head, 256), 256, 0, st>>>(
-            ws, wdec, state, pos, seq, nvalid, B, S, H, per_head, nseg);
-        DST(2);
+            ws, wdec, state, pos, seq, nvalid, B, S, H, per_head, nseg, channel ? D : 1);
+        DSC(2);
     }
+#undef DSC
 #undef DST
 #undef DSR
 #undef DSK
     return (int)hipGetLastError();
 }
 
+int nx_channel_decay(const void* z, long zs, int z_bf16, const float* bias, float inv_tau,
+                     float* out, long rows, int C, hipStream_t st) {
+    if (rows * C <= 0) return 0;
+    if (!bias) return -1;
+    dim3 grid(grid_for(rows * C, 256)), block(256);
+    if (z_bf16) channel_decay_kernel<bf16><<<grid, block, 0, st>>>(
+        (const bf16*)z, zs, bias, inv_tau, out, rows, C);
+    else channel_decay_kernel<float><<<grid, block, 0, st>>>(
+        (const float*)z, zs, bias, inv_tau, out, rows, C);
+    return (int)hipGetLastError();
+}
+
 int nx_group_gated_norm(const float* y, const void* gate, long gs, int gate_bf16, const float* w,
-                        float eps, int groups, int gate_first, void* out, int out_bf16,
-                        long rows, int C, hipStream_t st) {
+                        float eps, int groups, int gate_first, int wshared, void* out,
+                        int out_bf16, long rows, int C, hipStream_t st) {
     if (rows <= 0) return 0;
     if (groups <= 0 || C % groups != 0) return -1;
     const long waves = rows * groups;
     dim3 grid((unsigned)((waves + 3) / 4)), block(4 * WAVE);
 #define GN(TG, TO) group_gated_norm_kernel<TG, TO><<<grid, block, 0, st>>>( \
-        y, (const TG*)gate, gs, w, eps, groups, gate_first, (TO*)out, rows, C)
+        y, (const TG*)gate, gs, w, eps, groups, gate_first, wshared, (TO*)out, rows, C)
     if (gate_bf16 && out_bf16) GN(bf16, bf16);
     else if (gate_bf16) GN(bf16, float);
     else if (out_bf16) GN(float, bf16);
@@ -2937,7 +3213,8 @@ int nx_group_router(const float* logits, long ls, int E, int extra, int top, int
 
 int nx_router_fused(const void* x, long xs, int x_bf16, const float* w, int W, int E, int extra,
                     int top, int ngroups, int keep, float scale, int normalize, const float* corr,
-                    float* dense, int* idx, float* wts, long T, hipStream_t st) {
+                    const float* bias, float* dense, int* idx, float* wts, long T,
+                    hipStream_t st) {
     if (T <= 0) return 0;
     if (E <= 0 || top <= 0 || top > E || top > WAVE || ngroups <= 0 || E % ngroups != 0 ||
         keep <= 0 || keep > ngroups || (long)top > (long)(E / ngroups) * keep || W <= 0) return -1;
@@ -2948,49 +3225,43 @@ int nx_router_fused(const void* x, long xs, int x_bf16, const float* w, int W, i
                     ((uintptr_t)w % 16) == 0;
     dim3 grid((unsigned)T), block(RT_WAVES * WAVE);
     if (x_bf16) router_fused_kernel<bf16><<<grid, block, sh, st>>>(
-        (const bf16*)x, xs, w, W, vec, E, extra, top, ngroups, keep, scale, normalize, corr, dense,
-        idx, wts);
+        (const bf16*)x, xs, w, W, vec, E, extra, top, ngroups, keep, scale, normalize, corr, bias,
+        dense, idx, wts);
     else router_fused_kernel<float><<<grid, block, sh, st>>>(
-        (const float*)x, xs, w, W, vec, E, extra, top, ngroups, keep, scale, normalize, corr, dense,
-        idx, wts);
+        (const float*)x, xs, w, W, vec, E, extra, top, ngroups, keep, scale, normalize, corr, bias,
+        dense, idx, wts);
     return (int)hipGetLastError();
 }
 
 int nx_latent_row(const void* x, long xs, int is_bf16, const float* w, float eps,
-                  const float* inv_freq, int half, const int* pos, const int* slots, void* cache,
-                  long nslots, void* row, long rs, long ntok, int C, int R, hipStream_t st) {
+                  const float* inv_freq, int half, int split, const int* pos, const int* slots,
+                  void* cache, long nslots, void* row, long rs, long ntok, int C, int R, hipStream_t st) {
     if (ntok <= 0) return 0;
     if (C <= 0 || R < 0 || 2 * half > R || (half > 0 && !inv_freq)) return -1;
     dim3 grid((unsigned)((ntok + 3) / 4)), block(4 * WAVE);
     if (is_bf16) latent_row_kernel<bf16><<<grid, block, 0, st>>>(
-        (const bf16*)x, xs, w, eps, inv_freq, half, pos, slots, (bf16*)cache, nslots, (bf16*)row,
+        (const bf16*)x, xs, w, eps, inv_freq, half, split, pos, slots, (bf16*)cache, nslots, (bf16*)row,
         rs, ntok, C, R);
     else latent_row_kernel<float><<<grid, block, 0, st>>>(
-        (const float*)x, xs, w, eps, inv_freq, half, pos, slots, (float*)cache, nslots,
+        (const float*)x, xs, w, eps, inv_freq, half, split, pos, slots, (float*)cache, nslots,
         (float*)row, rs, ntok, C, R);
     return (int)hipGetLastError();
 }
 
-int nx_relu2_scale(const void* x, int is_bf16, const float* gates, int gcols, int ff, int E,
-                   void* out, long rows, int C, hipStream_t st) {
+int nx_act_scale(const void* x, int is_bf16, const float* gates, int gcols, int ff, int E,
+                 int act, void* out, long rows, int C, hipStream_t st) {
     if (rows * C <= 0) return 0;
-    if (ff <= 0 || (gates && (gcols < E || (C > E * ff && gcols < E + 1)))) return -1;
-    const int esz = is_bf16 ? 2 : 4;
+    if (ff <= 0 || (gates && gcols < E) || act < 0 || act > 1) return -1;
     const bool vec = (C % 8) == 0 && (ff % 8) == 0 && ((uintptr_t)x % 16) == 0 &&
-                     ((uintptr_t)out % 16) == 0 && esz > 0;
-    if (vec) {
-        dim3 grid(grid_for(rows * (C / 8), 256)), block(256);
-        if (is_bf16) relu2_scale_vec_kernel<bf16><<<grid, block, 0, st>>>(
-            (const bf16*)x, gates, gcols, ff, E, (bf16*)out, rows, C);
-        else relu2_scale_vec_kernel<float><<<grid, block, 0, st>>>(
-            (const float*)x, gates, gcols, ff, E, (float*)out, rows, C);
-    } else {
-        dim3 grid(grid_for(rows * C, 256)), block(256);
-        if (is_bf16) relu2_scale_kernel<bf16><<<grid, block, 0, st>>>(
-            (const bf16*)x, gates, gcols, ff, E, (bf16*)out, rows, C);
-        else relu2_scale_kernel<float><<<grid, block, 0, st>>>(
-            (const float*)x, gates, gcols, ff, E, (float*)out, rows, C);
-    }
+                     ((uintptr_t)out % 16) == 0;
+    dim3 grid(grid_for(vec ? rows * (C / 8) : rows * C, 256)), block(256);
+#define AS(T, A) do { if (vec) act_scale_vec_kernel<T, A><<<grid, block, 0, st>>>( \
+        (const T*)x, gates, gcols, ff, E, (T*)out, rows, C); \
+    else act_scale_kernel<T, A><<<grid, block, 0, st>>>( \
+        (const T*)x, gates, gcols, ff, E, (T*)out, rows, C); } while (0)
+    if (is_bf16) { if (act) AS(bf16, 1); else AS(bf16, 0); }
+    else { if (act) AS(float, 1); else AS(float, 0); }
+#undef AS
     return (int)hipGetLastError();
 }
 
@@ -3067,6 +3338,36 @@ int nx_embed_pos(const void* emb, const void* table, int is_bf16, const int* pos
         (const bf16*)emb, (const bf16*)table, pos, out, ntok, C, rows_in_table);
     else embed_pos_kernel<float><<<grid, block, 0, st>>>(
         (const float*)emb, (const float*)table, pos, out, ntok, C, rows_in_table);
+    return (int)hipGetLastError();
+}
+
+int nx_bigram_embed(const long long* ids, const int* pos, const int* seq, const int* nvalid,
+                    const void* emb, const void* table, int is_bf16, int* last, long long mul_prev,
+                    long long mul_cur, long long buckets, int vocab, float* out, int B, int S,
+                    int C, hipStream_t st) {
+    if ((long)B * S * C <= 0) return 0;
+    if (buckets <= 0 || vocab <= 0) return -1;
+    dim3 grid((unsigned)((long)B * S)), block(256);
+    const int vec = (C % 8) == 0 && ((uintptr_t)emb % 16) == 0 && ((uintptr_t)table % 16) == 0 &&
+                    ((uintptr_t)out % 16) == 0;
+    if (is_bf16) bigram_embed_kernel<bf16><<<grid, block, 0, st>>>(
+        ids, pos, seq, nvalid, (const bf16*)emb, (const bf16*)table, last, mul_prev, mul_cur,
+        buckets, vocab, out, S, C, vec);
+    else bigram_embed_kernel<float><<<grid, block, 0, st>>>(
+        ids, pos, seq, nvalid, (const float*)emb, (const float*)table, last, mul_prev, mul_cur,
+        buckets, vocab, out, S, C, vec);
+    return (int)hipGetLastError();
+}
+
+int nx_token_gate(const void* z, long zs, const long long* ids, const void* table, long ts,
+                  int off, int vocab, int is_bf16, void* out, long rows, int C, hipStream_t st) {
+    if (rows * C <= 0) return 0;
+    if (vocab <= 0 || off < 0 || (long)off + C > ts) return -1;
+    dim3 grid(grid_for(rows * C, 256)), block(256);
+    if (is_bf16) token_gate_kernel<bf16><<<grid, block, 0, st>>>(
+        (const bf16*)z, zs, ids, (const bf16*)table, ts, off, vocab, (bf16*)out, rows, C);
+    else token_gate_kernel<float><<<grid, block, 0, st>>>(
+        (const float*)z, zs, ids, (const float*)table, ts, off, vocab, (float*)out, rows, C);
     return (int)hipGetLastError();
 }
 

@@ -218,13 +218,14 @@ def topk_topp_sample(
 # p0..p0+n-1; pad columns carry position -1 and pad rows seq_id -1.
 
 def layer_norm(x: torch.Tensor, weight: torch.Tensor, eps: float,
-               out_dtype: torch.dtype) -> torch.Tensor:
-    """Bias-free LayerNorm with fp32 statistics."""
+               out_dtype: torch.dtype, bias=None) -> torch.Tensor:
+    """LayerNorm (optional bias) with fp32 statistics."""
     xf = x.float()
     mu = xf.mean(-1, keepdim=True)
     xc = xf - mu
     var = (xc * xc).mean(-1, keepdim=True)
-    return (xc * torch.rsqrt(var + eps) * weight.float()).to(out_dtype)
+    y = xc * torch.rsqrt(var + eps) * weight.float()
+    return (y if bias is None else y + bias.float()).to(out_dtype)
 
 
 def _row_extent(positions: torch.Tensor):
@@ -434,6 +435,15 @@ def rms_norm_rows(x: torch.Tensor, weight: torch.Tensor, eps: float,
     return y.to(out_dtype)
 
 
+def rotate_pairs(x: torch.Tensor, positions: torch.Tensor, inv_freq: torch.Tensor,
+                 half_split: bool) -> torch.Tensor:
+    """Rotary positions in interleaved pairs (2i, 2i+1) or half-split pairs
+    (i, i + len(inv_freq)); see :func:`rotate_interleaved`."""
+    if half_split:
+        return head_norm_rotate(x, positions, None, 0.0, inv_freq)
+    return rotate_interleaved(x, positions, inv_freq)
+
+
 def rotate_interleaved(x: torch.Tensor, positions: torch.Tensor,
                        inv_freq: torch.Tensor) -> torch.Tensor:
     """Rotary positions on channel pairs (2i, 2i+1) of the first
@@ -480,18 +490,26 @@ def head_norm_rotate(x: torch.Tensor, positions: torch.Tensor, norm_weight, eps:
     return torch.cat([u * c - v * sn, v * c + u * sn, xf[..., 2 * half:]], dim=-1)
 
 
+def channel_decay(z, bias, tau: float):
+    """sigmoid(z + bias)^(1/tau), fp32, through the logarithm."""
+    return torch.exp(torch.nn.functional.logsigmoid(z.float() + bias.float()) / tau)
+
+
 def decay_scan(q, k, v, state, positions, seq_ids, dim: int, vdim: int,
                dt=None, dt_bias=None, a_log=None, head_decay=None,
-               k_scale: float = 1.0, skip=None):
-    """Linear recurrence with a scalar decay per head and matrix state,
-    carried in ``state`` (slots, H, vdim, dim) fp32 (stored transposed):
+               k_scale: float = 1.0, skip=None, channel_logits=None, channel_bias=None,
+               tau: float = 1.0):
+    """Linear recurrence with a decay per head and matrix state, carried in ``state`` (slots, H, vdim, dim) fp32 (stored transposed):
 
         S_t = a_t S_{t-1} + k_t (w_t v_t)^T ;  o_t = S_t^T q_t (+ skip_h v_t)
 
-    Two ways to give the decay: ``dt`` (B,S,H) raw step-size projections with
+    Three ways to give the decay: ``dt`` (B,S,H) raw step-size projections with
     ``dt_bias`` and ``a_log`` (H,): w_t = softplus(dt + dt_bias), a_t =
     exp(-exp(a_log) w_t) (selective state spaces: k = B, q = C, v = x); or
-    ``head_decay`` (H,): a_t = head_decay, w_t = 1 (retention). q, k
+    ``head_decay`` (H,): a_t = head_decay, w_t = 1 (retention); or
+    ``channel_logits`` (B,S,H*dim) with ``channel_bias`` (H*dim,) and ``tau``:
+    a decay per head and KEY CHANNEL, S_t = diag(a_t) S_{t-1} + k_t v_t^T,
+    a_t = sigmoid(logits + bias)^(1/tau) (gated linear attention). q, k
     (B,S,G*dim) are shared by H/G consecutive heads, v (B,S,H*vdim); k is
     multiplied by ``k_scale``. Returns fp32 (B,S,H*vdim)."""
     B, S = positions.shape
@@ -505,6 +523,9 @@ def decay_scan(q, k, v, state, positions, seq_ids, dim: int, vdim: int,
     if dt is not None:
         w = torch.nn.functional.softplus(dt.float() + dt_bias.float(), threshold=20.0)
         a = torch.exp(-torch.exp(a_log.float()) * w)
+    elif channel_logits is not None:
+        a = channel_decay(channel_logits, channel_bias, tau).reshape(B, S, H, D)
+        w = torch.ones(B, S, H, dtype=torch.float32, device=v.device)
     else:
         a = head_decay.float().view(1, 1, H).expand(B, S, H)
         w = torch.ones(B, S, H, dtype=torch.float32, device=v.device)
@@ -518,7 +539,7 @@ def decay_scan(q, k, v, state, positions, seq_ids, dim: int, vdim: int,
         St = state[slot].float().transpose(-1, -2).clone() if int(p0s[b]) > 0 else torch.zeros(
             H, D, Dv, dtype=torch.float32, device=v.device)
         for t in range(n):
-            St = a[b, t].view(H, 1, 1) * St + kf[b, t].unsqueeze(-1) * (
+            St = a[b, t].view(H, -1, 1) * St + kf[b, t].unsqueeze(-1) * (
                 w[b, t].view(H, 1) * vf[b, t]).unsqueeze(1)
             out[b, t] = torch.einsum("hdv,hd->hv", St, qf[b, t])
         state[slot] = St.transpose(-1, -2).to(state.dtype)
@@ -530,8 +551,8 @@ def decay_scan(q, k, v, state, positions, seq_ids, dim: int, vdim: int,
 def group_gated_norm(y, gate, weight, eps: float, groups: int, gate_first: bool,
                      out_dtype=torch.float32):
     """RMS norm of (.., C) rows in ``groups`` equal parts (each part by its
-    own root mean square), optional weight (C,), and a silu gate applied
-    before the norm (``gate_first``) or after it."""
+    own root mean square), optional weight (C,) or, shared by the parts,
+    (C / groups,), and a silu gate applied before the norm (``gate_first``) or after it."""
     yf = y.float()
     g = torch.nn.functional.silu(gate.float())
     if gate_first:
@@ -540,7 +561,8 @@ def group_gated_norm(y, gate, weight, eps: float, groups: int, gate_first: bool,
     yg = yf.reshape(*shp[:-1], groups, shp[-1] // groups)
     yf = (yg * torch.rsqrt((yg * yg).mean(-1, keepdim=True) + eps)).reshape(shp)
     if weight is not None:
-        yf = yf * weight.float()
+        wf = weight.float()
+        yf = yf * (wf if wf.numel() == shp[-1] else wf.repeat(groups))
     if not gate_first:
         yf = yf * g
     return yf.to(out_dtype)
@@ -604,20 +626,23 @@ def clamped_glu_scale(hid, gates, expert_ff: int, num_experts: int, limit: float
     return out.to(out_dtype)
 
 
-def relu2_scale(hid, gates, expert_ff: int, num_experts: int, out_dtype):
-    """(T, E*ff + rest) hidden pre-activations -> relu(x)^2 times the token's
+def act_scale(hid, gates, expert_ff: int, num_experts: int, act: str, out_dtype):
+    """(T, E*ff + rest) hidden pre-activations -> act(x) times the token's
     gate of the column's owner: column c < E*ff belongs to expert c // ff,
-    the remaining columns (a shared expert) to gate column E; ``gates`` is
-    (T, E + 1), or (T, E) when there are no remaining columns, or None for a
-    plain relu(x)^2."""
+    the remaining columns (a shared expert) to gate column E, or to a gate of
+    one when ``gates`` has only E columns; ``gates`` None is a plain act(x).
+    ``act``: relu2 (squared relu) or gelu (the exact one)."""
     T, C = hid.shape
     E = num_experts
-    hf = torch.relu(hid.float()) ** 2
+    hf = hid.float()
+    hf = torch.relu(hf) ** 2 if act == "relu2" else torch.nn.functional.gelu(hf)
     if gates is None:
         return hf.to(out_dtype)
-    assert C == E * expert_ff or gates.shape[1] == E + 1
+    g = gates.float()[:, :E + 1]
+    if g.shape[1] == E:
+        g = torch.cat([g, torch.ones(T, 1, dtype=g.dtype, device=g.device)], dim=1)
     cols = (torch.arange(C, device=hid.device) // expert_ff).clamp(max=E)
-    return (hf * gates.float()[:, cols]).to(out_dtype)
+    return (hf * g[:, cols]).to(out_dtype)
 
 
 def scaled_residual(x, terms):
@@ -630,3 +655,33 @@ def scaled_residual(x, terms):
             yf = yf * torch.rsqrt((yf * yf).mean(-1, keepdim=True) + eps)
         x.add_(yf * w.float())
     return x
+
+
+def bigram_embedding(ids, embed, table, last, positions, seq_ids, mul_prev: int, mul_cur: int):
+    """embed[tok] + table[row] in fp32, row = (prev * mul_prev + tok *
+    mul_cur) mod buckets, buckets = rows of the table - 1; a sequence's first
+    token (position 0) takes row ``buckets``. The token before a step's first
+    column is ``last[slot]``, which is advanced to the row's last token. Pad
+    tokens give zero rows."""
+    B, S = ids.shape
+    buckets = table.shape[0] - 1
+    prev = torch.zeros_like(ids)
+    prev[:, 1:] = ids[:, :-1]
+    slots = seq_ids.long().clamp(min=0)
+    prev[:, 0] = last[slots].to(ids.dtype)
+    rows = (prev * int(mul_prev) + ids * int(mul_cur)) % buckets
+    rows = torch.where(positions > 0, rows, torch.full_like(rows, buckets))
+    x = embed[ids].float() + table[rows].float()
+    real = (positions >= 0) & (seq_ids >= 0).view(B, 1)
+    for b in range(B):
+        n = int(real[b].sum())
+        if n:
+            last[int(seq_ids[b])] = ids[b, n - 1].to(last.dtype)
+    return x * real.unsqueeze(-1)
+
+
+def token_gate(z, ids, table, offset: int):
+    """gelu_tanh(z) * table[ids][..., offset:offset + C], fp32."""
+    C = z.shape[-1]
+    e = table[ids.reshape(-1)][:, offset:offset + C].float().reshape(z.shape)
+    return torch.nn.functional.gelu(z.float(), approximate="tanh") * e

@@ -160,6 +160,13 @@ class StepLayout:
         self.stream_copy = None
         # True when every row of the step starts its sequence (a whole prompt)
         self.fresh = False
+        # dense rows of latent layers whose cache a later layer reads (whole
+        # prompts only), by the owner's cache index
+        self.latent_rows = {}
+        # the step's token ids and the (vocab, layers * dim) table that layers
+        # read them from, for models that use ids past the embedding
+        self.tokens = None
+        self.side_table = None
 
     def i32(self, t: torch.Tensor) -> torch.Tensor:
         """int32 copy of a per-step index tensor (block table, slot mapping),
@@ -172,18 +179,43 @@ class StepLayout:
 
 
 # ----------------------------------------------------------------------
-def layer_norm(x, weight, eps: float, out_dtype: torch.dtype):
-    """Bias-free LayerNorm of an fp32 stream, fp32 statistics."""
+def layer_norm(x, weight, eps: float, out_dtype: torch.dtype, bias=None):
+    """LayerNorm (optional bias) of an fp32 stream, fp32 statistics."""
     if x.is_cuda:
         lib = _load()
         x = _f32(x)
         out = torch.empty(x.shape, dtype=out_dtype, device=x.device)
         C = x.shape[-1]
-        _check(lib.nx_layer_norm(_p(x), _p(_f32(weight)), _p(out), _is_bf16(out),
+        _check(lib.nx_layer_norm(_p(x), _p(_f32(weight)),
+                                 _p(None if bias is None else _f32(bias)), _p(out), _is_bf16(out),
                                  ctypes.c_long(x.numel() // C), C,
                                  ctypes.c_float(eps), _stream()), "layer_norm")
         return out
-    return ref.layer_norm(x, weight, eps, out_dtype)
+    return ref.layer_norm(x, weight, eps, out_dtype, bias)
+
+
+def add_layer_norm(stream, y, alpha: float, weight, bias, eps: float, copy_dtype=None):
+    """Residual step with the norm after the sum, in place on the fp32 stream:
+    stream = layer_norm(alpha * stream + y) * weight + bias. Returns the new
+    stream in ``copy_dtype`` (the next sublayer's GEMM input; the stream
+    itself for float32), None without one."""
+    if stream.is_cuda:
+        lib = _load()
+        assert stream.dtype == torch.float32 and stream.is_contiguous()
+        y = y.contiguous()
+        assert y.numel() == stream.numel()
+        C = stream.shape[-1]
+        copy = None
+        if copy_dtype is not None and copy_dtype != torch.float32:
+            copy = torch.empty(stream.shape, dtype=copy_dtype, device=stream.device)
+        _check(lib.nx_add_layer_norm(
+            _p(stream), _p(y), _is_bf16(y), ctypes.c_float(alpha), _p(_f32(weight)),
+            _p(_f32(bias)), ctypes.c_float(eps), _p(copy), 0 if copy is None else 1,
+            ctypes.c_long(stream.numel() // C), C, _stream()), "add_layer_norm")
+    else:
+        stream.copy_(ref.layer_norm(alpha * stream + y.float(), weight, eps, torch.float32, bias))
+        copy = None if copy_dtype in (None, torch.float32) else stream.to(copy_dtype)
+    return stream if copy_dtype == torch.float32 else copy
 
 
 def short_conv(x, w, tail, step: StepLayout, activation: str = "none",
@@ -360,6 +392,15 @@ def gated_delta_rule(qkv, beta, a, dt_bias, a_log, gate, norm_w, eps: float,
                                 dim, vdim, out_dtype, gate_act)
 
 
+def head_product(a, w):
+    """Per-head product a (T,H,K) x w (H,N,K)^T -> (T,H,N), 32-bit sums."""
+    T, H, K = a.shape
+    out = torch.empty(T, H, w.shape[1], dtype=a.dtype, device=a.device)
+    # (the library's batched product gets no transposed right operand)
+    torch.bmm(a.transpose(0, 1), w.transpose(1, 2).contiguous(), out=out.transpose(0, 1))
+    return out
+
+
 def softcap(logits, cap: float):
     """cap * tanh(logits / cap) in fp32."""
     if logits.is_cuda:
@@ -391,19 +432,31 @@ def residual_add(x, a, sa: float = 1.0, b=None, sb: float = 1.0):
     return x
 
 
+def _gated_unit(gate_up, silu: bool):
+    I = gate_up.shape[-1] // 2
+    lib = _load()
+    gu = gate_up.contiguous()
+    out = torch.empty(gu.shape[:-1] + (I,), dtype=gu.dtype, device=gu.device)
+    _check(lib.nx_gelu_mul(_p(gu), _p(out), _is_bf16(gu),
+                           ctypes.c_long(gu.numel() // (2 * I)), I, int(silu), _stream()),
+           "gated_unit")
+    return out
+
+
 def gelu_tanh_mul_fused(gate_up):
     """(rows, 2I) [gate | up] -> gelu_tanh(gate) * up."""
-    I = gate_up.shape[-1] // 2
     if gate_up.is_cuda:
-        lib = _load()
-        gu = gate_up.contiguous()
-        out = torch.empty(gu.shape[:-1] + (I,), dtype=gu.dtype, device=gu.device)
-        _check(lib.nx_gelu_mul(_p(gu), _p(out), _is_bf16(gu),
-                               ctypes.c_long(gu.numel() // (2 * I)), I, _stream()),
-               "gelu_tanh_mul_fused")
-        return out
+        return _gated_unit(gate_up, False)
     g, u = gate_up.float().chunk(2, dim=-1)
     return ref.gelu_tanh_mul(g, u).to(gate_up.dtype)
+
+
+def silu_mul_fused(gate_up):
+    """(rows, 2I) [gate | up] -> silu(gate) * up."""
+    if gate_up.is_cuda:
+        return _gated_unit(gate_up, True)
+    g, u = gate_up.float().chunk(2, dim=-1)
+    return (torch.nn.functional.silu(g) * u).to(gate_up.dtype)
 
 
 def rms_norm(x, weight, eps: float, one_plus: bool = False, out_dtype=None, out=None):
@@ -477,8 +530,10 @@ def add_rms_norm(stream, y, weight, eps: float, one_plus: bool = True, copy_dtyp
     return stream if copy_dtype == torch.float32 else stream.to(copy_dtype)
 
 
-def rotate_interleaved(x, step: StepLayout, inv_freq, out=None, out_dtype=None):
-    """Rotary positions on interleaved channel pairs (2i, 2i+1) of the first
+def rotate_interleaved(x, step: StepLayout, inv_freq, out=None, out_dtype=None,
+                       half_split: bool = False):
+    """Rotary positions on interleaved channel pairs (2i, 2i+1) — or, with
+    ``half_split``, pairs (i, i + len(inv_freq)) — of the first
     2*len(inv_freq) channels of every head; angles p * inv_freq[i] in fp32.
     x (B,S,N,C), possibly a strided view; ``out`` likewise (may be a slice of
     a wider buffer). Channels past the rotated ones are copied."""
@@ -494,10 +549,10 @@ def rotate_interleaved(x, step: StepLayout, inv_freq, out=None, out_dtype=None):
             _p(x), ctypes.c_long(_token_stride(x)), ctypes.c_long(x.stride(2)), _is_bf16(x),
             _p(out), ctypes.c_long(_token_stride(out)), ctypes.c_long(out.stride(2)),
             _is_bf16(out),
-            _p(step.positions), _p(_f32(inv_freq)), inv_freq.numel(),
+            _p(step.positions), _p(_f32(inv_freq)), inv_freq.numel(), int(half_split),
             ctypes.c_long(B * S), N, C, _stream()), "rotate_interleaved")
         return out
-    y = ref.rotate_interleaved(x, step.positions, inv_freq).to(out_dtype)
+    y = ref.rotate_pairs(x, step.positions, inv_freq, half_split).to(out_dtype)
     if out is not None:
         out.copy_(y)
         return out
@@ -552,14 +607,36 @@ def head_norm_rotate(x, step: StepLayout, norm_weight, eps: float, inv_freq,
                                 mscale).reshape(B, S, N * C).to(out_dtype)
 
 
+def channel_decay(z, bias, tau: float):
+    """sigmoid(z + bias)^(1/tau) in fp32; z (B,S,C) may be a column slice."""
+    if z.is_cuda:
+        lib = _load()
+        C = z.shape[-1]
+        out = torch.empty(z.shape, dtype=torch.float32, device=z.device)
+        assert bias.numel() == C
+        _check(lib.nx_channel_decay(_p(z), ctypes.c_long(_rows_view(z)), _is_bf16(z),
+                                    _p(_f32(bias)), ctypes.c_float(1.0 / tau), _p(out),
+                                    ctypes.c_long(z.numel() // C), C, _stream()),
+               "channel_decay")
+        return out
+    return ref.channel_decay(z, bias, tau)
+
+
+# steps of at most this many tokens a row compute their channel decays inside
+# the scan (once per block of value channels) instead of in a launch of their own
+INLINE_DECAY_MAX_TOKENS = 4
+
+
 def decay_scan(q, k, v, state, step: StepLayout, dim: int, vdim: int, dt=None,
-               dt_bias=None, a_log=None, head_decay=None, k_scale: float = 1.0, skip=None):
-    """Scalar-decay linear recurrence with matrix state (see ref.decay_scan):
-    selective state spaces (``dt``/``dt_bias``/``a_log``) or fixed per-head
-    decays (``head_decay``). q, k (B,S,G*dim), v (B,S,H*vdim) may be column
+               dt_bias=None, a_log=None, head_decay=None, k_scale: float = 1.0, skip=None,
+               channel_logits=None, channel_bias=None, tau: float = 1.0):
+    """Decayed linear recurrence with matrix state (see ref.decay_scan):
+    selective state spaces (``dt``/``dt_bias``/``a_log``), fixed per-head
+    decays (``head_decay``) or a decay per key channel (``channel_logits``
+    (B,S,H*dim) with ``channel_bias`` and ``tau``). q, k (B,S,G*dim), v (B,S,H*vdim) may be column
     slices of wider tensors; ``state`` (slots, H, vdim, dim) fp32 is read
     (unless the row starts at position 0) and advanced. Returns fp32."""
-    assert (dt is None) != (head_decay is None)
+    assert sum(x is not None for x in (dt, head_decay, channel_logits)) == 1
     if v.is_cuda:
         lib = _load()
         B, S = v.shape[0], v.shape[1]
@@ -569,6 +646,13 @@ def decay_scan(q, k, v, state, step: StepLayout, dim: int, vdim: int, dt=None,
         assert state.is_contiguous() and tuple(state.shape[1:]) == (H, vdim, dim)
         assert H % G == 0 and q.shape[-1] == G * dim and k.shape[-1] == G * dim
         out = torch.empty(B, S, H * vdim, dtype=torch.float32, device=v.device)
+        channel, dch = channel_logits is not None, 1
+        if channel:
+            assert G == H and skip is None and channel_logits.shape[-1] == H * dim
+            assert channel_bias.numel() == H * dim
+            dt, dt_bias, dch = channel_logits, channel_bias, dim
+            if S > INLINE_DECAY_MAX_TOKENS:
+                dt, dt_bias = channel_decay(channel_logits, channel_bias, tau), None
         # a long row with few (row, head, channel block) workgroups is cut into
         # segments that scan side by side (two passes joined by a short serial
         # link over the segments' end states)
@@ -581,7 +665,7 @@ def decay_scan(q, k, v, state, step: StepLayout, dim: int, vdim: int, dt=None,
             if nseg > 1:
                 seglen = ((S + nseg - 1) // nseg + 15) // 16 * 16
                 ws = torch.empty(B * nseg * H * vdim * dim, dtype=torch.float32, device=v.device)
-                wdec = torch.empty(B * nseg * H, dtype=torch.float32, device=v.device)
+                wdec = torch.empty(B * nseg * H * dch, dtype=torch.float32, device=v.device)
         _check(lib.nx_decay_scan(
             _p(q), ctypes.c_long(_rows_view(q)), _p(k), ctypes.c_long(_rows_view(k)),
             _p(v), ctypes.c_long(_rows_view(v)), _is_bf16(v),
@@ -592,27 +676,32 @@ def decay_scan(q, k, v, state, step: StepLayout, dim: int, vdim: int, dt=None,
             _p(None if head_decay is None else _f32(head_decay)),
             ctypes.c_float(k_scale), _p(None if skip is None else _f32(skip)),
             _p(state), _p(step.positions), _p(step.seq_ids), _p(step.nvalid), _p(out),
-            B, S, H, G, dim, vdim, _p(ws), _p(wdec), nseg, seglen, _stream()), "decay_scan")
+            B, S, H, G, dim, vdim, _p(ws), _p(wdec), nseg, seglen, int(channel),
+            ctypes.c_float(1.0 / tau), _stream()), "decay_scan")
         return out
     return ref.decay_scan(q, k, v, state, step.positions, step.seq_ids, dim, vdim,
                           dt=dt, dt_bias=dt_bias, a_log=a_log, head_decay=head_decay,
-                          k_scale=k_scale, skip=skip)
+                          k_scale=k_scale, skip=skip, channel_logits=channel_logits,
+                          channel_bias=channel_bias, tau=tau)
 
 
 def group_gated_norm(y, gate, weight, eps: float, groups: int, gate_first: bool,
                      out_dtype=torch.float32):
     """RMS norm of fp32 rows in ``groups`` equal parts with a silu gate before
-    or after it and an optional weight (see ref.group_gated_norm). ``gate``
-    may be a column slice of a wider tensor."""
+    or after it and an optional weight, of the row's width or of one part's
+    (shared by the parts) (see ref.group_gated_norm). ``gate`` may be a column
+    slice of a wider tensor."""
     if y.is_cuda:
         lib = _load()
         C = y.shape[-1]
         assert y.dtype == torch.float32 and y.is_contiguous() and C % groups == 0
         out = torch.empty(y.shape, dtype=out_dtype, device=y.device)
+        assert weight is None or weight.numel() in (C, C // groups)
         _check(lib.nx_group_gated_norm(
             _p(y), _p(gate), ctypes.c_long(_rows_view(gate)), _is_bf16(gate),
             _p(None if weight is None else _f32(weight)), ctypes.c_float(eps), groups,
-            int(gate_first), _p(out), _is_bf16(out), ctypes.c_long(y.numel() // C), C,
+            int(gate_first), int(weight is not None and weight.numel() != C), _p(out),
+            _is_bf16(out), ctypes.c_long(y.numel() // C), C,
             _stream()), "group_gated_norm")
         return out
     return ref.group_gated_norm(y, gate, weight, eps, groups, gate_first, out_dtype)
@@ -650,9 +739,9 @@ FUSED_ROUTER_MAX_TOKENS = 512
 
 def route_tokens(x, weight, num_experts: int, top_k: int, n_groups: int = 1,
                  keep_groups: int = 1, scale: float = 1.0, normalize: bool = False,
-                 correction=None):
-    """Router product and selection: fp32 logits ``x.float() @ weight.T`` (x
-    (T, hidden) in any dtype, weight (E + extra, hidden) fp32), then
+                 correction=None, bias=None):
+    """Router product and selection: fp32 logits ``x.float() @ weight.T + bias``
+    (x (T, hidden) in any dtype, weight (E + extra, hidden) fp32), then
     :func:`group_limited_router`. Steps of few tokens do both in one launch;
     larger ones take the library product first."""
     T = x.shape[0]
@@ -668,18 +757,19 @@ def route_tokens(x, weight, num_experts: int, top_k: int, n_groups: int = 1,
             _p(x), ctypes.c_long(x.stride(0)), _is_bf16(x), _p(weight), weight.shape[1], E, C - E,
             top_k, max(n_groups, 1), max(min(keep_groups, n_groups), 1), ctypes.c_float(scale),
             int(normalize), _p(None if correction is None else _f32(correction)),
+            _p(None if bias is None else _f32(bias)),
             _p(dense), _p(idx), _p(wts), ctypes.c_long(T), _stream()), "route_tokens")
         return dense, idx, wts
-    logits = torch.nn.functional.linear(x.float(), weight)
+    logits = torch.nn.functional.linear(x.float(), weight, bias)
     return group_limited_router(logits, num_experts, top_k, n_groups, keep_groups, scale,
                                 normalize, correction=correction)
 
 
 def latent_row_write(x, norm_weight, eps: float, inv_freq, step: StepLayout, k_cache,
-                     slot_mapping, kv_rank: int, row=None):
+                     slot_mapping, kv_rank: int, row=None, half_split: bool = False):
     """Cache row of a latent layer in one pass: x (B,S,kv_rank + rot) (a column
-    slice is fine) -> [rms_norm(x[..., :kv_rank]) * w | interleaved-pair rotary
-    of the rest] scattered into the paged ``k_cache`` (blocks, block, 1,
+    slice is fine) -> [rms_norm(x[..., :kv_rank]) * w | rotary of the rest in
+    interleaved or ``half_split`` pairs] scattered into the paged ``k_cache`` (blocks, block, 1,
     kv_rank + rot) at ``slot_mapping``; ``row`` (B,S,kv_rank + rot, dense)
     also receives it when given."""
     B, S, CR = x.shape
@@ -691,43 +781,52 @@ def latent_row_write(x, norm_weight, eps: float, inv_freq, step: StepLayout, k_c
         assert row is None or (row.is_contiguous() and row.dtype == x.dtype and row.shape == x.shape)
         _check(lib.nx_latent_row(
             _p(x), ctypes.c_long(_token_stride(x)), _is_bf16(x), _p(_f32(norm_weight)),
-            ctypes.c_float(eps), _p(_f32(inv_freq)), inv_freq.numel(), _p(step.positions),
-            _p(step.i32(slot_mapping)), _p(k_cache),
+            ctypes.c_float(eps), _p(_f32(inv_freq)), inv_freq.numel(), int(half_split),
+            _p(step.positions), _p(step.i32(slot_mapping)), _p(k_cache),
             ctypes.c_long(k_cache.shape[0] * k_cache.shape[1]), _p(row),
             ctypes.c_long(0 if row is None else CR), ctypes.c_long(B * S), C, R, _stream()),
             "latent_row_write")
         return row
     r = torch.empty(B, S, CR, dtype=x.dtype, device=x.device)
     r[..., :C] = ref.rms_norm_rows(x[..., :C], norm_weight, eps, False, x.dtype)
-    r[..., C:] = ref.rotate_interleaved(x[..., C:].unsqueeze(2), step.positions,
-                                        inv_freq).squeeze(2).to(x.dtype)
+    r[..., C:] = ref.rotate_pairs(x[..., C:].unsqueeze(2), step.positions, inv_freq,
+                                  half_split).squeeze(2).to(x.dtype)
     ref.paged_kv_write(k_cache, None, r.view(B * S, 1, CR), None, slot_mapping)
     if row is not None:
         row.copy_(r)
     return row
 
 
-def relu2_scale(hid, gates, expert_ff: int, num_experts: int, out_dtype=None):
-    """relu(x)^2 of (T, E*ff + rest) pre-activations times the token's gate of
-    the column's expert; the remaining columns take gate column E (see
-    ref.relu2_scale). ``gates`` None: plain relu(x)^2."""
+EXPERT_ACTS = {"relu2": 0, "gelu": 1}
+
+
+def act_scale(hid, gates, expert_ff: int, num_experts: int, act: str = "relu2", out_dtype=None):
+    """act(x) of (T, E*ff + rest) pre-activations times the token's gate of the
+    column's expert; the remaining columns take gate column E, or one when
+    ``gates`` has only E columns (see ref.act_scale). ``act``: relu2 (squared
+    relu) or gelu (the exact one). ``gates`` None: plain act(x)."""
     out_dtype = out_dtype or hid.dtype
     if hid.is_cuda:
         lib = _load()
         T, C = hid.shape
         assert hid.is_contiguous() and out_dtype == hid.dtype
         out = torch.empty(T, C, dtype=out_dtype, device=hid.device)
+        code = EXPERT_ACTS[act]
         if gates is None:
-            _check(lib.nx_relu2_scale(_p(hid), _is_bf16(hid), _p(None), 0, max(C, 1), 1,
-                                      _p(out), ctypes.c_long(T), C, _stream()), "relu2_scale")
+            _check(lib.nx_act_scale(_p(hid), _is_bf16(hid), _p(None), 0, max(C, 1), 1, code,
+                                    _p(out), ctypes.c_long(T), C, _stream()), "act_scale")
             return out
-        assert gates.dtype == torch.float32 and gates.is_contiguous()
-        assert C == num_experts * expert_ff or gates.shape[1] == num_experts + 1
-        _check(lib.nx_relu2_scale(_p(hid), _is_bf16(hid), _p(gates), gates.shape[1], expert_ff,
-                                  num_experts, _p(out), ctypes.c_long(T), C, _stream()),
-               "relu2_scale")
+        assert gates.dtype == torch.float32 and gates.is_contiguous() and gates.shape[0] == T
+        _check(lib.nx_act_scale(_p(hid), _is_bf16(hid), _p(gates), gates.shape[1], expert_ff,
+                                num_experts, code, _p(out), ctypes.c_long(T), C, _stream()),
+               "act_scale")
         return out
-    return ref.relu2_scale(hid, gates, expert_ff, num_experts, out_dtype)
+    return ref.act_scale(hid, gates, expert_ff, num_experts, act, out_dtype)
+
+
+def relu2_scale(hid, gates, expert_ff: int, num_experts: int, out_dtype=None):
+    """:func:`act_scale` with the squared relu."""
+    return act_scale(hid, gates, expert_ff, num_experts, "relu2", out_dtype)
 
 
 def clamped_glu_scale(hid, gates, expert_ff: int, num_experts: int, limit: float,
@@ -813,3 +912,42 @@ def embed_positions(h, pos_table, step: StepLayout):
         return out
     p = step.positions.long().clamp(min=0, max=pos_table.shape[0] - 1)
     return h.float() + pos_table[p].float()
+
+
+def bigram_embedding(ids, embed, table, last, step: StepLayout, mul_prev: int, mul_cur: int):
+    """Token embedding rows plus a bigram row per token -> fp32 residual stream
+    (see ref.bigram_embedding). ids (B,S) int64; ``table`` has one more row
+    than buckets (the last serves a sequence's first token); ``last`` (slots,)
+    int32 carries each sequence's newest token and is advanced."""
+    if embed.is_cuda:
+        lib = _load()
+        B, S = ids.shape
+        assert ids.dtype == torch.int64 and ids.is_contiguous() and last.dtype == torch.int32
+        assert embed.dtype == table.dtype and embed.is_contiguous() and table.is_contiguous()
+        V, W = embed.shape
+        out = torch.empty(B, S, W, dtype=torch.float32, device=embed.device)
+        _check(lib.nx_bigram_embed(
+            _p(ids), _p(step.positions), _p(step.seq_ids), _p(step.nvalid), _p(embed), _p(table),
+            _is_bf16(embed), _p(last), ctypes.c_longlong(int(mul_prev)),
+            ctypes.c_longlong(int(mul_cur)), ctypes.c_longlong(table.shape[0] - 1), V, _p(out),
+            B, S, W, _stream()), "bigram_embedding")
+        return out
+    return ref.bigram_embedding(ids, embed, table, last, step.positions, step.seq_ids,
+                                mul_prev, mul_cur)
+
+
+def token_gate(z, ids, table, offset: int):
+    """gelu_tanh(z) times the token's channels [offset, offset + C) of ``table``
+    (vocab, >= offset + C). z (B,S,C) may be a column slice; ids (B,S) int64."""
+    C = z.shape[-1]
+    if z.is_cuda:
+        lib = _load()
+        assert ids.dtype == torch.int64 and ids.is_contiguous() and table.dtype == z.dtype
+        assert table.is_contiguous() and ids.numel() * C == z.numel()
+        out = torch.empty(z.shape, dtype=z.dtype, device=z.device)
+        _check(lib.nx_token_gate(_p(z), ctypes.c_long(_rows_view(z)), _p(ids), _p(table),
+                                 ctypes.c_long(table.stride(0)), int(offset), table.shape[0],
+                                 _is_bf16(z), _p(out), ctypes.c_long(ids.numel()), C, _stream()),
+               "token_gate")
+        return out
+    return ref.token_gate(z, ids, table, offset).to(z.dtype)

@@ -81,6 +81,11 @@ _REGISTRY: Dict[str, Tuple[str, str, str]] = {
         "TamilixInferenceConfig",
         "TamilixForCausalLM",
     ),
+    "risutar": (
+        "neuronx_distributed_inference_amd.models.risutar.modeling_risutar",
+        "RisutarInferenceConfig",
+        "RisutarForCausalLM",
+    ),
     "soputar": (
         "neuronx_distributed_inference_amd.models.soputar.modeling_soputar",
         "SoputarInferenceConfig",
