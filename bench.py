@@ -75,9 +75,9 @@ def parse_args():
                         "parallel, retention, routed experts; Tamilix: chunk-local slope "
                         "attention, windowed gated latent attention, identity-routed "
                         "experts) beside Llama at equal width/depth/ff/vocab")
-    p.add_argument("--hybrid-models", default="llama,nabelix,soputar,kuterax,tamilix",
-                   help="comma-separated subset of llama,nabelix,soputar,kuterax,tamilix "
-                        "for --hybrid")
+    p.add_argument("--hybrid-models", default="llama,nabelix,soputar,kuterax,tamilix,risutar",
+                   help="comma-separated subset of llama,nabelix,soputar,kuterax,tamilix,"
+                        "risutar for --hybrid")
     p.add_argument("--hybrid-sizes", default="2048,4096",
                    help="comma-separated layer widths for --hybrid")
     p.add_argument("--hybrid-layers", type=int, default=4)
@@ -119,6 +119,9 @@ def run_hybrid_bench(args):
     )
     from neuronx_distributed_inference_amd.models.tamilix.modeling_tamilix import (
         TamilixForCausalLM, TamilixInferenceConfig,
+    )
+    from neuronx_distributed_inference_amd.models.risutar.modeling_risutar import (
+        RisutarForCausalLM, RisutarInferenceConfig,
     )
 
     dtype = "bfloat16" if on_gpu else "float32"
@@ -231,6 +234,35 @@ def run_hybrid_bench(args):
                 neuron_config=ec, architecture="Tamilix", width=width, vocab=V,
                 layers=layers, norm={"eps": 1e-5}, embedding={"scale": 8.0})
             cls = TamilixForCausalLM
+        elif kind == "risutar":
+            # the design's layer mix, repeated to depth L: causal latent attention
+            # (512-wide latent + 64 rotated channels, query latent of 3/4 width)
+            # with a dense feed-forward, two gated linear attention layers and a
+            # latent layer that reads the first one's rows, all three with routed
+            # experts: four of sixteen of ff/8 plus a shared expert of ff/2
+            moe = {"kind": "moe", "expert": {"ff": ff // 8}, "shared": {"ff": ff // 2},
+                   "router": {"experts": 16, "top": 4}}
+            lat = {"heads": H, "dim": 128, "rot_dim": 64, "vdim": 128,
+                   "kv_rank": min(512, width // 4), "q_rank": width * 3 // 4,
+                   "scale": 192 ** -0.5, "rot": {"base": 10000.0, "dims": 64}}
+            gla = {"heads": H, "dim": 128, "vdim": 128, "tau": 16.0, "decay_rank": 16}
+            quad = [
+                {"type": "latent_attention", "mixer": lat, "mlp": {"kind": "dense", "ff": ff}},
+                {"type": "gla", "mixer": gla, "mlp": moe},
+                {"type": "gla", "mixer": gla, "mlp": moe},
+                {"type": "latent_attention", "mixer": dict(lat, kv_from=0), "mlp": moe},
+            ]
+            layers = []
+            for i in range(L):
+                lc = json.loads(json.dumps(quad[i % 4]))
+                if "kv_from" in lc["mixer"]:
+                    lc["mixer"]["kv_from"] = i - 3
+                layers.append(lc)
+            cfg = RisutarInferenceConfig(
+                neuron_config=ec, architecture="Risutar", width=width, vocab=V, layers=layers,
+                embedding={"bigram": {"buckets": 65536, "mul_prev": 40503, "mul_cur": 9973}},
+                token_side={"dim": 64}, postln_alpha=(2.0 * L) ** 0.25, norm={"eps": 1e-5})
+            cls = RisutarForCausalLM
         else:
             layer = {"type": "parallel", "mlp": {"kind": "dense", "ff": ff}, "mixer": {
                 "left": {"heads": H, "kv_heads": G, "dim": 128, "vdim": 128,
@@ -250,15 +282,15 @@ def run_hybrid_bench(args):
         else:
             m = cls(cfg).eval()
         with torch.no_grad():
-            for p in m.parameters():
-                if p.dim() >= 2 and p.requires_grad:   # caches/state do not
+            for n, p in m.named_parameters():
+                if p.dim() >= 2 and ".kv_mgr." not in n:   # not the caches and state
                     p.normal_(0, 0.02)
         m.reset()
         m.enable_submodels()
         return m
 
     for width in [int(x) for x in args.hybrid_sizes.split(",")]:
-        for kind in [k for k in ("llama", "nabelix", "soputar", "kuterax", "tamilix")
+        for kind in [k for k in ("llama", "nabelix", "soputar", "kuterax", "tamilix", "risutar")
                      if k in args.hybrid_models.split(",")]:
             with torch.inference_mode():
                 # ---- prefill: one prompt, three timed repetitions

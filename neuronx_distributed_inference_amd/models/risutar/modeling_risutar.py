@@ -191,6 +191,19 @@ def _fill_from_shapes(lc: dict, shape):
 
 
 # ----------------------------------------------------------------- mixers
+def _padded(splits: List[int]) -> List[int]:
+    """Column widths of a fused projection, completed to a multiple of 8 (rows
+    of its output then start on 16-byte boundaries in either dtype)."""
+    pad = -sum(splits) % 8
+    return splits + [pad] if pad else splits
+
+
+def _stack(parts: List[torch.Tensor]) -> torch.Tensor:
+    """Fused projection weight with the zero rows of :func:`_padded`."""
+    pad = -sum(p.shape[0] for p in parts) % 8
+    return torch.cat(parts + [parts[0].new_zeros(pad, parts[0].shape[1])], dim=0)
+
+
 class RisutarLatentMixer(nn.Module):
     def __init__(self, width: int, mc: dict, eps: float, dtype: torch.dtype):
         super().__init__()
@@ -204,7 +217,7 @@ class RisutarLatentMixer(nn.Module):
         # one GEMM for everything that reads the mixer's input: the query
         # latent, the head gates and (unless the rows are another layer's) the
         # key/value latent with the rotated key part
-        self.splits = [Q] + ([C + R] if self.source is None else []) + [H]
+        self.splits = _padded([Q] + ([C + R] if self.source is None else []) + [H])
         self.in_proj = ColumnParallelLinear(width, sum(self.splits), dtype=dtype, tp_degree=1)
         self.q_norm = StreamRMSNorm(Q, eps=eps, out_dtype=dtype)
         self.q_up = ColumnParallelLinear(Q, H * (D + R), dtype=dtype, tp_degree=1)
@@ -218,15 +231,15 @@ class RisutarLatentMixer(nn.Module):
 
     def forward(self, h, kv_mgr, run_idx: int, step):
         parts = torch.split(self.in_proj(h), self.splits, dim=-1)
-        dkv = parts[1] if self.source is None else None
+        dkv, gate = (parts[1], parts[2]) if self.source is None else (None, parts[1])
         q = self.q_up(self.q_norm(parts[0]))
-        return self.o_proj(self.core(q, dkv, kv_mgr, run_idx, step, gate=parts[-1]))
+        return self.o_proj(self.core(q, dkv, kv_mgr, run_idx, step, gate=gate))
 
     @staticmethod
     def convert(sd, s, d, w, f, out, mc):
         own = mc.get("kv_from") is None
-        out[d + "in_proj.weight"] = torch.cat(
-            [w(s + "dq")] + ([w(s + "dkv")] if own else []) + [w(s + "g")], dim=0)
+        out[d + "in_proj.weight"] = _stack(
+            [w(s + "dq")] + ([w(s + "dkv")] if own else []) + [w(s + "g")])
         out[d + "q_norm.weight"] = f(s + "dq.norm")
         out[d + "q_up.weight"] = w(s + "uq")
         if own:
@@ -247,7 +260,7 @@ class RisutarLinearMixer(nn.Module):
         self.core = GatedLinearAttention(H, D, Dv, mc["tau"], r, eps, dtype)
         # one GEMM for everything that reads the mixer's input: q, k, v, the
         # output gate, the first stage of the decay projection
-        self.splits = [H * D, H * D, H * Dv, H * Dv, r]
+        self.splits = _padded([H * D, H * D, H * Dv, H * Dv, r])
         self.in_proj = ColumnParallelLinear(width, sum(self.splits), dtype=dtype, tp_degree=1)
         self.o_proj = RowParallelLinear(H * Dv, width, dtype=dtype, tp_degree=1)
 
@@ -258,13 +271,13 @@ class RisutarLinearMixer(nn.Module):
         return self.core.state_shapes()
 
     def forward(self, h, kv_mgr, run_idx: int, step):
-        q, k, v, g, a = torch.split(self.in_proj(h), self.splits, dim=-1)
+        q, k, v, g, a = torch.split(self.in_proj(h), self.splits, dim=-1)[:5]
         return self.o_proj(self.core(q, k, v, g, a, kv_mgr.state, f"run{run_idx}", step))
 
     @staticmethod
     def convert(sd, s, d, w, f, out, mc):
-        out[d + "in_proj.weight"] = torch.cat(
-            [w(s + "q"), w(s + "k"), w(s + "v"), w(s + "g"), w(s + "a1")], dim=0)
+        out[d + "in_proj.weight"] = _stack(
+            [w(s + "q"), w(s + "k"), w(s + "v"), w(s + "g"), w(s + "a1")])
         out[d + "core.decay_up.weight"] = w(s + "a2")
         out[d + "core.decay_bias"] = f(s + "a2.b")
         out[d + "core.norm_weight"] = f(s + "norm")

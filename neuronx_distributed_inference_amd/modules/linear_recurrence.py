@@ -240,9 +240,8 @@ class GatedLinearAttention(nn.Module):
         """q, k (B,S,H*dim), v, gate (B,S,H*vdim), decay_low (B,S,rank): raw
         projections, column slices of one GEMM output are fine. Returns
         (B,S,H*vdim) in the gate's dtype."""
-        o = seqmix.decay_scan(q, k, v, states.get(key + ".mem"), step, self.dim, self.vdim,
-                              channel_logits=self.decay_up(decay_low),
-                              channel_bias=self.decay_bias, tau=self.tau,
-                              k_scale=self.dim ** -0.5)
-        return seqmix.group_gated_norm(o, gate, self.norm_weight, self.eps, self.num_heads,
-                                       gate_first=False, out_dtype=gate.dtype)
+        log_decay = seqmix.low_rank_decay(decay_low, self.decay_up.weight, self.decay_bias,
+                                          self.tau)
+        return seqmix.gated_linear_attention(
+            q, k, v, log_decay, gate, self.norm_weight, self.eps, states.get(key + ".mem"), step,
+            self.dim, self.vdim, k_scale=self.dim ** -0.5)

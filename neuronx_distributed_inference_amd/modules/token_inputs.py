@@ -59,5 +59,5 @@ class TokenSideInput(nn.Module):
                 step: seqmix.StepLayout, copy_dtype=None):
         """``x`` the fp32 stream (updated in place), ``h`` the same in the GEMM
         input dtype. Returns the new stream in ``copy_dtype`` (None: no copy)."""
-        g = seqmix.token_gate(self.gate(h), step.tokens, table, self.offset)
+        g = seqmix.token_gate_proj(h, self.gate.weight, step.tokens, table, self.offset)
         return self.norm.add_into(x, self.proj(g), copy_dtype)

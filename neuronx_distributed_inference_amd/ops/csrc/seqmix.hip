@@ -1930,9 +1930,7 @@ head_norm_rope_kernel(const TIn* __restrict__ x, long xt, long xh, TOut* __restr
 // global loads are coalesced and the serial loop reads only LDS.
 // Decay: selective (dt projection + dt_bias, a_log: w = softplus(dt + bias),
 // a = exp(-exp(a_log) w)) or fixed per head (head_decay: a = decay, w = 1). CH takes
-// `dt` (H*D wide) as decay logits, a = sigmoid(dt + dt_bias)^inv_tau (steps of few
-// tokens), or, with dt_bias = null, as the decays themselves, computed once per
-// token by channel_decay_kernel instead of once per value-channel block.
+// `dt` (H*D wide, fp32) as the decays' logarithms.
 //
 // Long rows with few workgroups are cut into `nseg` segments of `seglen`
 // tokens that run side by side; the recurrence is linear in the state, so
@@ -1946,24 +1944,6 @@ head_norm_rope_kernel(const TIn* __restrict__ x, long xt, long xh, TOut* __restr
 // MODE 0 is the plain single pass (decode steps, short portions, full batches).
 #define DS_TC 16
 
-// sigmoid(z)^inv_tau, through the logarithm: no underflow for very negative z
-DEV float channel_decay_(float z, float inv_tau) {
-    return expf((fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau);
-}
-
-template <typename T>
-__global__ void channel_decay_kernel(const T* __restrict__ z, long zs,
-                                     const float* __restrict__ bias, float inv_tau,
-                                     float* __restrict__ out, long rows, int C) {
-    const long total = rows * C;
-    for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < total;
-         i += (long)gridDim.x * blockDim.x) {
-        const long t = i / C;
-        const int c = i % C;
-        out[i] = channel_decay_(ldf<T>(z + t * zs + c) + bias[c], inv_tau);
-    }
-}
-
 template <typename T, typename TD, int R, int MODE, bool CH>
 __global__ void __launch_bounds__(256)
 decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, long ks,
@@ -1974,7 +1954,7 @@ decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, lon
                   const int* __restrict__ pos, const int* __restrict__ seq,
                   const int* __restrict__ nvalid, float* __restrict__ out, int S, int H, int G,
                   int D, int Dv, float* __restrict__ ws, float* __restrict__ wdec, int nseg,
-                  int seglen, float inv_tau) {
+                  int seglen) {
     constexpr int DP = 16 * R;
     __shared__ __attribute__((aligned(16))) float sd[CH ? DS_TC : 1][CH ? DP : 4];
     __shared__ __attribute__((aligned(16))) float sq[MODE == 1 ? 1 : DS_TC][DP], sk[DS_TC][DP];
@@ -2034,12 +2014,8 @@ decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, lon
             if (MODE != 1) sq[tt][d] = qv;
             sk[tt][d] = kv;
             if constexpr (CH) {
-                float a = 0.f;
-                if (tt < cnt && d < D) {
-                    a = ldf<TD>(dt + ((long)b * S + t0 + tt) * dts + (long)h * D + d);
-                    if (dt_bias) a = channel_decay_(a + dt_bias[(long)h * D + d], inv_tau);
-                }
-                sd[tt][d] = a;
+                sd[tt][d] = (tt < cnt && d < D)
+                    ? expf(ldf<TD>(dt + ((long)b * S + t0 + tt) * dts + (long)h * D + d)) : 0.f;
             }
         }
         {
@@ -2173,6 +2149,454 @@ __global__ void decay_scan_link_kernel(float* __restrict__ ws, const float* __re
             const float end = *p;
             *p = s;
             s = wdec[(((long)b * nseg + c) * H + h) * dch + (dch > 1 ? e % dch : 0)] * s + end;
+        }
+    }
+}
+
+// ------------------------------------------------- low-rank channel decays
+// log decay of a key channel: log(sigmoid(low[t] . w[c] + bias[c])) * inv_tau, all
+// fp32 (a very negative logit does not underflow). A thread owns one channel for
+// LRD_T tokens, whose low-rank rows sit in LDS.
+#define LRD_T 16
+#define LRD_R 64
+
+template <typename T>
+__global__ void __launch_bounds__(256)
+low_rank_decay_kernel(const T* __restrict__ low, long ls, const T* __restrict__ w, int vec,
+                      const float* __restrict__ bias, float inv_tau, float* __restrict__ out,
+                      long rows, int C, int rank) {
+    __shared__ float sl[LRD_T][LRD_R];
+    const int c = blockIdx.x * 256 + threadIdx.x;
+    for (long t0 = (long)blockIdx.y * LRD_T; t0 < rows; t0 += (long)gridDim.y * LRD_T) {
+        float acc[LRD_T];
+        const float b0 = c < C ? bias[c] : 0.f;
+#pragma unroll
+        for (int t = 0; t < LRD_T; ++t) acc[t] = b0;
+        for (int r0 = 0; r0 < rank; r0 += LRD_R) {
+            const int rn = min(LRD_R, rank - r0);
+            __syncthreads();
+            for (int i = threadIdx.x; i < LRD_T * LRD_R; i += 256) {
+                const int t = i / LRD_R, r = i % LRD_R;
+                sl[t][r] = (t0 + t < rows && r < rn) ? ldf<T>(low + (t0 + t) * ls + r0 + r) : 0.f;
+            }
+            __syncthreads();
+            if (c < C) {
+                for (int r = 0; r < rn; r += 8) {
+                    float wv[8];
+                    const T* wp = w + (long)c * rank + r0 + r;
+                    if (vec) {
+                        load8<T>(wp, wv);
+                    } else {
+#pragma unroll
+                        for (int e = 0; e < 8; ++e) wv[e] = r + e < rn ? ldf<T>(wp + e) : 0.f;
+                    }
+#pragma unroll
+                    for (int t = 0; t < LRD_T; ++t)
+#pragma unroll
+                        for (int e = 0; e < 8; ++e) acc[t] += wv[e] * sl[t][r + e];
+                }
+            }
+        }
+        if (c < C) {
+#pragma unroll
+            for (int t = 0; t < LRD_T; ++t)
+                if (t0 + t < rows) {
+                    const float z = acc[t];
+                    out[(t0 + t) * C + c] = (fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau;
+                }
+        }
+    }
+}
+
+// --------------------------- channel-decay recurrence in chunks, matrix cores
+// The recurrence of decay_scan_kernel<CH> for rows of many tokens, bf16 inputs, cut
+// into chunks of 64 tokens (4 sub-blocks of 16). With G the running sum of log
+// decays, token s reaches token t >= s through exp(G_t - G_s) per key channel:
+//   gla_chunk_state_kernel  E_c = sum_s k_s exp(G_end - G_s) v_s^T and exp(G_end)
+//                           of every chunk on its own;
+//   gla_chunk_link_kernel   serially over the chunks: start state of each (in place
+//                           over E_c) and the carried state;
+//   gla_chunk_out_kernel    o_t = (q_t exp(G_t)) S_c + sum_{s <= t} A_ts v_s, then the
+//                           per-head RMS norm, its weight and the silu gate.
+// Every exponent is taken relative to a sub-block's edge between the two tokens, so
+// it is never positive: no overflow, whatever the decays. A_ts of two different
+// sub-blocks is a product of two such factors (matrix cores); inside a sub-block it
+// is summed directly in fp32. fp32 operands of the matrix cores are split into bf16
+// terms: three for the keys that enter the state (24 bits), two elsewhere (16 bits);
+// accumulation and state are fp32.
+#define GC_N 64
+#define GC_VS (GC_N + 8)
+
+DEV void split_bf16_(float x, __bf16& hi, __bf16& lo) {
+    hi = (__bf16)x;
+    lo = (__bf16)(x - (float)hi);
+}
+
+// V^T of a chunk: (NT*16 channels, GC_VS) with zeros past the last token / channel
+template <int NT>
+DEV void gc_stage_vt_(const bf16* __restrict__ v, long vs, long tok0, int cnt, int Dv,
+                      uint16_t* __restrict__ vt, int tid) {
+    for (int c = tid; c < GC_N * NT * 2; c += 256) {
+        const int m = c % GC_N, part = c / GC_N;
+        uint4 raw = make_uint4(0, 0, 0, 0);
+        if (m < cnt && part * 8 < Dv)
+            raw = *reinterpret_cast<const uint4*>(v + (tok0 + m) * vs + part * 8);
+        const uint32_t u[4] = {raw.x, raw.y, raw.z, raw.w};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            vt[(part * 8 + 2 * e) * GC_VS + m] = (uint16_t)(u[e] & 0xffffu);
+            vt[(part * 8 + 2 * e + 1) * GC_VS + m] = (uint16_t)(u[e] >> 16);
+        }
+    }
+}
+
+template <int DP, int NT>
+__global__ void __launch_bounds__(256)
+gla_chunk_state_kernel(const bf16* __restrict__ k, long ks, const bf16* __restrict__ v, long vs,
+                       const float* __restrict__ ld, float k_scale, const int* __restrict__ pos,
+                       const int* __restrict__ seq, const int* __restrict__ nvalid,
+                       float* __restrict__ ws, float* __restrict__ wdec, int S, int H, int D,
+                       int Dv, int nc) {
+    __shared__ __attribute__((aligned(16))) uint16_t kt[3][DP * GC_VS];
+    __shared__ __attribute__((aligned(16))) uint16_t vt[NT * 16 * GC_VS];
+    __shared__ float tot[4][DP];
+    const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+    const int lr = lane & 15, lg = lane >> 4;
+    const int c = blockIdx.x % nc, d0 = blockIdx.x / nc * DP, h = blockIdx.y, b = blockIdx.z;
+    const int n = seq[b] < 0 ? 0 : nvalid[b];
+    const int cnt = min(GC_N, n - c * GC_N);
+    if (cnt <= 0) return;                                 // uniform
+    const long tok0 = (long)b * S + c * GC_N;
+    const int Dn = min(DP, D - d0);                       // this workgroup's key channels
+    const float* lp = ld + (long)h * D + d0;
+    const bf16* kp = k + (long)h * D + d0;
+    const long lst = (long)H * D;
+    gc_stage_vt_<NT>(v + (long)h * Dv, vs, tok0, cnt, Dv, vt, tid);
+    // one (channel, sub-block) task per thread and turn: its 16 log decays
+    for (int task = tid; task < 4 * DP; task += 256) {
+        const int d = task % DP, sb = task / DP;
+        float t = 0.f;
+        for (int i = 0; i < 16; ++i) {
+            const int m = sb * 16 + i;
+            if (m < cnt && d < Dn) t += lp[(tok0 + m) * lst + d];
+        }
+        tot[sb][d] = t;
+    }
+    __syncthreads();
+    for (int task = tid; task < 4 * DP; task += 256) {
+        const int d = task % DP, sb = task / DP;
+        float after = 0.f;                                // decays of the later tokens
+        for (int m = sb + 1; m < 4; ++m) after += tot[m][d];
+        float g[16], kv[16];
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            const int m = sb * 16 + i;
+            const bool ok = m < cnt && d < Dn;
+            g[i] = ok ? lp[(tok0 + m) * lst + d] : 0.f;
+            kv[i] = ok ? ldf<bf16>(kp + (tok0 + m) * ks + d) * k_scale : 0.f;
+        }
+#pragma unroll
+        for (int i = 15; i >= 0; --i) {
+            const float x = kv[i] * expf(after);
+            after += g[i];
+            const __bf16 a0 = (__bf16)x;
+            const float r1 = x - (float)a0;
+            const __bf16 a1 = (__bf16)r1;
+            const __bf16 a2 = (__bf16)(r1 - (float)a1);
+            const int at = d * GC_VS + sb * 16 + i;
+            kt[0][at] = __builtin_bit_cast(uint16_t, a0);
+            kt[1][at] = __builtin_bit_cast(uint16_t, a1);
+            kt[2][at] = __builtin_bit_cast(uint16_t, a2);
+        }
+        if (sb == 0 && d < Dn) wdec[(((long)b * nc + c) * H + h) * D + d0 + d] = expf(after);
+    }
+    __syncthreads();
+    float* wp = ws + (((long)b * nc + c) * H + h) * (long)Dv * D + d0;
+    constexpr int DT = DP / 16;
+    for (int tile = wv; tile < DT * NT; tile += 4) {
+        const int dt = tile % DT, nt = tile / DT;
+        if (nt * 16 >= Dv || dt * 16 >= Dn) continue;
+        f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk) {
+            const bf16x8_t va = *reinterpret_cast<const bf16x8_t*>(
+                vt + (nt * 16 + lr) * GC_VS + kk * 32 + lg * 8);
+#pragma unroll
+            for (int e = 2; e >= 0; --e) {                // small terms first
+                const bf16x8_t kb = *reinterpret_cast<const bf16x8_t*>(
+                    kt[e] + (dt * 16 + lr) * GC_VS + kk * 32 + lg * 8);
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va, kb, acc, 0, 0, 0);
+            }
+        }
+        const int d = dt * 16 + lr;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int nn = nt * 16 + lg * 4 + r;
+            if (nn < Dv && d < Dn) wp[(long)nn * D + d] = acc[r];
+        }
+    }
+}
+
+// start states of the chunks, in place over their contributions, and the carried
+// state; eight chunks' loads are in flight at a time
+__global__ void __launch_bounds__(256)
+gla_chunk_link_kernel(float* __restrict__ ws, const float* __restrict__ wdec,
+                      float* __restrict__ state, const int* __restrict__ pos,
+                      const int* __restrict__ seq, const int* __restrict__ nvalid, int B, int S,
+                      int H, int D, long per_head, int nc) {
+    const long total = (long)B * H * per_head;
+    for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < total;
+         i += (long)gridDim.x * blockDim.x) {
+        const long e = i % per_head;
+        const int h = (i / per_head) % H, b = i / (per_head * H), d = e % D;
+        const int slot = seq[b], n = slot < 0 ? 0 : nvalid[b];
+        if (n <= 0) continue;
+        const int chunks = (n + GC_N - 1) / GC_N;
+        float* sp = state + ((long)slot * H + h) * per_head + e;
+        float s = pos[(long)b * S] > 0 ? *sp : 0.f;
+        float* wp = ws + ((long)b * nc * H + h) * per_head + e;
+        const float* dp = wdec + ((long)b * nc * H + h) * D + d;
+        const long wst = (long)H * per_head, dst = (long)H * D;
+        for (int c0 = 0; c0 < chunks; c0 += 8) {
+            float en[8], dc[8];
+#pragma unroll
+            for (int j = 0; j < 8; ++j)
+                if (c0 + j < chunks) { en[j] = wp[(c0 + j) * wst]; dc[j] = dp[(c0 + j) * dst]; }
+#pragma unroll
+            for (int j = 0; j < 8; ++j)
+                if (c0 + j < chunks) { wp[(c0 + j) * wst] = s; s = dc[j] * s + en[j]; }
+        }
+        *sp = s;
+    }
+}
+
+template <int DP, int NT>
+__global__ void __launch_bounds__(256)
+gla_chunk_out_kernel(const bf16* __restrict__ q, long qs, const bf16* __restrict__ k, long ks,
+                     const bf16* __restrict__ v, long vs, const float* __restrict__ ld,
+                     float k_scale, const bf16* __restrict__ gate, long gs,
+                     const float* __restrict__ nw, float eps, const int* __restrict__ seq,
+                     const int* __restrict__ nvalid, const float* __restrict__ ws,
+                     bf16* __restrict__ out, int S, int H, int D, int Dv, int nc) {
+    constexpr int KS = DP + 8, LS = DP + 4, KK = DP / 32;
+    extern __shared__ __attribute__((aligned(16))) float smem[];
+    float* ll = smem;                                     // GC_N * LS: running log decay in a sub-block
+    float (*tot)[DP] = reinterpret_cast<float (*)[DP]>(ll + GC_N * LS);         // 4 x DP
+    uint16_t* kl = reinterpret_cast<uint16_t*>(ll + GC_N * LS + 4 * DP);        // GC_N * KS
+    uint16_t* vt = kl + GC_N * KS;                                              // NT * 16 * GC_VS
+    const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;    // wave = sub-block
+    const int lr = lane & 15, lg = lane >> 4;
+    const int c = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+    const int n = seq[b] < 0 ? 0 : nvalid[b];
+    const int cnt = min(GC_N, n - c * GC_N);
+    if (cnt <= 0) return;                                 // uniform
+    const long tok0 = (long)b * S + c * GC_N;
+    const bool tv = w * 16 + lr < cnt;
+    // this lane's query row (token 16 w + lr), channels kk*32 + lg*8 ..
+    uint4 qr[KK];
+#pragma unroll
+    for (int kk = 0; kk < KK; ++kk) {
+        const int d = kk * 32 + lg * 8;
+        qr[kk] = make_uint4(0, 0, 0, 0);
+        if (tv && d < D)
+            qr[kk] = *reinterpret_cast<const uint4*>(q + (tok0 + w * 16 + lr) * qs + (long)h * D + d);
+    }
+    gc_stage_vt_<NT>(v + (long)h * Dv, vs, tok0, cnt, Dv, vt, tid);
+    for (int i = tid; i < GC_N * (DP / 8); i += 256) {
+        const int m = i / (DP / 8), part = i % (DP / 8);
+        uint4 raw = make_uint4(0, 0, 0, 0);
+        if (m < cnt && part * 8 < D)
+            raw = *reinterpret_cast<const uint4*>(k + (tok0 + m) * ks + (long)h * D + part * 8);
+        *reinterpret_cast<uint4*>(kl + m * KS + part * 8) = raw;
+    }
+    for (int task = tid; task < 4 * DP; task += 256) {
+        const int d = task % DP, sb = task / DP;
+        float g[16];
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            const int m = sb * 16 + i;
+            g[i] = (m < cnt && d < D) ? ld[(tok0 + m) * (long)(H * D) + (long)h * D + d] : 0.f;
+        }
+        float t = 0.f;
+#pragma unroll
+        for (int i = 0; i < 16; ++i) { t += g[i]; ll[(sb * 16 + i) * LS + d] = t; }
+        tot[sb][d] = t;
+    }
+    __syncthreads();
+    if (w * 16 >= cnt) return;                            // no barriers below
+    float qf[KK][8], lt[KK][8], pre[KK][8];               // q, L_t, log decays of earlier sub-blocks
+#pragma unroll
+    for (int kk = 0; kk < KK; ++kk) {
+        const int d = kk * 32 + lg * 8;
+        const uint32_t u[4] = {qr[kk].x, qr[kk].y, qr[kk].z, qr[kk].w};
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            qf[kk][e] = __uint_as_float(e & 1 ? u[e / 2] & 0xffff0000u : u[e / 2] << 16);
+            lt[kk][e] = ll[(w * 16 + lr) * LS + d + e];
+            float pr = 0.f;
+            for (int m = 0; m < w; ++m) pr += tot[m][d + e];
+            pre[kk][e] = pr;
+        }
+    }
+    f32x4_t o[NT];
+#pragma unroll
+    for (int nt = 0; nt < NT; ++nt) o[nt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    // ---- (q exp(G_t)) S: S rows (value channel lr of the tile) from memory
+    {
+        const float* sp = ws + (((long)b * nc + c) * H + h) * (long)Dv * D;
+#pragma unroll
+        for (int kk = 0; kk < KK; ++kk) {
+            const int d = kk * 32 + lg * 8;
+            bf16x8_t qh, ql;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                __bf16 hi, lo;
+                split_bf16_(qf[kk][e] * __expf(pre[kk][e] + lt[kk][e]), hi, lo);
+                qh[e] = hi; ql[e] = lo;
+            }
+#pragma unroll
+            for (int nt = 0; nt < NT; ++nt) {
+                const int nn = nt * 16 + lr;
+                float sv[8];
+#pragma unroll
+                for (int e = 0; e < 8; ++e) sv[e] = 0.f;
+                if (nn < Dv && d < D) load8<float>(sp + (long)nn * D + d, sv);
+                bf16x8_t sh, sl;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) {
+                    __bf16 hi, lo;
+                    split_bf16_(sv[e], hi, lo);
+                    sh[e] = hi; sl[e] = lo;
+                }
+                o[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ql, sh, o[nt], 0, 0, 0);
+                o[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qh, sl, o[nt], 0, 0, 0);
+                o[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qh, sh, o[nt], 0, 0, 0);
+            }
+        }
+    }
+    // ---- A^T: lane gets keys 4*lg + r of sub-block j for query lr
+    float sc[4][4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) sc[j][r] = 0.f;
+    {   // own sub-block: exp(L_t - L_s) directly, channels split over the four lane groups
+        float part[16];
+#pragma unroll
+        for (int si = 0; si < 16; ++si) {
+            float a = 0.f;
+#pragma unroll
+            for (int kk = 0; kk < KK; ++kk) {
+                const int d = kk * 32 + lg * 8;
+                float kv[8], lv[8];
+                load8<bf16>(reinterpret_cast<const bf16*>(kl) + (w * 16 + si) * KS + d, kv);
+                load8<float>(ll + (w * 16 + si) * LS + d, lv);
+#pragma unroll
+                for (int e = 0; e < 8; ++e)
+                    a += qf[kk][e] * kv[e] * __expf(fminf(lt[kk][e] - lv[e], 0.f));
+            }
+            part[si] = a;
+        }
+#pragma unroll
+        for (int si = 0; si < 16; ++si) {
+            part[si] += __shfl_xor(part[si], 16, WAVE);
+            part[si] += __shfl_xor(part[si], 32, WAVE);
+        }
+        float own[4];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const float x01 = lg & 1 ? part[4 + r] : part[r];
+            const float x23 = lg & 1 ? part[12 + r] : part[8 + r];
+            own[r] = lg * 4 + r <= lr ? (lg & 2 ? x23 : x01) : 0.f;
+        }
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+            if (j == w)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) sc[j][r] = own[r] * k_scale;
+    }
+    // earlier sub-blocks: q exp(L_t) against k exp(sum between - ...)
+    if (w > 0) {
+        bf16x8_t qh[KK], ql[KK];
+        float btw[KK][8];                                 // log decays of the sub-blocks between
+#pragma unroll
+        for (int kk = 0; kk < KK; ++kk)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                __bf16 hi, lo;
+                split_bf16_(qf[kk][e] * __expf(lt[kk][e]), hi, lo);
+                qh[kk][e] = hi; ql[kk][e] = lo;
+                btw[kk][e] = 0.f;
+            }
+#pragma unroll
+        for (int j = 2; j >= 0; --j) {
+            if (j >= w) continue;                         // wave-uniform
+            f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int kk = 0; kk < KK; ++kk) {
+                const int d = kk * 32 + lg * 8;
+                float kv[8], lv[8], tv8[8];
+                load8<bf16>(reinterpret_cast<const bf16*>(kl) + (j * 16 + lr) * KS + d, kv);
+                load8<float>(ll + (j * 16 + lr) * LS + d, lv);
+                load8<float>(&tot[j][d], tv8);
+                bf16x8_t kh, klo;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) {
+                    __bf16 hi, lo;
+                    btw[kk][e] += tv8[e];                 // now from the start of j to the start of w
+                    split_bf16_(kv[e] * __expf(btw[kk][e] - lv[e]), hi, lo);
+                    kh[e] = hi; klo[e] = lo;
+                }
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(klo, qh[kk], acc, 0, 0, 0);
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kh, ql[kk], acc, 0, 0, 0);
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kh, qh[kk], acc, 0, 0, 0);
+            }
+#pragma unroll
+            for (int r = 0; r < 4; ++r) sc[j][r] = acc[r] * k_scale;
+        }
+    }
+    // ---- O += A V, two sub-blocks of keys at a time, A as hi + lo
+#pragma unroll
+    for (int pr = 0; pr < 2; ++pr) {
+        if (pr * 2 > w) continue;                         // wave-uniform
+        bf16x8_t ph, pl;
+#pragma unroll
+        for (int jj = 0; jj < 8; ++jj) {
+            __bf16 hi, lo;
+            split_bf16_(sc[pr * 2 + (jj >> 2)][jj & 3], hi, lo);
+            ph[jj] = hi; pl[jj] = lo;
+        }
+#pragma unroll
+        for (int nt = 0; nt < NT; ++nt) {
+            union { bf16x8_t v; uint2 h2[2]; } vb;
+            const uint16_t* vp = vt + (nt * 16 + lr) * GC_VS + pr * 32 + 4 * lg;
+            vb.h2[0] = *reinterpret_cast<const uint2*>(vp);
+            vb.h2[1] = *reinterpret_cast<const uint2*>(vp + 16);
+            o[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pl, vb.v, o[nt], 0, 0, 0);
+            o[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ph, vb.v, o[nt], 0, 0, 0);
+        }
+    }
+    // ---- norm over the head's channels (tiles x 16 lanes), weight, silu gate
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+        float ss = 0.f;
+#pragma unroll
+        for (int nt = 0; nt < NT; ++nt) ss += o[nt][r] * o[nt][r];   // channels past Dv are zero
+        ss += __shfl_xor(ss, 1, WAVE);
+        ss += __shfl_xor(ss, 2, WAVE);
+        ss += __shfl_xor(ss, 4, WAVE);
+        ss += __shfl_xor(ss, 8, WAVE);
+        const int t = w * 16 + lg * 4 + r;
+        if (t >= cnt) continue;
+        const float inv = 1.f / sqrtf(ss / Dv + eps);
+        const bf16* gp = gate + (tok0 + t) * gs + (long)h * Dv;
+        bf16* op = out + (tok0 + t) * (long)(H * Dv) + (long)h * Dv;
+#pragma unroll
+        for (int nt = 0; nt < NT; ++nt) {
+            const int nn = nt * 16 + lr;
+            if (nn >= Dv) continue;
+            const float gv = __bfloat162float(gp[nn]);
+            op[nn] = __float2bfloat16(o[nt][r] * inv * nw[nn] * (gv * sigmoidf_(gv)));
         }
     }
 }
@@ -2665,6 +3089,93 @@ __global__ void token_gate_kernel(const T* __restrict__ z, long zs,
     }
 }
 
+// The same with the gating projection z = h . wg^T inside: workgroup = 16 tokens x
+// 16 channels on the matrix cores, the product's inner dimension split over 8 waves
+// and summed through LDS.
+__global__ void __launch_bounds__(512)
+token_gate_proj_kernel(const bf16* __restrict__ x, long xs, const bf16* __restrict__ wg, int K,
+                       const long long* __restrict__ ids, const bf16* __restrict__ table, long ts,
+                       int off, int vocab, bf16* __restrict__ out, long rows, int C) {
+    __shared__ float red[8][256];
+    const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+    const int lr = lane & 15, lg = lane >> 4;
+    const long t0 = (long)blockIdx.y * 16;
+    const int n0 = blockIdx.x * 16;
+    const bool tok = t0 + lr < rows, ch = n0 + lr < C;
+    const bf16* xp = x + (tok ? t0 + lr : 0) * xs + lg * 8;
+    const bf16* wp = wg + (long)(ch ? n0 + lr : 0) * K + lg * 8;
+    f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    for (int k0 = wv * 32; k0 < K; k0 += 8 * 32) {
+        uint4 xa = make_uint4(0, 0, 0, 0), wa = make_uint4(0, 0, 0, 0);
+        if (k0 + lg * 8 < K) {
+            if (tok) xa = *reinterpret_cast<const uint4*>(xp + k0);
+            if (ch) wa = *reinterpret_cast<const uint4*>(wp + k0);
+        }
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+            __builtin_bit_cast(bf16x8_t, xa), __builtin_bit_cast(bf16x8_t, wa), acc, 0, 0, 0);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) red[wv][(lg * 4 + r) * 16 + lr] = acc[r];
+    __syncthreads();
+    if (tid < 256) {
+        const long t = t0 + tid / 16;
+        const int n = n0 + tid % 16;
+        if (t < rows && n < C) {
+            float z = 0.f;
+#pragma unroll
+            for (int i = 0; i < 8; ++i) z += red[i][tid];
+            const long long id = min(max(ids[t], 0ll), (long long)vocab - 1);
+            out[t * C + n] = __float2bfloat16(
+                gelu_tanh_(z) * __bfloat162float(table[id * ts + off + n]));
+        }
+    }
+}
+
+// ------------------------------------------------ one product per head, few tokens
+// out[t, h, n] = sum_k a[t, h, k] w[h, n, k] (both operands contiguous over k).
+// Workgroup = 16 output channels of a head x 64 tokens; its 4 waves split k and sum
+// through LDS, so every weight row is fetched once.
+__global__ void __launch_bounds__(256)
+head_product_kernel(const bf16* __restrict__ a, const bf16* __restrict__ w,
+                    bf16* __restrict__ out, int T, int H, int K, int N) {
+    __shared__ float red[4][4][256];
+    const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+    const int lr = lane & 15, lg = lane >> 4;
+    const int n0 = blockIdx.x * 16, h = blockIdx.y, t0 = blockIdx.z * 64;
+    const bool ch = n0 + lr < N;
+    const bf16* wp = w + ((long)h * N + (ch ? n0 + lr : 0)) * K + lg * 8;
+    f32x4_t acc[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+    for (int k0 = wv * 32; k0 < K; k0 += 4 * 32) {
+        const bool kin = k0 + lg * 8 < K;
+        uint4 wa = make_uint4(0, 0, 0, 0);
+        if (kin && ch) wa = *reinterpret_cast<const uint4*>(wp + k0);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int t = t0 + i * 16 + lr;
+            uint4 av = make_uint4(0, 0, 0, 0);
+            if (kin && t < T)
+                av = *reinterpret_cast<const uint4*>(a + ((long)t * H + h) * K + k0 + lg * 8);
+            acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                __builtin_bit_cast(bf16x8_t, av), __builtin_bit_cast(bf16x8_t, wa), acc[i], 0, 0, 0);
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) red[wv][i][(lg * 4 + r) * 16 + lr] = acc[i][r];
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int t = t0 + i * 16 + tid / 16, n = n0 + tid % 16;
+        if (t < T && n < N)
+            out[((long)t * H + h) * N + n] = __float2bfloat16(
+                red[0][i][tid] + red[1][i][tid] + red[2][i][tid] + red[3][i][tid]);
+    }
+}
+
 // ------------------------------------- residual sum of weighted, optionally normed terms
 // x[row] += sum_i f_i(y_i[row]) * w_i, f_i = RMS norm over the row or identity.
 // One workgroup per row; statistics fp32.
@@ -3127,12 +3638,12 @@ int nx_decay_scan(const void* q, long qs, const void* k, long ks, const void* v,
                   const float* a_log, const float* head_decay, float k_scale, const float* skip,
                   float* state, const int* pos, const int* seq, const int* nvalid, float* out,
                   int B, int S, int H, int G, int D, int Dv, float* ws, float* wdec, int nseg,
-                  int seglen, int channel, float inv_tau, hipStream_t st) {
+                  int seglen, int channel, hipStream_t st) {
     if ((long)B * S <= 0) return 0;
     if (D <= 0 || Dv <= 0 || G <= 0 || H % G != 0 || D > 256) return -1;
     if ((dt == nullptr) == (head_decay == nullptr)) return -2;
     if (dt && !channel && (!dt_bias || !a_log)) return -2;
-    if (channel && (!dt || a_log || skip)) return -2;
+    if (channel && (!dt || dt_bf16 || a_log || skip)) return -2;
     if (H > 65535 || B > 65535) return -3;
     // the kernel reads state rows 16 bytes at a time when dim % 4 == 0
     if (((uintptr_t)state % 16) != 0 || ((uintptr_t)ws % 16) != 0) return -5;
@@ -3143,15 +3654,16 @@ int nx_decay_scan(const void* q, long qs, const void* k, long ks, const void* v,
 #define DSK(T, TD, RV, MD, CHV) decay_scan_kernel<T, TD, RV, MD, CHV><<<grid, block, 0, st>>>( \
         (const T*)q, qs, (const T*)k, ks, (const T*)v, vs, (const TD*)dt, dts, dt_bias, a_log, \
         head_decay, k_scale, skip, state, pos, seq, nvalid, out, S, H, G, D, Dv, ws, wdec, nseg, \
-        seglen, inv_tau)
+        seglen)
 #define DSR(T, TD, MD, CHV) do { if (D <= 16) DSK(T, TD, 1, MD, CHV); \
         else if (D <= 32) DSK(T, TD, 2, MD, CHV); \
         else if (D <= 64) DSK(T, TD, 4, MD, CHV); else if (D <= 128) DSK(T, TD, 8, MD, CHV); \
         else DSK(T, TD, 16, MD, CHV); } while (0)
-#define DST(MD, CHV) do { \
-        if (in_bf16) { if (dt_bf16) DSR(bf16, bf16, MD, CHV); else DSR(bf16, float, MD, CHV); } \
-        else { if (dt_bf16) DSR(float, bf16, MD, CHV); else DSR(float, float, MD, CHV); } } while (0)
-#define DSC(MD) do { if (channel) DST(MD, true); else DST(MD, false); } while (0)
+#define DST(MD) do { \
+        if (in_bf16) { if (dt_bf16) DSR(bf16, bf16, MD, false); else DSR(bf16, float, MD, false); } \
+        else { if (dt_bf16) DSR(float, bf16, MD, false); else DSR(float, float, MD, false); } } while (0)
+#define DSC(MD) do { if (!channel) DST(MD); else if (in_bf16) DSR(bf16, float, MD, true); \
+        else DSR(float, float, MD, true); } while (0)
     if (nseg == 1) {
         DSC(0);
     } else {
@@ -3168,15 +3680,57 @@ int nx_decay_scan(const void* q, long qs, const void* k, long ks, const void* v,
     return (int)hipGetLastError();
 }
 
-int nx_channel_decay(const void* z, long zs, int z_bf16, const float* bias, float inv_tau,
-                     float* out, long rows, int C, hipStream_t st) {
+int nx_low_rank_decay(const void* low, long ls, const void* w, int is_bf16, const float* bias,
+                      float inv_tau, float* out, long rows, int C, int rank, hipStream_t st) {
     if (rows * C <= 0) return 0;
-    if (!bias) return -1;
-    dim3 grid(grid_for(rows * C, 256)), block(256);
-    if (z_bf16) channel_decay_kernel<bf16><<<grid, block, 0, st>>>(
-        (const bf16*)z, zs, bias, inv_tau, out, rows, C);
-    else channel_decay_kernel<float><<<grid, block, 0, st>>>(
-        (const float*)z, zs, bias, inv_tau, out, rows, C);
+    if (!bias || rank <= 0) return -1;
+    const int vec = (rank % 8) == 0 && ((uintptr_t)w % 16) == 0;
+    const long gy = (rows + LRD_T - 1) / LRD_T;
+    dim3 grid((C + 255) / 256, (unsigned)(gy > 32768 ? 32768 : gy)), block(256);
+    if (is_bf16) low_rank_decay_kernel<bf16><<<grid, block, 0, st>>>(
+        (const bf16*)low, ls, (const bf16*)w, vec, bias, inv_tau, out, rows, C, rank);
+    else low_rank_decay_kernel<float><<<grid, block, 0, st>>>(
+        (const float*)low, ls, (const float*)w, vec, bias, inv_tau, out, rows, C, rank);
+    return (int)hipGetLastError();
+}
+
+// chunked form of the channel-decay recurrence with the gated read-out norm fused:
+// bf16 q/k/v/gate/out, D and Dv multiples of 8 up to 128
+int nx_gla_chunked(const void* q, long qs, const void* k, long ks, const void* v, long vs,
+                   const float* ld, float k_scale, const void* gate, long gs, const float* nw,
+                   float eps, float* state, const int* pos, const int* seq, const int* nvalid,
+                   float* ws, float* wdec, void* out, int B, int S, int H, int D, int Dv,
+                   hipStream_t st) {
+    if ((long)B * S <= 0) return 0;
+    if (D <= 0 || Dv <= 0 || D > 128 || Dv > 128 || (D % 8) || (Dv % 8)) return -1;
+    if ((qs % 8) || (ks % 8) || (vs % 8) || ((uintptr_t)q % 16) || ((uintptr_t)k % 16) ||
+        ((uintptr_t)v % 16) || ((uintptr_t)ws % 16) || !gate || !nw) return -2;
+    const int nc = (S + GC_N - 1) / GC_N;
+    if (H > 65535 || B > 65535) return -3;
+    dim3 grid(nc, H, B), block(256);
+#define GC(DPV, NT) do { \
+        constexpr int DPB = DPV < 64 ? DPV : 64; \
+        const size_t lsh = (size_t)(GC_N * (DPV + 4) + 4 * DPV) * 4 + \
+                           (size_t)(GC_N * (DPV + 8) + NT * 16 * GC_VS) * 2; \
+        static bool attr_set = false; \
+        if (!attr_set) { \
+            if (hipFuncSetAttribute((const void*)gla_chunk_out_kernel<DPV, NT>, \
+                    hipFuncAttributeMaxDynamicSharedMemorySize, (int)lsh) != hipSuccess) return -5; \
+            attr_set = true; \
+        } \
+        dim3 gst(nc * ((D + DPB - 1) / DPB), H, B); \
+        gla_chunk_state_kernel<DPB, NT><<<gst, block, 0, st>>>( \
+            (const bf16*)k, ks, (const bf16*)v, vs, ld, k_scale, pos, seq, nvalid, ws, wdec, S, H, \
+            D, Dv, nc); \
+        gla_chunk_link_kernel<<<grid_for((long)B * H * Dv * D, 256), 256, 0, st>>>( \
+            ws, wdec, state, pos, seq, nvalid, B, S, H, D, (long)Dv * D, nc); \
+        gla_chunk_out_kernel<DPV, NT><<<grid, block, lsh, st>>>( \
+            (const bf16*)q, qs, (const bf16*)k, ks, (const bf16*)v, vs, ld, k_scale, \
+            (const bf16*)gate, gs, nw, eps, seq, nvalid, ws, (bf16*)out, S, H, D, Dv, nc); } while (0)
+#define GCN(DPV) do { if (Dv <= 64) GC(DPV, 4); else GC(DPV, 8); } while (0)
+    if (D <= 32) GCN(32); else if (D <= 64) GCN(64); else GCN(128);
+#undef GCN
+#undef GC
     return (int)hipGetLastError();
 }
 
@@ -3368,6 +3922,29 @@ int nx_token_gate(const void* z, long zs, const long long* ids, const void* tabl
         (const bf16*)z, zs, ids, (const bf16*)table, ts, off, vocab, (bf16*)out, rows, C);
     else token_gate_kernel<float><<<grid, block, 0, st>>>(
         (const float*)z, zs, ids, (const float*)table, ts, off, vocab, (float*)out, rows, C);
+    return (int)hipGetLastError();
+}
+
+int nx_token_gate_proj(const void* x, long xs, const void* wg, int K, const long long* ids,
+                       const void* table, long ts, int off, int vocab, void* out, long rows, int C,
+                       hipStream_t st) {
+    if (rows * C <= 0) return 0;
+    if (vocab <= 0 || off < 0 || (long)off + C > ts || K <= 0 || (K % 8) || (xs % 8) ||
+        ((uintptr_t)x % 16) || ((uintptr_t)wg % 16) || (rows + 15) / 16 > 65535) return -1;
+    dim3 grid((C + 15) / 16, (unsigned)((rows + 15) / 16)), block(512);
+    token_gate_proj_kernel<<<grid, block, 0, st>>>((const bf16*)x, xs, (const bf16*)wg, K, ids,
+                                                   (const bf16*)table, ts, off, vocab, (bf16*)out,
+                                                   rows, C);
+    return (int)hipGetLastError();
+}
+
+int nx_head_product(const void* a, const void* w, void* out, int T, int H, int K, int N,
+                    hipStream_t st) {
+    if ((long)T * H * N <= 0) return 0;
+    if (K <= 0 || (K % 8) || ((uintptr_t)a % 16) || ((uintptr_t)w % 16) || H > 65535) return -1;
+    dim3 grid((N + 15) / 16, H, (T + 63) / 64), block(256);
+    head_product_kernel<<<grid, block, 0, st>>>((const bf16*)a, (const bf16*)w, (bf16*)out, T, H,
+                                                K, N);
     return (int)hipGetLastError();
 }
 

@@ -490,15 +490,15 @@ def head_norm_rotate(x: torch.Tensor, positions: torch.Tensor, norm_weight, eps:
     return torch.cat([u * c - v * sn, v * c + u * sn, xf[..., 2 * half:]], dim=-1)
 
 
-def channel_decay(z, bias, tau: float):
-    """sigmoid(z + bias)^(1/tau), fp32, through the logarithm."""
-    return torch.exp(torch.nn.functional.logsigmoid(z.float() + bias.float()) / tau)
+def low_rank_decay(low, weight, bias, tau: float):
+    """log(sigmoid(low @ weight.T + bias)) / tau, fp32."""
+    z = torch.nn.functional.linear(low.float(), weight.float(), bias.float())
+    return torch.nn.functional.logsigmoid(z) / tau
 
 
 def decay_scan(q, k, v, state, positions, seq_ids, dim: int, vdim: int,
                dt=None, dt_bias=None, a_log=None, head_decay=None,
-               k_scale: float = 1.0, skip=None, channel_logits=None, channel_bias=None,
-               tau: float = 1.0):
+               k_scale: float = 1.0, skip=None, log_decay=None):
     """Linear recurrence with a decay per head and matrix state, carried in ``state`` (slots, H, vdim, dim) fp32 (stored transposed):
 
         S_t = a_t S_{t-1} + k_t (w_t v_t)^T ;  o_t = S_t^T q_t (+ skip_h v_t)
@@ -507,9 +507,8 @@ def decay_scan(q, k, v, state, positions, seq_ids, dim: int, vdim: int,
     ``dt_bias`` and ``a_log`` (H,): w_t = softplus(dt + dt_bias), a_t =
     exp(-exp(a_log) w_t) (selective state spaces: k = B, q = C, v = x); or
     ``head_decay`` (H,): a_t = head_decay, w_t = 1 (retention); or
-    ``channel_logits`` (B,S,H*dim) with ``channel_bias`` (H*dim,) and ``tau``:
-    a decay per head and KEY CHANNEL, S_t = diag(a_t) S_{t-1} + k_t v_t^T,
-    a_t = sigmoid(logits + bias)^(1/tau) (gated linear attention). q, k
+    ``log_decay`` (B,S,H*dim): a decay per head and KEY CHANNEL, S_t =
+    diag(exp(log_decay_t)) S_{t-1} + k_t v_t^T (gated linear attention). q, k
     (B,S,G*dim) are shared by H/G consecutive heads, v (B,S,H*vdim); k is
     multiplied by ``k_scale``. Returns fp32 (B,S,H*vdim)."""
     B, S = positions.shape
@@ -523,8 +522,8 @@ def decay_scan(q, k, v, state, positions, seq_ids, dim: int, vdim: int,
     if dt is not None:
         w = torch.nn.functional.softplus(dt.float() + dt_bias.float(), threshold=20.0)
         a = torch.exp(-torch.exp(a_log.float()) * w)
-    elif channel_logits is not None:
-        a = channel_decay(channel_logits, channel_bias, tau).reshape(B, S, H, D)
+    elif log_decay is not None:
+        a = torch.exp(log_decay.float()).reshape(B, S, H, D)
         w = torch.ones(B, S, H, dtype=torch.float32, device=v.device)
     else:
         a = head_decay.float().view(1, 1, H).expand(B, S, H)

@@ -392,10 +392,19 @@ def gated_delta_rule(qkv, beta, a, dt_bias, a_log, gate, norm_w, eps: float,
                                 dim, vdim, out_dtype, gate_act)
 
 
+HEAD_PRODUCT_MAX_TOKENS = 256
+
+
 def head_product(a, w):
     """Per-head product a (T,H,K) x w (H,N,K)^T -> (T,H,N), 32-bit sums."""
     T, H, K = a.shape
     out = torch.empty(T, H, w.shape[1], dtype=a.dtype, device=a.device)
+    if a.is_cuda and a.dtype == torch.bfloat16 and K % 8 == 0 and T <= HEAD_PRODUCT_MAX_TOKENS \
+            and a.is_contiguous() and w.is_contiguous():
+        assert w.dtype == a.dtype and w.shape[0] == H and w.shape[2] == K
+        _check(_load().nx_head_product(_p(a), _p(w), _p(out), T, H, K, w.shape[1], _stream()),
+               "head_product")
+        return out
     # (the library's batched product gets no transposed right operand)
     torch.bmm(a.transpose(0, 1), w.transpose(1, 2).contiguous(), out=out.transpose(0, 1))
     return out
@@ -607,36 +616,34 @@ def head_norm_rotate(x, step: StepLayout, norm_weight, eps: float, inv_freq,
                                 mscale).reshape(B, S, N * C).to(out_dtype)
 
 
-def channel_decay(z, bias, tau: float):
-    """sigmoid(z + bias)^(1/tau) in fp32; z (B,S,C) may be a column slice."""
-    if z.is_cuda:
+def low_rank_decay(low, weight, bias, tau: float):
+    """Logarithms of per-channel decays from a low-rank projection:
+    log(sigmoid(low @ weight.T + bias)) / tau in fp32. low (B,S,rank) may be a
+    column slice; weight (C, rank) in the same dtype, bias (C,) fp32."""
+    if low.is_cuda:
         lib = _load()
-        C = z.shape[-1]
-        out = torch.empty(z.shape, dtype=torch.float32, device=z.device)
+        C, rank = weight.shape
+        assert low.shape[-1] == rank and low.dtype == weight.dtype and weight.is_contiguous()
         assert bias.numel() == C
-        _check(lib.nx_channel_decay(_p(z), ctypes.c_long(_rows_view(z)), _is_bf16(z),
-                                    _p(_f32(bias)), ctypes.c_float(1.0 / tau), _p(out),
-                                    ctypes.c_long(z.numel() // C), C, _stream()),
-               "channel_decay")
+        out = torch.empty(low.shape[:-1] + (C,), dtype=torch.float32, device=low.device)
+        _check(lib.nx_low_rank_decay(
+            _p(low), ctypes.c_long(_rows_view(low)), _p(weight), _is_bf16(low), _p(_f32(bias)),
+            ctypes.c_float(1.0 / tau), _p(out), ctypes.c_long(low.numel() // rank), C, rank,
+            _stream()), "low_rank_decay")
         return out
-    return ref.channel_decay(z, bias, tau)
-
-
-# steps of at most this many tokens a row compute their channel decays inside
-# the scan (once per block of value channels) instead of in a launch of their own
-INLINE_DECAY_MAX_TOKENS = 4
+    return ref.low_rank_decay(low, weight, bias, tau)
 
 
 def decay_scan(q, k, v, state, step: StepLayout, dim: int, vdim: int, dt=None,
                dt_bias=None, a_log=None, head_decay=None, k_scale: float = 1.0, skip=None,
-               channel_logits=None, channel_bias=None, tau: float = 1.0):
+               log_decay=None):
     """Decayed linear recurrence with matrix state (see ref.decay_scan):
     selective state spaces (``dt``/``dt_bias``/``a_log``), fixed per-head
-    decays (``head_decay``) or a decay per key channel (``channel_logits``
-    (B,S,H*dim) with ``channel_bias`` and ``tau``). q, k (B,S,G*dim), v (B,S,H*vdim) may be column
+    decays (``head_decay``) or a decay per key channel (its logarithm
+    ``log_decay`` (B,S,H*dim) fp32). q, k (B,S,G*dim), v (B,S,H*vdim) may be column
     slices of wider tensors; ``state`` (slots, H, vdim, dim) fp32 is read
     (unless the row starts at position 0) and advanced. Returns fp32."""
-    assert sum(x is not None for x in (dt, head_decay, channel_logits)) == 1
+    assert sum(x is not None for x in (dt, head_decay, log_decay)) == 1
     if v.is_cuda:
         lib = _load()
         B, S = v.shape[0], v.shape[1]
@@ -646,13 +653,11 @@ def decay_scan(q, k, v, state, step: StepLayout, dim: int, vdim: int, dt=None,
         assert state.is_contiguous() and tuple(state.shape[1:]) == (H, vdim, dim)
         assert H % G == 0 and q.shape[-1] == G * dim and k.shape[-1] == G * dim
         out = torch.empty(B, S, H * vdim, dtype=torch.float32, device=v.device)
-        channel, dch = channel_logits is not None, 1
+        channel, dch = log_decay is not None, 1
         if channel:
-            assert G == H and skip is None and channel_logits.shape[-1] == H * dim
-            assert channel_bias.numel() == H * dim
-            dt, dt_bias, dch = channel_logits, channel_bias, dim
-            if S > INLINE_DECAY_MAX_TOKENS:
-                dt, dt_bias = channel_decay(channel_logits, channel_bias, tau), None
+            assert G == H and skip is None and log_decay.shape[-1] == H * dim
+            assert log_decay.dtype == torch.float32
+            dt, dch = log_decay, dim
         # a long row with few (row, head, channel block) workgroups is cut into
         # segments that scan side by side (two passes joined by a short serial
         # link over the segments' end states)
@@ -677,12 +682,47 @@ def decay_scan(q, k, v, state, step: StepLayout, dim: int, vdim: int, dt=None,
             ctypes.c_float(k_scale), _p(None if skip is None else _f32(skip)),
             _p(state), _p(step.positions), _p(step.seq_ids), _p(step.nvalid), _p(out),
             B, S, H, G, dim, vdim, _p(ws), _p(wdec), nseg, seglen, int(channel),
-            ctypes.c_float(1.0 / tau), _stream()), "decay_scan")
+            _stream()), "decay_scan")
         return out
     return ref.decay_scan(q, k, v, state, step.positions, step.seq_ids, dim, vdim,
                           dt=dt, dt_bias=dt_bias, a_log=a_log, head_decay=head_decay,
-                          k_scale=k_scale, skip=skip, channel_logits=channel_logits,
-                          channel_bias=channel_bias, tau=tau)
+                          k_scale=k_scale, skip=skip, log_decay=log_decay)
+
+
+CHUNKED_GLA_MIN_TOKENS = 96
+
+
+def gated_linear_attention(q, k, v, log_decay, gate, norm_weight, eps: float, state,
+                           step: StepLayout, dim: int, vdim: int, k_scale: float = 1.0):
+    """Recurrence with a decay per key channel and its gated read-out norm:
+    decay_scan(log_decay) -> RMS norm per head (weight shared by the heads) ->
+    times silu(gate), in the gate's dtype. Long bf16 rows run in chunks on the
+    matrix cores with the norm and gate fused; everything else is the scan
+    and the norm kernel."""
+    B, S = v.shape[0], v.shape[1]
+    H = v.shape[-1] // vdim
+    if v.is_cuda and S >= CHUNKED_GLA_MIN_TOKENS and dim <= 128 and vdim <= 128 and \
+            dim % 8 == 0 and vdim % 8 == 0 and \
+            all(t.dtype == torch.bfloat16 for t in (q, k, v, gate)) and \
+            all(_rows_view(t) % 8 == 0 and t.data_ptr() % 16 == 0 for t in (q, k, v)):
+        lib = _load()
+        assert log_decay.dtype == torch.float32 and log_decay.is_contiguous()
+        assert log_decay.shape[-1] == H * dim == q.shape[-1] == k.shape[-1]
+        assert state.dtype == torch.float32 and state.is_contiguous()
+        assert tuple(state.shape[1:]) == (H, vdim, dim) and norm_weight.numel() == vdim
+        nc = (S + 63) // 64
+        ws = torch.empty(B * nc * H * vdim * dim, dtype=torch.float32, device=v.device)
+        wdec = torch.empty(B * nc * H * dim, dtype=torch.float32, device=v.device)
+        out = torch.empty(B, S, H * vdim, dtype=torch.bfloat16, device=v.device)
+        _check(lib.nx_gla_chunked(
+            _p(q), ctypes.c_long(_rows_view(q)), _p(k), ctypes.c_long(_rows_view(k)),
+            _p(v), ctypes.c_long(_rows_view(v)), _p(log_decay), ctypes.c_float(k_scale),
+            _p(gate), ctypes.c_long(_rows_view(gate)), _p(_f32(norm_weight)), ctypes.c_float(eps),
+            _p(state), _p(step.positions), _p(step.seq_ids), _p(step.nvalid), _p(ws), _p(wdec),
+            _p(out), B, S, H, dim, vdim, _stream()), "gated_linear_attention")
+        return out
+    o = decay_scan(q, k, v, state, step, dim, vdim, log_decay=log_decay, k_scale=k_scale)
+    return group_gated_norm(o, gate, norm_weight, eps, H, gate_first=False, out_dtype=gate.dtype)
 
 
 def group_gated_norm(y, gate, weight, eps: float, groups: int, gate_first: bool,
@@ -951,3 +991,22 @@ def token_gate(z, ids, table, offset: int):
                "token_gate")
         return out
     return ref.token_gate(z, ids, table, offset).to(z.dtype)
+
+
+def token_gate_proj(h, weight, ids, table, offset: int):
+    """:func:`token_gate` of the projection z = h @ weight.T; narrow bf16
+    projections take one launch for product, gelu and gate."""
+    C, K = weight.shape
+    if h.is_cuda and h.dtype == torch.bfloat16 and K % 8 == 0 and C <= 256 and \
+            h.is_contiguous() and weight.is_contiguous() and ids.numel() <= 1 << 20:
+        lib = _load()
+        assert ids.dtype == torch.int64 and ids.is_contiguous() and h.shape[-1] == K
+        assert table.dtype == weight.dtype == h.dtype and table.is_contiguous()
+        out = torch.empty(h.shape[:-1] + (C,), dtype=h.dtype, device=h.device)
+        assert ids.numel() * C == out.numel()
+        _check(lib.nx_token_gate_proj(
+            _p(h), ctypes.c_long(K), _p(weight), K, _p(ids), _p(table),
+            ctypes.c_long(table.stride(0)), int(offset), table.shape[0], _p(out),
+            ctypes.c_long(ids.numel()), C, _stream()), "token_gate_proj")
+        return out
+    return token_gate(torch.nn.functional.linear(h, weight), ids, table, offset)
