@@ -1201,15 +1201,19 @@ latent_decode_mfma_kernel(const bf16* __restrict__ q, long qstride, const bf16* 
     }
 }
 
-// one wave per (token, head): out = sum_i o_i e^(m_i - M) / (sum_i l_i e^(m_i - M)
+// one wave per (token, head, LM_W value channels): out = sum_i o_i e^(m_i - M) / (sum_i l_i e^(m_i - M)
 // + e^(sink - M)), M the largest of the splits' maxima and the sink
+#define LM_W 128
 __global__ void latent_decode_merge_kernel(const float* __restrict__ ws,
                                            const float* __restrict__ sink,
                                            const int* __restrict__ pos, const int* __restrict__ seq,
                                            bf16* __restrict__ out, long ntok, int S, int H, int Dv,
                                            int nks, const bf16* __restrict__ gate, long gstride) {
     const int lane = threadIdx.x & (WAVE - 1);
-    const long wid = (long)blockIdx.x * (blockDim.x / WAVE) + threadIdx.x / WAVE;
+    const int parts = (Dv + LM_W - 1) / LM_W;
+    const long id = (long)blockIdx.x * (blockDim.x / WAVE) + threadIdx.x / WAVE;
+    const long wid = id / parts;
+    const int d0 = (id % parts) * LM_W;
     if (wid >= ntok * H) return;
     const long tok = wid / H;
     const int h = wid % H;
@@ -1231,7 +1235,9 @@ __global__ void latent_decode_merge_kernel(const float* __restrict__ ws,
         const float mi = i < nks ? wp[i * (long)(Dv + 2) + Dv] : -INFINITY;
         wgt[i] = mi > -INFINITY ? expf(mi - M) * inv : 0.f;
     }
-    for (int d = lane; d < Dv; d += WAVE) {
+#pragma unroll
+    for (int d = d0 + lane; d < d0 + LM_W; d += WAVE) {
+        if (d >= Dv) break;
         float o = 0.f;
 #pragma unroll
         for (int i = 0; i < 8; ++i)
@@ -2156,11 +2162,10 @@ __global__ void decay_scan_link_kernel(float* __restrict__ ws, const float* __re
 // ------------------------------------------------- low-rank channel decays
 // log decay of a key channel: log(sigmoid(low[t] . w[c] + bias[c])) * inv_tau, all
 // fp32 (a very negative logit does not underflow). A thread owns one channel for
-// LRD_T tokens, whose low-rank rows sit in LDS.
-#define LRD_T 16
+// LRD_T tokens (few in steps of few tokens), whose low-rank rows sit in LDS.
 #define LRD_R 64
 
-template <typename T>
+template <typename T, int LRD_T>
 __global__ void __launch_bounds__(256)
 low_rank_decay_kernel(const T* __restrict__ low, long ls, const T* __restrict__ w, int vec,
                       const float* __restrict__ bias, float inv_tau, float* __restrict__ out,
@@ -2220,28 +2225,41 @@ low_rank_decay_kernel(const T* __restrict__ low, long ls, const T* __restrict__ 
 //                           per-head RMS norm, its weight and the silu gate.
 // Every exponent is taken relative to a sub-block's edge between the two tokens, so
 // it is never positive: no overflow, whatever the decays. A_ts of two different
-// sub-blocks is a product of two such factors (matrix cores); inside a sub-block it
-// is summed directly in fp32. fp32 operands of the matrix cores are split into bf16
+// sub-blocks is a product of two such factors (matrix cores), and so it is inside a
+// sub-block whose decays are mild; otherwise it is summed directly in fp32. fp32 operands of the matrix cores are split into bf16
 // terms: three for the keys that enter the state (24 bits), two elsewhere (16 bits);
 // accumulation and state are fp32.
 #define GC_N 64
 #define GC_VS (GC_N + 8)
+
+DEV float exp2_(float x) { return __builtin_amdgcn_exp2f(x); }   // hardware, 1 ulp
 
 DEV void split_bf16_(float x, __bf16& hi, __bf16& lo) {
     hi = (__bf16)x;
     lo = (__bf16)(x - (float)hi);
 }
 
-// V^T of a chunk: (NT*16 channels, GC_VS) with zeros past the last token / channel
-template <int NT>
-DEV void gc_stage_vt_(const bf16* __restrict__ v, long vs, long tok0, int cnt, int Dv,
-                      uint16_t* __restrict__ vt, int tid) {
-    for (int c = tid; c < GC_N * NT * 2; c += 256) {
-        const int m = c % GC_N, part = c / GC_N;
-        uint4 raw = make_uint4(0, 0, 0, 0);
-        if (m < cnt && part * 8 < Dv)
-            raw = *reinterpret_cast<const uint4*>(v + (tok0 + m) * vs + part * 8);
-        const uint32_t u[4] = {raw.x, raw.y, raw.z, raw.w};
+// 64 token rows of P*8 bf16 channels each, 16 bytes a time, into registers: all loads
+// are in flight together (addresses are clamped, not branched around), zeros past the
+// last token (cnt >= 1) and channel (n, a multiple of 8)
+template <int P>
+DEV void gc_load_rows_(const bf16* __restrict__ x, long xs, int cnt, int n, uint4* r, int tid) {
+#pragma unroll
+    for (int i = 0; i < P / 4; ++i) {
+        const int c = tid + i * 256, m = c % GC_N, part = c / GC_N;
+        const uint4 v = *reinterpret_cast<const uint4*>(
+            x + (long)min(m, cnt - 1) * xs + min(part * 8, n - 8));
+        const bool ok = m < cnt && part * 8 < n;
+        r[i] = make_uint4(ok ? v.x : 0, ok ? v.y : 0, ok ? v.z : 0, ok ? v.w : 0);
+    }
+}
+// registers of gc_load_rows_ -> V^T (P*8 channels, GC_VS)
+template <int P>
+DEV void gc_store_vt_(const uint4* r, uint16_t* __restrict__ vt, int tid) {
+#pragma unroll
+    for (int i = 0; i < P / 4; ++i) {
+        const int c = tid + i * 256, m = c % GC_N, part = c / GC_N;
+        const uint32_t u[4] = {r[i].x, r[i].y, r[i].z, r[i].w};
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
             vt[(part * 8 + 2 * e) * GC_VS + m] = (uint16_t)(u[e] & 0xffffu);
@@ -2271,30 +2289,34 @@ gla_chunk_state_kernel(const bf16* __restrict__ k, long ks, const bf16* __restri
     const float* lp = ld + (long)h * D + d0;
     const bf16* kp = k + (long)h * D + d0;
     const long lst = (long)H * D;
-    gc_stage_vt_<NT>(v + (long)h * Dv, vs, tok0, cnt, Dv, vt, tid);
-    // one (channel, sub-block) task per thread and turn: its 16 log decays
-    for (int task = tid; task < 4 * DP; task += 256) {
-        const int d = task % DP, sb = task / DP;
+    // one (channel, sub-block of 16 tokens) task per thread
+    static_assert(4 * DP <= 256, "one task per thread");
+    uint4 vr[NT / 2];
+    gc_load_rows_<NT * 2>(v + tok0 * vs + (long)h * Dv, vs, cnt, Dv, vr, tid);
+    const int d = tid % DP, sb = tid / DP;
+    float g[16], kv[16];
+    if (sb < 4) {
         float t = 0.f;
-        for (int i = 0; i < 16; ++i) {
-            const int m = sb * 16 + i;
-            if (m < cnt && d < Dn) t += lp[(tok0 + m) * lst + d];
-        }
-        tot[sb][d] = t;
-    }
-    __syncthreads();
-    for (int task = tid; task < 4 * DP; task += 256) {
-        const int d = task % DP, sb = task / DP;
-        float after = 0.f;                                // decays of the later tokens
-        for (int m = sb + 1; m < 4; ++m) after += tot[m][d];
-        float g[16], kv[16];
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
             const int m = sb * 16 + i;
             const bool ok = m < cnt && d < Dn;
-            g[i] = ok ? lp[(tok0 + m) * lst + d] : 0.f;
-            kv[i] = ok ? ldf<bf16>(kp + (tok0 + m) * ks + d) * k_scale : 0.f;
+            const long tk = tok0 + min(m, cnt - 1);
+            const int dc = min(d, Dn - 1);
+            const float gv = lp[tk * lst + dc], kk = ldf<bf16>(kp + tk * ks + dc);
+            g[i] = ok ? gv : 0.f;
+            kv[i] = ok ? kk * k_scale : 0.f;
         }
+#pragma unroll
+        for (int i = 0; i < 16; ++i) t += g[i];
+        tot[sb][d] = t;
+    }
+    gc_store_vt_<NT * 2>(vr, vt, tid);
+    __syncthreads();
+    if (sb < 4) {
+        float after = 0.f;                                // decays of the later tokens
+        for (int m = sb + 1; m < 4; ++m) after += tot[m][d];
+        bf16x8_t t0[2], t1[2], t2[2];                     // the three terms of 16 tokens
 #pragma unroll
         for (int i = 15; i >= 0; --i) {
             const float x = kv[i] * expf(after);
@@ -2302,11 +2324,16 @@ gla_chunk_state_kernel(const bf16* __restrict__ k, long ks, const bf16* __restri
             const __bf16 a0 = (__bf16)x;
             const float r1 = x - (float)a0;
             const __bf16 a1 = (__bf16)r1;
-            const __bf16 a2 = (__bf16)(r1 - (float)a1);
-            const int at = d * GC_VS + sb * 16 + i;
-            kt[0][at] = __builtin_bit_cast(uint16_t, a0);
-            kt[1][at] = __builtin_bit_cast(uint16_t, a1);
-            kt[2][at] = __builtin_bit_cast(uint16_t, a2);
+            t0[i >> 3][i & 7] = a0;
+            t1[i >> 3][i & 7] = a1;
+            t2[i >> 3][i & 7] = (__bf16)(r1 - (float)a1);
+        }
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+            const int at = d * GC_VS + sb * 16 + u * 8;
+            *reinterpret_cast<bf16x8_t*>(kt[0] + at) = t0[u];
+            *reinterpret_cast<bf16x8_t*>(kt[1] + at) = t1[u];
+            *reinterpret_cast<bf16x8_t*>(kt[2] + at) = t2[u];
         }
         if (sb == 0 && d < Dn) wdec[(((long)b * nc + c) * H + h) * D + d0 + d] = expf(after);
     }
@@ -2328,17 +2355,18 @@ gla_chunk_state_kernel(const bf16* __restrict__ k, long ks, const bf16* __restri
                 acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va, kb, acc, 0, 0, 0);
             }
         }
-        const int d = dt * 16 + lr;
+        const int dd = dt * 16 + lr;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const int nn = nt * 16 + lg * 4 + r;
-            if (nn < Dv && d < Dn) wp[(long)nn * D + d] = acc[r];
+            if (nn < Dv && dd < Dn) wp[(long)nn * D + dd] = acc[r];
         }
     }
 }
 
 // start states of the chunks, in place over their contributions, and the carried
-// state; eight chunks' loads are in flight at a time
+// state; eight chunks' loads are in flight at a time. A start state leaves as its two
+// bf16 terms (the high one in the high half of the word), ready for the read-out.
 __global__ void __launch_bounds__(256)
 gla_chunk_link_kernel(float* __restrict__ ws, const float* __restrict__ wdec,
                       float* __restrict__ state, const int* __restrict__ pos,
@@ -2364,14 +2392,21 @@ gla_chunk_link_kernel(float* __restrict__ ws, const float* __restrict__ wdec,
                 if (c0 + j < chunks) { en[j] = wp[(c0 + j) * wst]; dc[j] = dp[(c0 + j) * dst]; }
 #pragma unroll
             for (int j = 0; j < 8; ++j)
-                if (c0 + j < chunks) { wp[(c0 + j) * wst] = s; s = dc[j] * s + en[j]; }
+                if (c0 + j < chunks) {
+                    __bf16 hi, lo;
+                    split_bf16_(s, hi, lo);
+                    wp[(c0 + j) * wst] = __uint_as_float(
+                        ((uint32_t)__builtin_bit_cast(uint16_t, hi) << 16) |
+                        __builtin_bit_cast(uint16_t, lo));
+                    s = dc[j] * s + en[j];
+                }
         }
         *sp = s;
     }
 }
 
 template <int DP, int NT>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, 2)
 gla_chunk_out_kernel(const bf16* __restrict__ q, long qs, const bf16* __restrict__ k, long ks,
                      const bf16* __restrict__ v, long vs, const float* __restrict__ ld,
                      float k_scale, const bf16* __restrict__ gate, long gs,
@@ -2401,25 +2436,49 @@ gla_chunk_out_kernel(const bf16* __restrict__ q, long qs, const bf16* __restrict
         if (tv && d < D)
             qr[kk] = *reinterpret_cast<const uint4*>(q + (tok0 + w * 16 + lr) * qs + (long)h * D + d);
     }
-    gc_stage_vt_<NT>(v + (long)h * Dv, vs, tok0, cnt, Dv, vt, tid);
-    for (int i = tid; i < GC_N * (DP / 8); i += 256) {
-        const int m = i / (DP / 8), part = i % (DP / 8);
-        uint4 raw = make_uint4(0, 0, 0, 0);
-        if (m < cnt && part * 8 < D)
-            raw = *reinterpret_cast<const uint4*>(k + (tok0 + m) * ks + (long)h * D + part * 8);
-        *reinterpret_cast<uint4*>(kl + m * KS + part * 8) = raw;
+    // start state, this lane's rows (value channel lr of every tile), packed terms:
+    // the first block of key channels is fetched here, the next ones while one is used
+    const float* sp = ws + (((long)b * nc + c) * H + h) * (long)Dv * D + (long)lr * D + lg * 8;
+    uint4 sr[NT][2];
+#define GC_FETCH(KKI)                                                                      \
+    _Pragma("unroll") for (int nt = 0; nt < NT; ++nt) {                                    \
+        sr[nt][0] = sr[nt][1] = make_uint4(0, 0, 0, 0);                                    \
+        if (nt * 16 + lr < Dv && (KKI) * 32 + lg * 8 < D) {                                \
+            const float* rp = sp + (long)nt * 16 * D + (KKI) * 32;                         \
+            sr[nt][0] = *reinterpret_cast<const uint4*>(rp);                               \
+            sr[nt][1] = *reinterpret_cast<const uint4*>(rp + 4);                           \
+        }                                                                                  \
     }
-    for (int task = tid; task < 4 * DP; task += 256) {
-        const int d = task % DP, sb = task / DP;
-        float g[16];
+    GC_FETCH(0)
+    uint4 vr[NT / 2], kr[DP / 32];
+    gc_load_rows_<NT * 2>(v + tok0 * vs + (long)h * Dv, vs, cnt, Dv, vr, tid);
+    gc_load_rows_<DP / 8>(k + tok0 * ks + (long)h * D, ks, cnt, D, kr, tid);
+    constexpr int TASKS = (4 * DP + 255) / 256;           // (channel, sub-block) per thread
+    float g[TASKS][16];
 #pragma unroll
-        for (int i = 0; i < 16; ++i) {
-            const int m = sb * 16 + i;
-            g[i] = (m < cnt && d < D) ? ld[(tok0 + m) * (long)(H * D) + (long)h * D + d] : 0.f;
-        }
+    for (int x = 0; x < TASKS; ++x) {
+        const int task = tid + x * 256, d = min(task % DP, D - 1), sb = task / DP;
+#pragma unroll
+        for (int i = 0; i < 16; ++i)
+            g[x][i] = ld[(tok0 + min(sb * 16 + i, cnt - 1)) * (long)(H * D) + (long)h * D + d];
+    }
+    gc_store_vt_<NT * 2>(vr, vt, tid);
+#pragma unroll
+    for (int i = 0; i < DP / 32; ++i) {
+        const int x = tid + i * 256;
+        *reinterpret_cast<uint4*>(kl + (x % GC_N) * KS + (x / GC_N) * 8) = kr[i];
+    }
+#pragma unroll
+    for (int x = 0; x < TASKS; ++x) {
+        const int task = tid + x * 256, d = task % DP, sb = task / DP;
+        if (sb >= 4) continue;                            // DP = 32: half the threads
         float t = 0.f;
 #pragma unroll
-        for (int i = 0; i < 16; ++i) { t += g[i]; ll[(sb * 16 + i) * LS + d] = t; }
+        for (int i = 0; i < 16; ++i) {
+            // base 2 from here on; tokens past the last and padding channels stand still
+            t += (sb * 16 + i < cnt && d < D) ? g[x][i] * 1.4426950408889634f : 0.f;
+            ll[(sb * 16 + i) * LS + d] = t;
+        }
         tot[sb][d] = t;
     }
     __syncthreads();
@@ -2443,44 +2502,52 @@ gla_chunk_out_kernel(const bf16* __restrict__ q, long qs, const bf16* __restrict
     for (int nt = 0; nt < NT; ++nt) o[nt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     // ---- (q exp(G_t)) S: S rows (value channel lr of the tile) from memory
     {
-        const float* sp = ws + (((long)b * nc + c) * H + h) * (long)Dv * D;
 #pragma unroll
         for (int kk = 0; kk < KK; ++kk) {
-            const int d = kk * 32 + lg * 8;
             bf16x8_t qh, ql;
 #pragma unroll
             for (int e = 0; e < 8; ++e) {
                 __bf16 hi, lo;
-                split_bf16_(qf[kk][e] * __expf(pre[kk][e] + lt[kk][e]), hi, lo);
+                split_bf16_(qf[kk][e] * exp2_(pre[kk][e] + lt[kk][e]), hi, lo);
                 qh[e] = hi; ql[e] = lo;
             }
 #pragma unroll
             for (int nt = 0; nt < NT; ++nt) {
-                const int nn = nt * 16 + lr;
-                float sv[8];
-#pragma unroll
-                for (int e = 0; e < 8; ++e) sv[e] = 0.f;
-                if (nn < Dv && d < D) load8<float>(sp + (long)nn * D + d, sv);
-                bf16x8_t sh, sl;
-#pragma unroll
-                for (int e = 0; e < 8; ++e) {
-                    __bf16 hi, lo;
-                    split_bf16_(sv[e], hi, lo);
-                    sh[e] = hi; sl[e] = lo;
-                }
+                const uint4 s0 = sr[nt][0], s1 = sr[nt][1];
+                // two words (hi | lo) each -> a pair of high and a pair of low terms
+                const uint4 hv = make_uint4(
+                    (s0.x >> 16) | (s0.y & 0xffff0000u), (s0.z >> 16) | (s0.w & 0xffff0000u),
+                    (s1.x >> 16) | (s1.y & 0xffff0000u), (s1.z >> 16) | (s1.w & 0xffff0000u));
+                const uint4 lv = make_uint4(
+                    (s0.x & 0xffffu) | (s0.y << 16), (s0.z & 0xffffu) | (s0.w << 16),
+                    (s1.x & 0xffffu) | (s1.y << 16), (s1.z & 0xffffu) | (s1.w << 16));
+                const bf16x8_t sh = __builtin_bit_cast(bf16x8_t, hv);
+                const bf16x8_t sl = __builtin_bit_cast(bf16x8_t, lv);
                 o[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ql, sh, o[nt], 0, 0, 0);
                 o[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qh, sl, o[nt], 0, 0, 0);
                 o[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qh, sh, o[nt], 0, 0, 0);
             }
+            if (kk + 1 < KK) GC_FETCH(kk + 1)
         }
     }
+#undef GC_FETCH
     // ---- A^T: lane gets keys 4*lg + r of sub-block j for query lr
     float sc[4][4];
 #pragma unroll
     for (int j = 0; j < 4; ++j)
 #pragma unroll
         for (int r = 0; r < 4; ++r) sc[j][r] = 0.f;
-    {   // own sub-block: exp(L_t - L_s) directly, channels split over the four lane groups
+    // Own sub-block: when no channel decays by more than 2^-60 inside it, exp(L_t) and
+    // exp(-L_s) are both far from overflow and the product form below serves it too
+    // (what it gives for s > t is dropped); else exp(L_t - L_s) is taken directly,
+    // channels split over the four lane groups.
+    bool mild = true;
+#pragma unroll
+    for (int kk = 0; kk < KK; ++kk)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) mild = mild && tot[w][kk * 32 + lg * 8 + e] > -60.f;
+    mild = __all(mild);
+    if (!mild) {
         float part[16];
 #pragma unroll
         for (int si = 0; si < 16; ++si) {
@@ -2493,7 +2560,7 @@ gla_chunk_out_kernel(const bf16* __restrict__ q, long qs, const bf16* __restrict
                 load8<float>(ll + (w * 16 + si) * LS + d, lv);
 #pragma unroll
                 for (int e = 0; e < 8; ++e)
-                    a += qf[kk][e] * kv[e] * __expf(fminf(lt[kk][e] - lv[e], 0.f));
+                    a += qf[kk][e] * kv[e] * exp2_(lt[kk][e] - lv[e]);   // s > t: dropped below
             }
             part[si] = a;
         }
@@ -2515,8 +2582,9 @@ gla_chunk_out_kernel(const bf16* __restrict__ q, long qs, const bf16* __restrict
 #pragma unroll
                 for (int r = 0; r < 4; ++r) sc[j][r] = own[r] * k_scale;
     }
-    // earlier sub-blocks: q exp(L_t) against k exp(sum between - ...)
-    if (w > 0) {
+    // earlier sub-blocks (and a mild own one): q exp(L_t) against k exp(what lies
+    // between s and the start of the own sub-block)
+    {
         bf16x8_t qh[KK], ql[KK];
         float btw[KK][8];                                 // log decays of the sub-blocks between
 #pragma unroll
@@ -2524,13 +2592,13 @@ gla_chunk_out_kernel(const bf16* __restrict__ q, long qs, const bf16* __restrict
 #pragma unroll
             for (int e = 0; e < 8; ++e) {
                 __bf16 hi, lo;
-                split_bf16_(qf[kk][e] * __expf(lt[kk][e]), hi, lo);
+                split_bf16_(qf[kk][e] * exp2_(lt[kk][e]), hi, lo);
                 qh[kk][e] = hi; ql[kk][e] = lo;
                 btw[kk][e] = 0.f;
             }
 #pragma unroll
-        for (int j = 2; j >= 0; --j) {
-            if (j >= w) continue;                         // wave-uniform
+        for (int j = 3; j >= 0; --j) {
+            if (j > w || (j == w && !mild)) continue;     // wave-uniform
             f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int kk = 0; kk < KK; ++kk) {
@@ -2543,8 +2611,8 @@ gla_chunk_out_kernel(const bf16* __restrict__ q, long qs, const bf16* __restrict
 #pragma unroll
                 for (int e = 0; e < 8; ++e) {
                     __bf16 hi, lo;
-                    btw[kk][e] += tv8[e];                 // now from the start of j to the start of w
-                    split_bf16_(kv[e] * __expf(btw[kk][e] - lv[e]), hi, lo);
+                    if (j < w) btw[kk][e] += tv8[e];      // now from the start of j to the start of w
+                    split_bf16_(kv[e] * exp2_(btw[kk][e] - lv[e]), hi, lo);
                     kh[e] = hi; klo[e] = lo;
                 }
                 acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(klo, qh[kk], acc, 0, 0, 0);
@@ -2552,7 +2620,8 @@ gla_chunk_out_kernel(const bf16* __restrict__ q, long qs, const bf16* __restrict
                 acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kh, qh[kk], acc, 0, 0, 0);
             }
 #pragma unroll
-            for (int r = 0; r < 4; ++r) sc[j][r] = acc[r] * k_scale;
+            for (int r = 0; r < 4; ++r)
+                sc[j][r] = j < w || lg * 4 + r <= lr ? acc[r] * k_scale : 0.f;
         }
     }
     // ---- O += A V, two sub-blocks of keys at a time, A as hi + lo
@@ -2577,6 +2646,14 @@ gla_chunk_out_kernel(const bf16* __restrict__ q, long qs, const bf16* __restrict
         }
     }
     // ---- norm over the head's channels (tiles x 16 lanes), weight, silu gate
+    float gw[4][NT];                                      // gates, loads in flight together
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+        const bf16* gp = gate + (tok0 + min(w * 16 + lg * 4 + r, cnt - 1)) * gs + (long)h * Dv;
+#pragma unroll
+        for (int nt = 0; nt < NT; ++nt)
+            gw[r][nt] = __bfloat162float(gp[min(nt * 16 + lr, Dv - 1)]);
+    }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
         float ss = 0.f;
@@ -2589,13 +2666,12 @@ gla_chunk_out_kernel(const bf16* __restrict__ q, long qs, const bf16* __restrict
         const int t = w * 16 + lg * 4 + r;
         if (t >= cnt) continue;
         const float inv = 1.f / sqrtf(ss / Dv + eps);
-        const bf16* gp = gate + (tok0 + t) * gs + (long)h * Dv;
         bf16* op = out + (tok0 + t) * (long)(H * Dv) + (long)h * Dv;
 #pragma unroll
         for (int nt = 0; nt < NT; ++nt) {
             const int nn = nt * 16 + lr;
             if (nn >= Dv) continue;
-            const float gv = __bfloat162float(gp[nn]);
+            const float gv = gw[r][nt];
             op[nn] = __float2bfloat16(o[nt][r] * inv * nw[nn] * (gv * sigmoidf_(gv)));
         }
     }
@@ -3147,7 +3223,7 @@ head_product_kernel(const bf16* __restrict__ a, const bf16* __restrict__ w,
     f32x4_t acc[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
+#pragma unroll 4
     for (int k0 = wv * 32; k0 < K; k0 += 4 * 32) {
         const bool kin = k0 + lg * 8 < K;
         uint4 wa = make_uint4(0, 0, 0, 0);
@@ -3369,7 +3445,7 @@ int nx_paged_attn(const void* q, long qstride, const void* kc, long ktok, long k
         else LD(640);
 #undef LD
         if (nks > 1) {
-            const long waves = (long)B * S * H;
+            const long waves = (long)B * S * H * ((Dv + LM_W - 1) / LM_W);
             latent_decode_merge_kernel<<<(unsigned)((waves + 3) / 4), 4 * WAVE, 0, st>>>(
                 ws, sink, pos, seq, (bf16*)out, (long)B * S, S, H, Dv, nks, (const bf16*)gate,
                 gstride);
@@ -3685,12 +3761,14 @@ int nx_low_rank_decay(const void* low, long ls, const void* w, int is_bf16, cons
     if (rows * C <= 0) return 0;
     if (!bias || rank <= 0) return -1;
     const int vec = (rank % 8) == 0 && ((uintptr_t)w % 16) == 0;
-    const long gy = (rows + LRD_T - 1) / LRD_T;
+    const int tt = rows <= 512 ? 2 : 16;
+    const long gy = (rows + tt - 1) / tt;
     dim3 grid((C + 255) / 256, (unsigned)(gy > 32768 ? 32768 : gy)), block(256);
-    if (is_bf16) low_rank_decay_kernel<bf16><<<grid, block, 0, st>>>(
-        (const bf16*)low, ls, (const bf16*)w, vec, bias, inv_tau, out, rows, C, rank);
-    else low_rank_decay_kernel<float><<<grid, block, 0, st>>>(
-        (const float*)low, ls, (const float*)w, vec, bias, inv_tau, out, rows, C, rank);
+#define LRD(T, TT) low_rank_decay_kernel<T, TT><<<grid, block, 0, st>>>( \
+        (const T*)low, ls, (const T*)w, vec, bias, inv_tau, out, rows, C, rank)
+    if (is_bf16) { if (tt == 2) LRD(bf16, 2); else LRD(bf16, 16); }
+    else { if (tt == 2) LRD(float, 2); else LRD(float, 16); }
+#undef LRD
     return (int)hipGetLastError();
 }
 

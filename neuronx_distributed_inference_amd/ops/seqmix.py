@@ -995,10 +995,10 @@ def token_gate(z, ids, table, offset: int):
 
 def token_gate_proj(h, weight, ids, table, offset: int):
     """:func:`token_gate` of the projection z = h @ weight.T; narrow bf16
-    projections take one launch for product, gelu and gate."""
+    projections of few tokens take one launch for product, gelu and gate."""
     C, K = weight.shape
     if h.is_cuda and h.dtype == torch.bfloat16 and K % 8 == 0 and C <= 256 and \
-            h.is_contiguous() and weight.is_contiguous() and ids.numel() <= 1 << 20:
+            h.is_contiguous() and weight.is_contiguous() and ids.numel() <= 1024:
         lib = _load()
         assert ids.dtype == torch.int64 and ids.is_contiguous() and h.shape[-1] == K
         assert table.dtype == weight.dtype == h.dtype and table.is_contiguous()
