@@ -708,7 +708,8 @@ paged_attn_mfma_kernel(const bf16* __restrict__ q, long qstride, const bf16* __r
     __shared__ float ra1[MA_ROWS], ra2[MA_ROWS], rsink[MA_ROWS];
     const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
     const int lr = lane & 15, lg = lane >> 4;
-    const int b = blockIdx.z, g = blockIdx.y / nsplit, t0 = blockIdx.x * QT;
+    // the last tokens of a row see the most keys: they start first
+    const int b = blockIdx.z, g = blockIdx.y / nsplit, t0 = (gridDim.x - 1 - blockIdx.x) * QT;
     const int dv0 = (blockIdx.y % nsplit) * DVP;         // first value channel of this split
     const int dvn = min(DVP, Dv - dv0);
     const int rep = H / G;
@@ -756,92 +757,66 @@ paged_attn_mfma_kernel(const bf16* __restrict__ q, long qstride, const bf16* __r
 #pragma unroll
     for (int nb = 0; nb < DVP / 16; ++nb) o_acc[nb] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 
-    // a tile's K and V lines travel global -> registers -> LDS. With PREFETCH
-    // (wide rows: one workgroup per CU, nothing else to hide latency) the next
-    // tile's loads are issued before the current tile's products; without, the
-    // registers are reused and more workgroups share a CU
+    // A tile's K and V lines travel global -> registers -> LDS, all loads of a tile in
+    // flight together: the keys' cache slots are looked up one tile ahead (LDS, two
+    // buffers) and addresses are clamped rather than branched around. With PREFETCH
+    // the next tile's loads are issued before the current tile's products; without,
+    // the registers are reused and more workgroups share a CU.
+    __shared__ int kslot[2][MA_KT];
+#define MA_SLOTS(BASE, BUF)                                                                \
+    if (tid < MA_KT) {                                                                     \
+        const int mm = min((BASE) + tid, n - 1);                                           \
+        const int j = mm < nfirst ? mm : lo + (mm - nfirst);                               \
+        const int blk = bt[j / bsz];                                                       \
+        kslot[BUF][tid] = (blk < 0 ? 0 : blk) * bsz + (j % bsz);                           \
+    }
     constexpr int NKI = (MA_KT * (DKP / 8) + 255) / 256;
     constexpr int NVI = (MA_KT * (DVP / 8) + 255) / 256;
+    const bf16* kbase = kc + (long)g * khead;
+    const bf16* vbase = vc + (long)g * vhead + dv0;
     uint4 rk[NKI], rv[NVI];
-#define MA_FETCH(BASE)                                                                     \
+#define MA_FETCH(BASE, BUF)                                                                \
     {                                                                                      \
         _Pragma("unroll") for (int x = 0; x < NKI; ++x) {                                  \
             const int c = tid + x * 256;                                                   \
-            const int m = c / (DKP / 8), part = c % (DKP / 8);                             \
-            uint4 raw = make_uint4(0, 0, 0, 0);                                            \
-            if (c < MA_KT * (DKP / 8) && (BASE) + m < n && part * 8 < Dk) {                \
-                const int mm = (BASE) + m;                                                 \
-                const int j = mm < nfirst ? mm : lo + (mm - nfirst);                       \
-                const int blk = bt[j / bsz];                                               \
-                const long slot = (long)(blk < 0 ? 0 : blk) * bsz + (j % bsz);             \
-                raw = *reinterpret_cast<const uint4*>(kc + slot * ktok + (long)g * khead + part * 8); \
-            }                                                                              \
-            rk[x] = raw;                                                                   \
+            const int m = min(c / (DKP / 8), MA_KT - 1), part = c % (DKP / 8);             \
+            rk[x] = *reinterpret_cast<const uint4*>(                                       \
+                kbase + (long)kslot[BUF][m] * ktok + min(part * 8, Dk - 8));               \
         }                                                                                  \
         _Pragma("unroll") for (int x = 0; x < NVI; ++x) {                                  \
             const int c = tid + x * 256;                                                   \
             const int m = c % MA_KT, part = c / MA_KT;   /* consecutive lanes: consecutive keys */ \
-            uint4 raw = make_uint4(0, 0, 0, 0);                                            \
-            if (c < MA_KT * (DVP / 8) && (BASE) + m < n && part * 8 < dvn) {               \
-                const int mm = (BASE) + m;                                                 \
-                const int j = mm < nfirst ? mm : lo + (mm - nfirst);                       \
-                const int blk = bt[j / bsz];                                               \
-                const long slot = (long)(blk < 0 ? 0 : blk) * bsz + (j % bsz);             \
-                raw = *reinterpret_cast<const uint4*>(vc + slot * vtok + (long)g * vhead + dv0 + \
-                                                      part * 8);                           \
-            }                                                                              \
-            rv[x] = raw;                                                                   \
+            rv[x] = *reinterpret_cast<const uint4*>(                                       \
+                vbase + (long)kslot[BUF][m] * vtok + min(part * 8, dvn - 8));              \
         }                                                                                  \
     }
-    if constexpr (PREFETCH) MA_FETCH(0)
-    for (int base = 0; base < n; base += MA_KT) {
-        if constexpr (!PREFETCH) {
-            // ---- global -> LDS directly: K row-major, V transposed
-            for (int c = tid; c < MA_KT * (DKP / 8); c += 256) {
-                const int m = c / (DKP / 8), part = c % (DKP / 8);
-                uint4 raw = make_uint4(0, 0, 0, 0);
-                if (base + m < n && part * 8 < Dk) {
-                    const int mm = base + m;
-                    const int j = mm < nfirst ? mm : lo + (mm - nfirst);
-                    const int blk = bt[j / bsz];
-                    const long slot = (long)(blk < 0 ? 0 : blk) * bsz + (j % bsz);
-                    raw = *reinterpret_cast<const uint4*>(kc + slot * ktok + (long)g * khead + part * 8);
-                }
-                *reinterpret_cast<uint4*>(k_lds + m * KS + part * 8) = raw;
-            }
-            for (int c = tid; c < MA_KT * (DVP / 8); c += 256) {
-                const int m = c % MA_KT, part = c / MA_KT;   // consecutive lanes: consecutive keys
-                uint4 raw = make_uint4(0, 0, 0, 0);
-                if (base + m < n && part * 8 < dvn) {
-                    const int mm = base + m;
-                    const int j = mm < nfirst ? mm : lo + (mm - nfirst);
-                    const int blk = bt[j / bsz];
-                    const long slot = (long)(blk < 0 ? 0 : blk) * bsz + (j % bsz);
-                    raw = *reinterpret_cast<const uint4*>(vc + slot * vtok + (long)g * vhead + dv0 +
-                                                          part * 8);
-                }
-                const uint32_t u[4] = {raw.x, raw.y, raw.z, raw.w};
-#pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    vt_lds[(part * 8 + 2 * e) * VS + m] = (uint16_t)(u[e] & 0xffffu);
-                    vt_lds[(part * 8 + 2 * e + 1) * VS + m] = (uint16_t)(u[e] >> 16);
-                }
-            }
-        }
-        // ---- (prefetched) registers -> LDS
-        if constexpr (PREFETCH) {
+    MA_SLOTS(0, 0)
+    __syncthreads();
+    if constexpr (PREFETCH) MA_FETCH(0, 0)
+    int buf = 0;
+    for (int base = 0; base < n; base += MA_KT, buf ^= 1) {
+        if constexpr (!PREFETCH) MA_FETCH(base, buf)
+        if (base + MA_KT < n) MA_SLOTS(base + MA_KT, buf ^ 1)
+        // ---- registers -> LDS: K row-major, V transposed; zeros past the last key
+        // and the last channel
 #pragma unroll
         for (int x = 0; x < NKI; ++x) {
             const int c = tid + x * 256;
+            const int m = c / (DKP / 8), part = c % (DKP / 8);
+            const bool ok = base + m < n && part * 8 < Dk;
+            const uint4 raw = make_uint4(ok ? rk[x].x : 0, ok ? rk[x].y : 0, ok ? rk[x].z : 0,
+                                         ok ? rk[x].w : 0);
             if (c < MA_KT * (DKP / 8))
-                *reinterpret_cast<uint4*>(k_lds + (c / (DKP / 8)) * KS + (c % (DKP / 8)) * 8) = rk[x];
+                *reinterpret_cast<uint4*>(k_lds + m * KS + part * 8) = raw;
         }
 #pragma unroll
         for (int x = 0; x < NVI; ++x) {
             const int c = tid + x * 256;
+            const int m = c % MA_KT, part = c / MA_KT;
+            const bool ok = base + m < n && part * 8 < dvn;
+            const uint32_t u[4] = {ok ? rv[x].x : 0, ok ? rv[x].y : 0, ok ? rv[x].z : 0,
+                                   ok ? rv[x].w : 0};
             if (c < MA_KT * (DVP / 8)) {
-                const int m = c % MA_KT, part = c / MA_KT;
-                const uint32_t u[4] = {rv[x].x, rv[x].y, rv[x].z, rv[x].w};
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
                     vt_lds[(part * 8 + 2 * e) * VS + m] = (uint16_t)(u[e] & 0xffffu);
@@ -849,10 +824,9 @@ paged_attn_mfma_kernel(const bf16* __restrict__ q, long qstride, const bf16* __r
                 }
             }
         }
-        }
         __syncthreads();
         if constexpr (PREFETCH) {
-            if (base + MA_KT < n) MA_FETCH(base + MA_KT) // in flight during the products below
+            if (base + MA_KT < n) MA_FETCH(base + MA_KT, buf ^ 1) // in flight during the products
         }
         // ---- S^T = K Q^T: lane gets keys 16*kb + 4*lg + r of its own row lr
         float sv[KB][4];
@@ -960,6 +934,7 @@ paged_attn_mfma_kernel(const bf16* __restrict__ q, long qstride, const bf16* __r
         __syncthreads();
     }
 #undef MA_FETCH
+#undef MA_SLOTS
     // ---- epilogue: rows 4*lg + r of this wave, channel 16*nb + lr. A sink adds
     // one term to the row's denominator (computed by the lane that owns the row)
     float fin = l_run > 0.f ? 1.f / l_run : 0.f;
