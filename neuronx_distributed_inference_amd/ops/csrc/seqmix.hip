@@ -3443,7 +3443,7 @@ int nx_paged_attn(const void* q, long qstride, const void* kc, long ktok, long k
             const int QTm = MA_ROWS / rp;
             const int nsplit = wide ? (Dv + 127) / 128 : 1;
             dim3 gm((S + QTm - 1) / QTm, G * nsplit, B), bm(256);
-#define MA(DKV, DVV, KTV) paged_attn_mfma_kernel<DKV, DVV, KTV, (KTV == 32)><<<gm, bm, 0, st>>>( \
+#define MA(DKV, DVV, KTV) paged_attn_mfma_kernel<DKV, DVV, KTV, (KTV == 32 || (DKV == 192 && DVV == 128))><<<gm, bm, 0, st>>>( \
         (const bf16*)q, qstride, (const bf16*)kc, (const bf16*)vc, pos, seq, btab, max_blocks, \
         r1, r2, (const bf16*)gate, gstride, (bf16*)out, H, G, Dk, Dv, bsz, S, scale, window, \
         keep, QTm, ktok, khead, vtok, vhead, sink, cap, qt_coef, qt_every, nsplit, ghead, cmask)
