@@ -708,9 +708,15 @@ paged_attn_mfma_kernel(const bf16* __restrict__ q, long qstride, const bf16* __r
     __shared__ float ra1[MA_ROWS], ra2[MA_ROWS], rsink[MA_ROWS];
     const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
     const int lr = lane & 15, lg = lane >> 4;
+    // Workgroups go to the 8 XCDs in turn: renumber them so that an XCD works on
+    // whole heads, whose keys and values then stay in its L2
+    const int nwg = gridDim.x * gridDim.y;
+    int wg = blockIdx.y * gridDim.x + blockIdx.x;
+    if (nwg % 8 == 0) wg = (wg % 8) * (nwg / 8) + wg / 8;
+    const int by = wg / gridDim.x, bx = wg % gridDim.x;
     // the last tokens of a row see the most keys: they start first
-    const int b = blockIdx.z, g = blockIdx.y / nsplit, t0 = (gridDim.x - 1 - blockIdx.x) * QT;
-    const int dv0 = (blockIdx.y % nsplit) * DVP;         // first value channel of this split
+    const int b = blockIdx.z, g = by / nsplit, t0 = (gridDim.x - 1 - bx) * QT;
+    const int dv0 = (by % nsplit) * DVP;         // first value channel of this split
     const int dvn = min(DVP, Dv - dv0);
     const int rep = H / G;
     if (seq[b] < 0) return;
