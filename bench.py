@@ -74,7 +74,9 @@ def parse_args():
                         "attention layers; Kuterax: sink attention + state space in "
                         "parallel, retention, routed experts; Tamilix: chunk-local slope "
                         "attention, windowed gated latent attention, identity-routed "
-                        "experts) beside Llama at equal width/depth/ff/vocab")
+                        "experts; Risutar: latent attention, gated linear attention, "
+                        "routed gelu experts) beside Llama at equal "
+                        "width/depth/ff/vocab")
     p.add_argument("--hybrid-models", default="llama,nabelix,soputar,kuterax,tamilix,risutar",
                    help="comma-separated subset of llama,nabelix,soputar,kuterax,tamilix,"
                         "risutar for --hybrid")
