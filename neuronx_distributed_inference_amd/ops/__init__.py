@@ -428,7 +428,7 @@ def attention_decode(q, k_cache, v_cache, seq_lens, seq_ids=None, scale=None,
             # odd GQA shards (e.g. 96q/8kv models, replicate-to-TP
             # 70B configs): split the q heads per KV head into <=8-wide
             # groups and run the kernel per group (KV re-read per split;
-            # correctness first — VERDICT r01 weak #9)
+            # correctness first)
             half = (gq + 1) // 2
             qg = q.view(B, Hkv, gq, Sq, D)
             outs = []
