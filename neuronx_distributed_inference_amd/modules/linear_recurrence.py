@@ -1,7 +1,8 @@
 """Linear-recurrence token mixer cores with matrix state: the gated delta
 rule (below), selective state spaces (:class:`StateSpaceDuality`),
-retention (:class:`Retention`) and gated linear attention
-(:class:`GatedLinearAttention`).
+retention (:class:`Retention`), gated linear attention
+(:class:`GatedLinearAttention`) and the matrix memory with exponential gates
+(:class:`ExponentialGateMemory`).
 
 Gated delta rule.
 
@@ -245,3 +246,53 @@ class GatedLinearAttention(nn.Module):
         return seqmix.gated_linear_attention(
             q, k, v, log_decay, gate, self.norm_weight, self.eps, states.get(key + ".mem"), step,
             self.dim, self.vdim, k_scale=self.dim ** -0.5)
+
+
+class ExponentialGateMemory(nn.Module):
+    """Matrix memory with exponential input gates and a normalizer (the mLSTM
+    of xLSTM): per head a (dim x vdim) fp32 matrix S, a dim-long vector n and
+    a running maximum m from zero; with the log gates
+
+        i_t = cap tanh(z_i / cap) ,  f_t = log sigmoid(cap tanh(z_f / cap)) ,
+
+        m_t = max(f_t + m_{t-1}, i_t)
+        S_t = exp(f_t + m_{t-1} - m_t) S_{t-1} + exp(i_t - m_t) k_t v_t^T
+        n_t likewise with k_t alone
+        o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6)
+
+    with q scaled by dim^-1/2. Each head's read-out is divided by its root mean
+    square, weighted (one weight per head and channel) and multiplied by the
+    sigmoid of a gate projection.
+
+    The caller owns the q/k/v/gate/z_i/z_f and the output projections; the gate
+    biases live here and enter in fp32. n is kept as one more row of S (that of
+    a value channel which is always one), so one recurrence carries both; S, n
+    and m live in the cache manager's :class:`RecurrentStateManager`.
+    """
+
+    def __init__(self, num_heads: int, dim: int, vdim: int, gate_cap: float, eps: float):
+        super().__init__()
+        self.num_heads = num_heads
+        self.dim = dim
+        self.vdim = vdim
+        self.gate_cap = float(gate_cap)
+        self.eps = float(eps)
+        f32 = dict(dtype=torch.float32)
+        self.i_bias = nn.Parameter(torch.zeros(num_heads, **f32), requires_grad=False)
+        self.f_bias = nn.Parameter(torch.zeros(num_heads, **f32), requires_grad=False)
+        self.norm_weight = nn.Parameter(torch.ones(num_heads * vdim, **f32), requires_grad=False)
+
+    def state_shapes(self):
+        return {"mem": (self.num_heads, self.vdim + 1, self.dim),   # S transposed, then n
+                "max": (self.num_heads,)}
+
+    def forward(self, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torch.Tensor,
+                i_gate: torch.Tensor, f_gate: torch.Tensor, states, key: str,
+                step: seqmix.StepLayout) -> torch.Tensor:
+        """q, k (B,S,H*dim), v, gate (B,S,H*vdim), i_gate, f_gate (B,S,H): raw
+        projections, column slices of one GEMM output are fine. Returns
+        (B,S,H*vdim) in the gate's dtype."""
+        return seqmix.mlstm(
+            q, k, v, i_gate, f_gate, gate, self.i_bias, self.f_bias, self.gate_cap,
+            self.norm_weight, self.eps, states.get(key + ".mem"), states.get(key + ".max"), step,
+            self.dim, self.vdim)

@@ -397,22 +397,27 @@ class MoELayer(nn.Module):
 
 
 class GroupLimitedRouter(nn.Module):
-    """Softmax router whose experts form groups of neighbours: a group scores
-    as its best expert, and only experts of the ``keep_groups`` best groups
+    """Router over softmax (or, ``score="sigmoid"``, sigmoid) scores whose
+    experts form groups of neighbours: a group scores as its best expert (the
+    sum of its two best with ``group_top=2``), and only experts of the ``keep_groups`` best groups
     compete for the ``top_k`` places. The weights are the chosen experts'
-    softmax scores over ALL experts times ``scale`` (renormalised over the
-    chosen ones first when ``normalize``). Logits, softmax and selection are
+    scores over ALL experts times ``scale`` (divided by their sum plus
+    ``norm_eps`` first when ``normalize``). Logits, scores and selection are
     fp32. ``extra_gates`` further rows of the weight are per-token sigmoid
     gates computed by the same fp32 product (a shared expert's gate). With
     ``correction`` a stored per-expert offset is added to the scores for the
-    choice only; the weights stay the uncorrected scores. With ``bias`` a
-    stored offset is part of the logits. ``normalize`` without groups is a
-    softmax over the chosen logits only."""
+    choice (of groups too) only; the weights stay the uncorrected scores. With
+    ``bias`` a stored offset is part of the logits. ``normalize`` of softmax
+    scores without groups is a softmax over the chosen logits only."""
 
     def __init__(self, hidden_size: int, num_experts: int, top_k: int, n_groups: int = 1,
                  keep_groups: int = 1, scale: float = 1.0, normalize: bool = False,
-                 extra_gates: int = 0, correction: bool = False, bias: bool = False):
+                 extra_gates: int = 0, correction: bool = False, bias: bool = False,
+                 score: str = "softmax", group_top: int = 1, norm_eps: float = 0.0):
         super().__init__()
+        self.score = score
+        self.group_top = group_top
+        self.norm_eps = float(norm_eps)
         assert num_experts % max(n_groups, 1) == 0 and top_k <= num_experts
         self.num_experts = num_experts
         self.top_k = top_k
@@ -436,7 +441,8 @@ class GroupLimitedRouter(nn.Module):
 
         return seqmix.route_tokens(x, self.weight, self.num_experts, self.top_k, self.n_groups,
                                    self.keep_groups, self.scale, self.normalize,
-                                   correction=self.correction, bias=self.bias)
+                                   correction=self.correction, bias=self.bias, score=self.score,
+                                   group_top=self.group_top, norm_eps=self.norm_eps)
 
 
 class FusedUngatedExperts(nn.Module):
@@ -487,22 +493,29 @@ class FusedUngatedExperts(nn.Module):
 
 
 class GroupRoutedFeedForward(nn.Module):
-    """Mixture of two-matrix experts (``act``) behind a
-    :class:`GroupLimitedRouter`, with an optional shared expert that runs for
+    """Mixture of two-matrix experts (``act`` relu2 or gelu) or of gated
+    three-matrix experts (``act="silu_glu"``) behind a
+    :class:`GroupLimitedRouter` (``router``: its further options), with an optional shared expert that runs for
     every token (``shared_ff`` = 0: none), scaled by a per-token sigmoid gate
     or, without ``shared_gate``, by one."""
 
     def __init__(self, hidden_size: int, num_experts: int, top_k: int, expert_ff: int,
                  dtype: torch.dtype, n_groups: int = 1, keep_groups: int = 1,
                  scale: float = 1.0, normalize: bool = False, shared_ff: int = 0,
-                 shared_gate: bool = True, act: str = "relu2", router_bias: bool = False):
+                 shared_gate: bool = True, act: str = "relu2", router_bias: bool = False,
+                 router: Optional[dict] = None):
         super().__init__()
         self.router = GroupLimitedRouter(hidden_size, num_experts, top_k, n_groups, keep_groups,
                                          scale, normalize,
                                          extra_gates=1 if shared_ff and shared_gate else 0,
-                                         bias=router_bias)
-        self.experts = FusedUngatedExperts(num_experts, hidden_size, expert_ff, shared_ff, dtype,
-                                           act=act)
+                                         bias=router_bias, **(router or {}))
+        if act == "silu_glu":
+            assert not shared_gate, "gated experts take no gate for the shared one"
+            self.experts = FusedGatedExperts(num_experts, hidden_size, expert_ff, 0.0, dtype,
+                                             shared_ff, act="silu")
+        else:
+            self.experts = FusedUngatedExperts(num_experts, hidden_size, expert_ff, shared_ff,
+                                               dtype, act=act)
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         shape = h.shape
@@ -513,7 +526,8 @@ class GroupRoutedFeedForward(nn.Module):
 
 class FusedGatedExperts(nn.Module):
     """Three-matrix experts ``W_down(g * sigmoid(alpha g) * (u + 1))`` with
-    ``g = min(W_gate x, limit)`` and ``u = clamp(W_up x, +-limit)``, stacked
+    ``g = min(W_gate x, limit)`` and ``u = clamp(W_up x, +-limit)``, or
+    (``act="silu"``) ``W_down(silu(W_gate x) * W_up x)``, stacked
     so that ALL experts and an optional always-on shared expert (own size
     and clamp) are two GEMMs: ``gate_up`` holds the gate rows of every
     expert, then of the shared one, then the up rows in the same order;
@@ -526,8 +540,10 @@ class FusedGatedExperts(nn.Module):
 
     def __init__(self, num_experts: int, hidden_size: int, expert_ff: int, limit: float,
                  dtype: torch.dtype, shared_ff: int = 0, shared_limit: float = 0.0,
-                 alpha: float = 1.702, tp_degree: int = 1):
+                 alpha: float = 1.702, tp_degree: int = 1, act: str = "clamped"):
         super().__init__()
+        assert act in ("clamped", "silu")
+        self.act = act
         from neuronx_distributed_inference_amd.parallel.layers import (
             ColumnParallelLinear,
             RowParallelLinear,
@@ -559,6 +575,9 @@ class FusedGatedExperts(nn.Module):
         from neuronx_distributed_inference_amd.ops import seqmix
 
         hid = self.gate_up(x)
+        if self.act == "silu":
+            return self.down(seqmix.silu_glu_scale(hid, gates, self.expert_ff, self.num_experts,
+                                                   out_dtype=hid.dtype))
         return self.down(seqmix.clamped_glu_scale(
             hid, gates, self.expert_ff, self.num_experts, self.limit, self.shared_limit,
             self.alpha, out_dtype=hid.dtype))

@@ -62,18 +62,18 @@ class LayerNorm(nn.Module):
 
 
 class StreamLayerNorm(nn.Module):
-    """LayerNorm with bias for models whose residual stream is fp32. Besides
+    """LayerNorm (with or without ``bias``) for models whose residual stream is fp32. Besides
     the plain call, :meth:`sum_into` does the residual step of designs that
     norm after the sum, ``stream = norm(alpha * stream + y)``, in one kernel
     and hands back the new stream in the next GEMM's input dtype."""
 
     def __init__(self, hidden_size: int, eps: float = 1e-5,
-                 out_dtype: torch.dtype = torch.float32):
+                 out_dtype: torch.dtype = torch.float32, bias: bool = True):
         super().__init__()
         self.weight = nn.Parameter(torch.ones(hidden_size, dtype=torch.float32),
                                    requires_grad=False)
         self.bias = nn.Parameter(torch.zeros(hidden_size, dtype=torch.float32),
-                                 requires_grad=False)
+                                 requires_grad=False) if bias else None
         self.eps = float(eps)
         self.out_dtype = out_dtype
 
@@ -86,6 +86,7 @@ class StreamLayerNorm(nn.Module):
     def sum_into(self, stream: torch.Tensor, y: torch.Tensor, alpha: float, copy_dtype=None):
         from neuronx_distributed_inference_amd.ops import seqmix
 
+        assert self.bias is not None
         return seqmix.add_layer_norm(stream, y, alpha, self.weight, self.bias, self.eps,
                                      copy_dtype)
 

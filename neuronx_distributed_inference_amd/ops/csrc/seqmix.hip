@@ -1554,6 +1554,28 @@ template <> DEV void store8<bf16>(bf16* p, const float* v) {
     *reinterpret_cast<uint4*>(p) = make_uint4(pk[0], pk[1], pk[2], pk[3]);
 }
 
+// 4 consecutive elements as floats, one 8- or 16-byte access
+template <typename T> DEV void load4(const T* p, float* v);
+template <> DEV void load4<bf16>(const bf16* p, float* v) {
+    const uint2 raw = *reinterpret_cast<const uint2*>(p);
+    v[0] = __uint_as_float(raw.x << 16); v[1] = __uint_as_float(raw.x & 0xffff0000u);
+    v[2] = __uint_as_float(raw.y << 16); v[3] = __uint_as_float(raw.y & 0xffff0000u);
+}
+template <> DEV void load4<float>(const float* p, float* v) {
+    const float4 a = *reinterpret_cast<const float4*>(p);
+    v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
+}
+template <typename T> DEV void store4(T* p, const float* v);
+template <> DEV void store4<float>(float* p, const float* v) {
+    *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+}
+template <> DEV void store4<bf16>(bf16* p, const float* v) {
+    union { bf16 h[4]; uint2 u; } x;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) x.h[e] = __float2bfloat16(v[e]);
+    *reinterpret_cast<uint2*>(p) = x.u;
+}
+
 template <typename TIn, typename TOut>
 __global__ void __launch_bounds__(LN_THREADS)
 rms_norm_vec_kernel(const TIn* __restrict__ x, long xs, const float* __restrict__ w, int one_plus,
@@ -1916,8 +1938,10 @@ head_norm_rope_kernel(const TIn* __restrict__ x, long xt, long xh, TOut* __restr
 // are staged through LDS in chunks of DS_TC (q, k, v, decay, step size), so
 // global loads are coalesced and the serial loop reads only LDS.
 // Decay: selective (dt projection + dt_bias, a_log: w = softplus(dt + bias),
-// a = exp(-exp(a_log) w)) or fixed per head (head_decay: a = decay, w = 1). CH takes
-// `dt` (H*D wide, fp32) as the decays' logarithms.
+// a = exp(-exp(a_log) w)), fixed per head (head_decay: a = decay, w = 1), or given
+// (wgt: a = exp(dt), w = wgt, both per head and token). CH takes
+// `dt` (H*D wide, fp32) as the decays' logarithms. `ones`: the last of the Dv value
+// channels is not read but one (a normalizer row).
 //
 // Long rows with few workgroups are cut into `nseg` segments of `seglen`
 // tokens that run side by side; the recurrence is linear in the state, so
@@ -1941,7 +1965,7 @@ decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, lon
                   const int* __restrict__ pos, const int* __restrict__ seq,
                   const int* __restrict__ nvalid, float* __restrict__ out, int S, int H, int G,
                   int D, int Dv, float* __restrict__ ws, float* __restrict__ wdec, int nseg,
-                  int seglen) {
+                  int seglen, const float* __restrict__ wgt, int ones) {
     constexpr int DP = 16 * R;
     __shared__ __attribute__((aligned(16))) float sd[CH ? DS_TC : 1][CH ? DP : 4];
     __shared__ __attribute__((aligned(16))) float sq[MODE == 1 ? 1 : DS_TC][DP], sk[DS_TC][DP];
@@ -2009,12 +2033,17 @@ decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, lon
             const int tt = tid >> 4, cc = tid & 15;       // 256 = DS_TC * 16
             float vv = 0.f;
             if (tt < cnt && c0 + cc < Dv)
-                vv = ldf<T>(v + ((long)b * S + t0 + tt) * vs + (long)h * Dv + c0 + cc);
+                vv = ones && c0 + cc == Dv - 1 ? 1.f
+                    : ldf<T>(v + ((long)b * S + t0 + tt) * vs + (long)h * (Dv - ones) + c0 + cc);
             sv[tt][cc] = vv;
         }
         if (!CH && tid < cnt) {
             float a, w = 1.f;
-            if (dt) {
+            if (wgt) {
+                const long tok = (long)b * S + t0 + tid;
+                w = wgt[tok * H + h];
+                a = expf(ldf<TD>(dt + tok * dts + h));
+            } else if (dt) {
                 w = softplusf_(ldf<TD>(dt + ((long)b * S + t0 + tid) * dts + h) + dt_bias[h]);
                 a = expf(-expf(a_log[h]) * w);
             } else {
@@ -2346,26 +2375,27 @@ gla_chunk_state_kernel(const bf16* __restrict__ k, long ks, const bf16* __restri
 }
 
 // start states of the chunks, in place over their contributions, and the carried
-// state; eight chunks' loads are in flight at a time. A start state leaves as its two
+// state (dch: decay channels, the key dimension or 1); eight chunks' loads are in
+// flight at a time. A start state leaves as its two
 // bf16 terms (the high one in the high half of the word), ready for the read-out.
 __global__ void __launch_bounds__(256)
 gla_chunk_link_kernel(float* __restrict__ ws, const float* __restrict__ wdec,
                       float* __restrict__ state, const int* __restrict__ pos,
                       const int* __restrict__ seq, const int* __restrict__ nvalid, int B, int S,
-                      int H, int D, long per_head, int nc) {
+                      int H, int dch, long per_head, int nc) {
     const long total = (long)B * H * per_head;
     for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < total;
          i += (long)gridDim.x * blockDim.x) {
         const long e = i % per_head;
-        const int h = (i / per_head) % H, b = i / (per_head * H), d = e % D;
+        const int h = (i / per_head) % H, b = i / (per_head * H), d = dch > 1 ? e % dch : 0;
         const int slot = seq[b], n = slot < 0 ? 0 : nvalid[b];
         if (n <= 0) continue;
         const int chunks = (n + GC_N - 1) / GC_N;
         float* sp = state + ((long)slot * H + h) * per_head + e;
         float s = pos[(long)b * S] > 0 ? *sp : 0.f;
         float* wp = ws + ((long)b * nc * H + h) * per_head + e;
-        const float* dp = wdec + ((long)b * nc * H + h) * D + d;
-        const long wst = (long)H * per_head, dst = (long)H * D;
+        const float* dp = wdec + ((long)b * nc * H + h) * dch + d;
+        const long wst = (long)H * per_head, dst = (long)H * dch;
         for (int c0 = 0; c0 < chunks; c0 += 8) {
             float en[8], dc[8];
 #pragma unroll
@@ -2696,11 +2726,13 @@ __global__ void group_gated_norm_kernel(const float* __restrict__ y, const TG* _
 }
 
 // ------------------------------------------------------- group-limited router
-// One wave per token: softmax over E logits (fp32), group score = best expert of
-// the group, `keep` best groups stay, `top` best experts among them are chosen
+// One wave per token: scores = softmax over E logits or their sigmoids (fp32), group
+// score = best expert of the group or (gtwo) the sum of its two best, `keep` best
+// groups stay, `top` best experts among them are chosen
 // (ties: lowest index). Writes the dense (T, E + extra) weight row (zeros at
 // unchosen experts, sigmoid gates in the extra columns), the chosen indices and
-// their weights = score * scale (renormalised over the chosen first if asked).
+// their weights = score * scale (renormalised over the chosen first if asked, the
+// sum plus norm_eps).
 // `corr` (E, or null) is added to the scores for the group ranking and the choice
 // only.
 // A row whose logits are not numbers (the garbage of a pad token) selects the
@@ -2719,18 +2751,27 @@ DEV void wave_argmax(float& v, int& i) {
 // `dp`, chosen indices `idx` and weights `wts`; `cand` is 2E + ngroups floats of
 // LDS scratch
 DEV void route_select_(const float* lp, int E, int extra, int top, int ngroups, int keep,
-                       float scale, int normalize, const float* __restrict__ corr, float* cand,
+                       float scale, int normalize, const float* __restrict__ corr, int sig,
+                       int gtwo, float norm_eps, float* cand,
                        float* __restrict__ dp, int* __restrict__ idx, float* __restrict__ wts,
                        int lane) {
     float* gsc = cand + E;
     float* sco = gsc + ngroups;                   // the uncorrected scores (the weights)
-    float m = -INFINITY;
-    for (int e = lane; e < E; e += WAVE) m = fmaxf(m, lp[e]);
-    m = wave_max(m);
-    float sum = 0.f;
-    for (int e = lane; e < E; e += WAVE) { const float x = expf(lp[e] - m); cand[e] = x; sum += x; }
-    sum = wave_sum(sum);
-    const float rs = 1.f / sum;
+    float rs = 1.f;
+    if (sig) {                                    // uniform
+        for (int e = lane; e < E; e += WAVE) cand[e] = sigmoidf_(lp[e]);
+    } else {
+        float m = -INFINITY;
+        for (int e = lane; e < E; e += WAVE) m = fmaxf(m, lp[e]);
+        m = wave_max(m);
+        float sum = 0.f;
+        for (int e = lane; e < E; e += WAVE) {
+            const float x = expf(lp[e] - m);
+            cand[e] = x;
+            sum += x;
+        }
+        rs = 1.f / wave_sum(sum);
+    }
     for (int e = lane; e < E; e += WAVE) {
         const float sc = cand[e] * rs;
         sco[e] = sc;
@@ -2742,9 +2783,13 @@ DEV void route_select_(const float* lp, int E, int extra, int top, int ngroups, 
     const int per = E / ngroups;
     if (ngroups > 1 && keep < ngroups) {
         for (int gi = lane; gi < ngroups; gi += WAVE) {
-            float gm = -INFINITY;
-            for (int j = 0; j < per; ++j) gm = fmaxf(gm, cand[gi * per + j]);
-            gsc[gi] = gm;
+            float g1 = -INFINITY, g2 = -INFINITY;         // the two best of the group
+            for (int j = 0; j < per; ++j) {
+                const float x = cand[gi * per + j];
+                g2 = fmaxf(g2, fminf(g1, x));
+                g1 = fmaxf(g1, x);
+            }
+            gsc[gi] = gtwo && per > 1 ? g1 + g2 : g1;
         }
         __builtin_amdgcn_wave_barrier();
         for (int r = 0; r < keep; ++r) {
@@ -2781,7 +2826,7 @@ DEV void route_select_(const float* lp, int E, int extra, int top, int ngroups, 
         wsum += bv;
         __builtin_amdgcn_wave_barrier();
     }
-    const float f = normalize ? scale / wsum : scale;
+    const float f = normalize ? scale / (wsum + norm_eps) : scale;
     if (top <= WAVE) {
         if (lane < top) {
             idx[lane] = myi;
@@ -2794,15 +2839,15 @@ DEV void route_select_(const float* lp, int E, int extra, int top, int ngroups, 
 __global__ void __launch_bounds__(RT_WAVES * WAVE)
 group_router_kernel(const float* __restrict__ logits, long ls, int E, int extra, int top,
                     int ngroups, int keep, float scale, int normalize,
-                    const float* __restrict__ corr,
+                    const float* __restrict__ corr, int sig, int gtwo, float norm_eps,
                     float* __restrict__ dense, int* __restrict__ idx, float* __restrict__ wts,
                     long T) {
     extern __shared__ float rsm[];                // per wave: E choice scores + ngroups + E scores
     const int lane = threadIdx.x & (WAVE - 1), wv = threadIdx.x / WAVE;
     const long t = (long)blockIdx.x * RT_WAVES + wv;
     if (t >= T) return;
-    route_select_(logits + t * ls, E, extra, top, ngroups, keep, scale, normalize, corr,
-                  rsm + (long)wv * (2 * E + ngroups), dense + t * (long)(E + extra),
+    route_select_(logits + t * ls, E, extra, top, ngroups, keep, scale, normalize, corr, sig,
+                  gtwo, norm_eps, rsm + (long)wv * (2 * E + ngroups), dense + t * (long)(E + extra),
                   idx + t * top, wts + t * top, lane);
 }
 
@@ -2816,7 +2861,8 @@ template <typename T>
 __global__ void __launch_bounds__(RT_WAVES * WAVE)
 router_fused_kernel(const T* __restrict__ x, long xs, const float* __restrict__ w, int W, int vec,
                     int E, int extra, int top, int ngroups, int keep, float scale, int normalize,
-                    const float* __restrict__ corr, const float* __restrict__ bias,
+                    const float* __restrict__ corr, const float* __restrict__ bias, int sig,
+                    int gtwo, float norm_eps,
                     float* __restrict__ dense, int* __restrict__ idx, float* __restrict__ wts) {
     extern __shared__ float rsm[];                // E + extra logits, then the selection scratch
     __shared__ float part[RT_WAVES][8];
@@ -2864,7 +2910,8 @@ router_fused_kernel(const T* __restrict__ x, long xs, const float* __restrict__ 
         __syncthreads();
     }
     if (wv != 0) return;
-    route_select_(rsm, E, extra, top, ngroups, keep, scale, normalize, corr, rsm + E + extra,
+    route_select_(rsm, E, extra, top, ngroups, keep, scale, normalize, corr, sig, gtwo,
+                  norm_eps, rsm + E + extra,
                   dense + t * (long)(E + extra), idx + t * top, wts + t * top, lane);
 }
 
@@ -2918,16 +2965,20 @@ __global__ void act_scale_vec_kernel(const T* __restrict__ x, const float* __res
     }
 }
 
-// --------------------------------- clamped gated units of stacked experts
+// ----------------------------------------- gated units of stacked experts
 // x (rows, 2C) = [gate | up] pre-activations of C = E*ff + shared columns.
 // out[t, c] = glu(gate, up; limit) * gates[t, c / ff] for c < E*ff (an expert's
 // columns, times the token's routing weight), glu(gate, up; shared_limit) for the
-// rest (an always-on shared expert); glu = g sigmoid(alpha g) (u + 1) on the
-// clamped pre-activations.
-template <typename T>
-__global__ void clamped_glu_scale_kernel(const T* __restrict__ x, const float* __restrict__ gates,
-                                         long gs, int ff, int E, float limit, float slimit,
-                                         float alpha, T* __restrict__ out, long rows, int C) {
+// rest (an always-on shared expert). ACT 0: glu = g sigmoid(alpha g) (u + 1) on the
+// clamped pre-activations; ACT 1: glu = g sigmoid(g) u, no clamp.
+template <int ACT> DEV float expert_glu_(float g, float u, float limit, float alpha) {
+    return ACT == 0 ? clamped_glu_(g, u, limit, alpha) : g * sigmoidf_(g) * u;
+}
+
+template <typename T, int ACT>
+__global__ void glu_scale_kernel(const T* __restrict__ x, const float* __restrict__ gates,
+                                 long gs, int ff, int E, float limit, float slimit,
+                                 float alpha, T* __restrict__ out, long rows, int C) {
     const long total = rows * C;
     const int ne = E * ff;
     for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < total;
@@ -2938,17 +2989,17 @@ __global__ void clamped_glu_scale_kernel(const T* __restrict__ x, const float* _
         const float gw = own ? gates[t * gs + c / ff] : 1.f;
         float o = 0.f;
         if (gw != 0.f)
-            o = clamped_glu_(ldf<T>(x + t * 2 * C + c), ldf<T>(x + t * 2 * C + C + c),
-                             own ? limit : slimit, alpha) * gw;
+            o = expert_glu_<ACT>(ldf<T>(x + t * 2 * C + c), ldf<T>(x + t * 2 * C + C + c),
+                                 own ? limit : slimit, alpha) * gw;
         stf<T>(out + i, o);
     }
 }
 
-template <typename T>
-__global__ void clamped_glu_scale_vec_kernel(const T* __restrict__ x,
-                                             const float* __restrict__ gates, long gs, int ff,
-                                             int E, float limit, float slimit, float alpha,
-                                             T* __restrict__ out, long rows, int C) {
+template <typename T, int ACT>
+__global__ void glu_scale_vec_kernel(const T* __restrict__ x,
+                                     const float* __restrict__ gates, long gs, int ff,
+                                     int E, float limit, float slimit, float alpha,
+                                     T* __restrict__ out, long rows, int C) {
     const int C8 = C / 8;
     const long total = rows * C8;
     const int ne = E * ff;
@@ -2965,7 +3016,7 @@ __global__ void clamped_glu_scale_vec_kernel(const T* __restrict__ x,
             load8<T>(x + t * 2 * C + C + c, u);
             const float lim = own ? limit : slimit;
 #pragma unroll
-            for (int e = 0; e < 8; ++e) o[e] = clamped_glu_(g[e], u[e], lim, alpha) * gw;
+            for (int e = 0; e < 8; ++e) o[e] = expert_glu_<ACT>(g[e], u[e], lim, alpha) * gw;
         } else {
 #pragma unroll
             for (int e = 0; e < 8; ++e) o[e] = 0.f;
@@ -3268,6 +3319,793 @@ scaled_residual_kernel(float* __restrict__ x, const T* __restrict__ y0,
 }
 
 // =================================================================== C ABI
+// ------------------------------------------------- parallel residual streams
+// A token's residual is NS streams of C channels (fp32). One step: every stream anew
+// from the old ones, x_t = sum_s mix[s, t] x_s + wout[t] * y (y null: the streams are
+// only read), then u = sum_t win[t] x_t (win null: their plain sum) and, with nw, its
+// layer norm (mean, variance of the deviations, weight, no bias) in the next GEMM's
+// type, else u itself in fp32. `xstr` is the distance between a token's streams in
+// `xin`; 0 reads one row for all of them (streams that still equal the embedding).
+// One workgroup per token. The vector form reads and writes each operand once (new
+// streams go straight out, u stays in registers) and may run in place.
+template <typename T, int NS, int NV>
+__global__ void __launch_bounds__(LN_THREADS)
+hyper_step_vec_kernel(const float* xin, long xrow, long xstr, const T* __restrict__ y,
+                      const float* __restrict__ mix, const float* __restrict__ wout, float* xout,
+                      const float* __restrict__ win, const float* __restrict__ nw, float eps,
+                      T* __restrict__ hout, float* __restrict__ uout, int C) {
+    __shared__ float red[LN_THREADS / WAVE];
+    const long row = blockIdx.x;
+    float wi[NS];
+#pragma unroll
+    for (int t = 0; t < NS; ++t) wi[t] = win ? win[t] : 1.f;
+    float u[NV][4];
+    float sum = 0.f;
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+        const int c = (j * LN_THREADS + threadIdx.x) * 4;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) u[j][e] = 0.f;
+        if (c >= C) continue;
+        float x[NS][4], yv[4];
+#pragma unroll
+        for (int s = 0; s < NS; ++s) {
+            const float4 v = *reinterpret_cast<const float4*>(xin + row * xrow + s * xstr + c);
+            x[s][0] = v.x; x[s][1] = v.y; x[s][2] = v.z; x[s][3] = v.w;
+        }
+        if (y) {
+            load4<T>(y + row * C + c, yv);
+#pragma unroll
+            for (int t = 0; t < NS; ++t) {
+                float o[4];
+                const float wo = wout[t];
+#pragma unroll
+                for (int e = 0; e < 4; ++e) o[e] = wo * yv[e];
+#pragma unroll
+                for (int s = 0; s < NS; ++s) {
+                    const float m = mix[s * NS + t];
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) o[e] += m * x[s][e];
+                }
+                if (xout)
+                    *reinterpret_cast<float4*>(xout + (row * NS + t) * (long)C + c) =
+                        make_float4(o[0], o[1], o[2], o[3]);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) u[j][e] += wi[t] * o[e];
+            }
+        } else {
+#pragma unroll
+            for (int t = 0; t < NS; ++t)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) u[j][e] += wi[t] * x[t][e];
+        }
+        if (!nw)
+            *reinterpret_cast<float4*>(uout + row * C + c) =
+                make_float4(u[j][0], u[j][1], u[j][2], u[j][3]);
+        sum += u[j][0] + u[j][1] + u[j][2] + u[j][3];
+    }
+    if (!nw) return;                                      // uniform
+    const float mean = block_sum(sum, red) / C;
+    float q = 0.f;
+#pragma unroll
+    for (int j = 0; j < NV; ++j)
+        if ((j * LN_THREADS + threadIdx.x) * 4 < C)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) { u[j][e] -= mean; q += u[j][e] * u[j][e]; }
+    const float inv = 1.f / sqrtf(block_sum(q, red) / C + eps);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+        const int c = (j * LN_THREADS + threadIdx.x) * 4;
+        if (c >= C) continue;
+        const float4 w4 = *reinterpret_cast<const float4*>(nw + c);
+        const float o[4] = {u[j][0] * inv * w4.x, u[j][1] * inv * w4.y, u[j][2] * inv * w4.z,
+                            u[j][3] * inv * w4.w};
+        store4<T>(hout + row * C + c, o);
+    }
+}
+
+// scalar form: any number of streams, width and alignment; not in place
+template <typename T>
+__global__ void __launch_bounds__(LN_THREADS)
+hyper_step_kernel(const float* __restrict__ xin, long xrow, long xstr, const T* __restrict__ y,
+                  const float* __restrict__ mix, const float* __restrict__ wout,
+                  float* __restrict__ xout, const float* __restrict__ win,
+                  const float* __restrict__ nw, float eps, T* __restrict__ hout,
+                  float* __restrict__ uout, float* __restrict__ scratch, int NS, int C) {
+    __shared__ float red[LN_THREADS / WAVE];
+    const long row = blockIdx.x;
+    const float* xr = xin + row * xrow;
+    float* ur = (nw ? scratch : uout) + row * C;          // re-read by the same thread only
+    float sum = 0.f;
+    for (int c = threadIdx.x; c < C; c += LN_THREADS) {
+        float u = 0.f;
+        const float yv = y ? ldf<T>(y + row * C + c) : 0.f;
+        for (int t = 0; t < NS; ++t) {
+            float o;
+            if (y) {
+                o = wout[t] * yv;
+                for (int s = 0; s < NS; ++s) o += mix[s * NS + t] * xr[s * xstr + c];
+                if (xout) xout[(row * NS + t) * (long)C + c] = o;
+            } else {
+                o = xr[t * xstr + c];
+            }
+            u += (win ? win[t] : 1.f) * o;
+        }
+        ur[c] = u;
+        sum += u;
+    }
+    if (!nw) return;                                      // uniform
+    const float mean = block_sum(sum, red) / C;
+    float q = 0.f;
+    for (int c = threadIdx.x; c < C; c += LN_THREADS) { const float d = ur[c] - mean; q += d * d; }
+    const float inv = 1.f / sqrtf(block_sum(q, red) / C + eps);
+    for (int c = threadIdx.x; c < C; c += LN_THREADS)
+        stf<T>(hout + row * C + c, (ur[c] - mean) * inv * nw[c]);
+}
+
+// ------------------------------------- attention rows of a step in one launch
+// Queries and keys of a token: rotary positions (half-split pairs i, i + half of the
+// first 2*half channels, fp32 angle pos * inv_freq[i]; half = 0: none), then (unorm)
+// divided by the head's root mean square over D; queries go to a dense buffer, keys
+// into the token's page slot. Values, optionally mixed with another layer's values of
+// the same token, v' = (1 - lam) v + lam v_first (fp32), go into the page slot as they
+// come. One workgroup per token: the angles' cosines and sines are made once for all
+// heads. Pad tokens get zero queries and write no page.
+template <typename T>
+__global__ void __launch_bounds__(256)
+qkv_rows_vec_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, long ks,
+                    const T* __restrict__ v, long vs, const T* __restrict__ vf, long vfs,
+                    const float* __restrict__ lam, const int* __restrict__ pos,
+                    const int* __restrict__ slots, const float* __restrict__ inv_freq, int half,
+                    int unorm, float eps, T* __restrict__ qo, T* __restrict__ kc,
+                    T* __restrict__ vc, long nslots, int H, int G, int D, int Dv, int lanes) {
+    __shared__ __attribute__((aligned(16))) float cs[HN_MAXC / 2], sn[HN_MAXC / 2];
+    const long tok = blockIdx.x;
+    const int tid = threadIdx.x;
+    const int p = pos[tok];
+    if (p < 0) {
+        const float z[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+        for (int c = tid * 8; c < H * D; c += 256 * 8) store8<T>(qo + tok * H * D + c, z);
+        return;
+    }
+    for (int i = tid; i < half; i += 256) {
+        float s_, c_;
+        sincosf((float)p * inv_freq[i], &s_, &c_);
+        cs[i] = c_;
+        sn[i] = s_;
+    }
+    const long slot = slots[tok];
+    const bool wr = slot >= 0 && slot < nslots;
+    if (wr) {
+        const float l = vf ? *lam : 0.f;
+        for (int c = tid * 8; c < G * Dv; c += 256 * 8) {
+            float x[8];
+            load8<T>(v + tok * vs + c, x);
+            if (vf) {
+                float f[8];
+                load8<T>(vf + tok * vfs + c, f);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) x[e] = (1.f - l) * x[e] + l * f[e];
+            }
+            store8<T>(vc + slot * (long)(G * Dv) + c, x);
+        }
+    }
+    __syncthreads();
+    // `lanes` (a power of two, at most a wave) neighbours share a head, 8 channels each
+    const int li = tid % lanes, c = li * 8;
+    for (int u = tid / lanes; u < H + G; u += 256 / lanes) {
+        const bool isq = u < H;
+        const T* xp = isq ? q + tok * qs + (long)u * D : k + tok * ks + (long)(u - H) * D;
+        float x[8];
+        float ss = 0.f;
+        const bool ok = c < D;
+        if (ok) {
+            load8<T>(xp + c, x);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) ss += x[e] * x[e];
+        }
+        float inv = 1.f;                                  // rotation leaves the norm as it is
+        if (unorm) {
+            for (int o = lanes / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, WAVE);
+            inv = 1.f / sqrtf(ss / D + eps);
+        }
+        if (!ok) continue;
+        if (c < 2 * half) {
+            const bool lo = c < half;
+            const int a = lo ? c : c - half;
+            float w[8], cv[8], sv[8];
+            load8<T>(xp + (lo ? c + half : a), w);        // the partner channels
+            load8<float>(cs + a, cv);
+            load8<float>(sn + a, sv);
+#pragma unroll
+            for (int e = 0; e < 8; ++e)
+                x[e] = lo ? x[e] * cv[e] - w[e] * sv[e] : x[e] * cv[e] + w[e] * sv[e];
+        }
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[e] *= inv;
+        if (isq) store8<T>(qo + (tok * H + u) * (long)D + c, x);
+        else if (wr) store8<T>(kc + (slot * G + (u - H)) * (long)D + c, x);
+    }
+}
+
+// scalar form: any sizes and alignment; a wave per head
+template <typename T>
+__global__ void __launch_bounds__(256)
+qkv_rows_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, long ks,
+                const T* __restrict__ v, long vs, const T* __restrict__ vf, long vfs,
+                const float* __restrict__ lam, const int* __restrict__ pos,
+                const int* __restrict__ slots, const float* __restrict__ inv_freq, int half,
+                int unorm, float eps, T* __restrict__ qo, T* __restrict__ kc,
+                T* __restrict__ vc, long nslots, int H, int G, int D, int Dv) {
+    __shared__ float cs[HN_MAXC / 2], sn[HN_MAXC / 2];
+    const long tok = blockIdx.x;
+    const int tid = threadIdx.x, lane = tid & (WAVE - 1), wv = tid / WAVE;
+    const int p = pos[tok];
+    if (p < 0) {
+        for (int c = tid; c < H * D; c += 256) stf<T>(qo + tok * H * D + c, 0.f);
+        return;
+    }
+    for (int i = tid; i < half; i += 256) {
+        float s_, c_;
+        sincosf((float)p * inv_freq[i], &s_, &c_);
+        cs[i] = c_;
+        sn[i] = s_;
+    }
+    const long slot = slots[tok];
+    const bool wr = slot >= 0 && slot < nslots;
+    if (wr) {
+        const float l = vf ? *lam : 0.f;
+        for (int c = tid; c < G * Dv; c += 256) {
+            float x = ldf<T>(v + tok * vs + c);
+            if (vf) x = (1.f - l) * x + l * ldf<T>(vf + tok * vfs + c);
+            stf<T>(vc + slot * (long)(G * Dv) + c, x);
+        }
+    }
+    __syncthreads();
+    for (int u = wv; u < H + G; u += 4) {
+        const bool isq = u < H;
+        const T* xp = isq ? q + tok * qs + (long)u * D : k + tok * ks + (long)(u - H) * D;
+        T* op = isq ? qo + (tok * H + u) * (long)D
+                    : (wr ? kc + (slot * G + (u - H)) * (long)D : nullptr);
+        float inv = 1.f;
+        if (unorm) {
+            float ss = 0.f;
+            for (int c = lane; c < D; c += WAVE) { const float x = ldf<T>(xp + c); ss += x * x; }
+            inv = 1.f / sqrtf(wave_sum(ss) / D + eps);
+        }
+        if (!op) continue;                                // wave-uniform
+        for (int i = lane; i < half; i += WAVE) {
+            const float a = ldf<T>(xp + i), b = ldf<T>(xp + i + half);
+            stf<T>(op + i, (a * cs[i] - b * sn[i]) * inv);
+            stf<T>(op + i + half, (b * cs[i] + a * sn[i]) * inv);
+        }
+        for (int c = 2 * half + lane; c < D; c += WAVE) stf<T>(op + c, ldf<T>(xp + c) * inv);
+    }
+}
+
+// -------------------------------------- matrix memory with exponential gates
+// Per head: log input gate i = cap tanh(z_i / cap), log forget gate f = log sigmoid(cap
+// tanh(z_f / cap)) (z with their fp32 biases), running maximum m_t = max(f + m_{t-1}, i)
+// from m = 0; S_t = a_t S_{t-1} + w_t k v^T and n_t likewise with k alone, a_t = exp(f +
+// m_{t-1} - m_t), w_t = exp(i - m_t), o = S^T q / (max(|n.q|, exp(-m)) + 1e-6). The
+// state of a head is (Dv + 1) rows of D key channels: a row per value channel, then n
+// (the row of a value channel that is always one). Both exponents are never positive.
+DEV void mlstm_gate_(float zi, float zf, float cap, float& i, float& f) {
+    i = cap * tanhf(zi / cap);
+    const float x = cap * tanhf(zf / cap);
+    f = fminf(x, 0.f) - log1pf(expf(-fabsf(x)));
+}
+
+#define MG_THREADS 512
+// One workgroup per (row, head): log a, w and m of every token of the step, and the
+// carried m. A thread owns consecutive tokens; (sum of f, running maximum from minus
+// infinity) pairs of the threads' spans are combined by a scan, then every thread
+// walks its span from its true start.
+template <typename T>
+__global__ void __launch_bounds__(MG_THREADS)
+mlstm_gates_kernel(const T* __restrict__ zi, long zis, const T* __restrict__ zf, long zfs,
+                   const float* __restrict__ bi, const float* __restrict__ bf, float cap,
+                   float* __restrict__ mstate, const int* __restrict__ pos,
+                   const int* __restrict__ seq, const int* __restrict__ nvalid,
+                   float* __restrict__ ld, float* __restrict__ wt, float* __restrict__ mx,
+                   int S, int H) {
+    __shared__ float wf[MG_THREADS / WAVE], wm[MG_THREADS / WAVE];
+    const int h = blockIdx.x, b = blockIdx.y;
+    const int slot = seq[b], n = slot < 0 ? 0 : nvalid[b];
+    if (n <= 0) return;                                   // uniform
+    const int tid = threadIdx.x, lane = tid & (WAVE - 1), wv = tid / WAVE;
+    const int per = (n + MG_THREADS - 1) / MG_THREADS;
+    const int t0 = min(n, tid * per), t1 = min(n, t0 + per);
+    const float bih = bi[h], bfh = bf[h];
+    const long tok0 = (long)b * S;
+    float F = 0.f, M = -INFINITY;
+    for (int t = t0; t < t1; ++t) {
+        float i, f;
+        mlstm_gate_(ldf<T>(zi + (tok0 + t) * zis + h) + bih,
+                    ldf<T>(zf + (tok0 + t) * zfs + h) + bfh, cap, i, f);
+        F += f;
+        M = fmaxf(M + f, i);
+    }
+    float pf = F, pm = M;                                 // inclusive over the wave
+#pragma unroll
+    for (int o = 1; o < WAVE; o <<= 1) {
+        const float of = __shfl_up(pf, o, WAVE), om = __shfl_up(pm, o, WAVE);
+        if (lane >= o) { pm = fmaxf(om + pf, pm); pf += of; }
+    }
+    if (lane == WAVE - 1) { wf[wv] = pf; wm[wv] = pm; }
+    __syncthreads();
+    float m = pos[tok0] > 0 ? mstate[(long)slot * H + h] : 0.f;
+    for (int x = 0; x < wv; ++x) m = fmaxf(m + wf[x], wm[x]);
+    const float ef = __shfl_up(pf, 1, WAVE), em = __shfl_up(pm, 1, WAVE);
+    if (lane > 0) m = fmaxf(m + ef, em);
+    for (int t = t0; t < t1; ++t) {
+        float i, f;
+        mlstm_gate_(ldf<T>(zi + (tok0 + t) * zis + h) + bih,
+                    ldf<T>(zf + (tok0 + t) * zfs + h) + bfh, cap, i, f);
+        const float kept = f + m;
+        m = fmaxf(kept, i);
+        const long at = (tok0 + t) * H + h;
+        ld[at] = kept - m;
+        wt[at] = expf(i - m);
+        mx[at] = m;
+    }
+    __syncthreads();                                      // every thread has read the carried m
+    if (t1 == n && t0 < n) mstate[(long)slot * H + h] = m;
+}
+
+// Read-out of the scan's rows o (rows, H, Dv + 1) fp32: a wave per (token, head)
+// divides by the normalizer, then by the head's root mean square, times the weight
+// (H * Dv) and the sigmoid of the gate.
+template <typename T>
+__global__ void mlstm_readout_kernel(const float* __restrict__ o, const float* __restrict__ mx,
+                                     const T* __restrict__ gate, long gs,
+                                     const float* __restrict__ nw, float eps,
+                                     const int* __restrict__ pos, T* __restrict__ out, long rows,
+                                     int H, int Dv) {
+    const int lane = threadIdx.x & (WAVE - 1);
+    const long id = (long)blockIdx.x * (blockDim.x / WAVE) + threadIdx.x / WAVE;
+    if (id >= rows * H) return;
+    const long row = id / H;
+    const int h = id % H;
+    T* op = out + row * (long)H * Dv + (long)h * Dv;
+    if (pos[row] < 0) {
+        for (int c = lane; c < Dv; c += WAVE) stf<T>(op + c, 0.f);
+        return;
+    }
+    const float* rp = o + id * (Dv + 1);
+    const float inv = 1.f / (fmaxf(fabsf(rp[Dv]), expf(-mx[id])) + 1e-6f);
+    float ss = 0.f;
+    for (int c = lane; c < Dv; c += WAVE) { const float x = rp[c] * inv; ss += x * x; }
+    const float nrm = inv / sqrtf(wave_sum(ss) / Dv + eps);
+    const T* gp = gate + row * gs + (long)h * Dv;
+    for (int c = lane; c < Dv; c += WAVE)
+        stf<T>(op + c, rp[c] * nrm * nw[h * Dv + c] * sigmoidf_(ldf<T>(gp + c)));
+}
+
+#define MD_THREADS 512
+// Single-token steps in one launch: gates, state update, read-out, norm and gate of a
+// (row, head). `lanes` (a power of two, at most a wave) neighbours share a state row;
+// with `vec` each of them holds four consecutive channels, else the channels lane,
+// lane + lanes, ... (at most four).
+template <typename T>
+__global__ void __launch_bounds__(MD_THREADS)
+mlstm_decode_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, long ks,
+                    const T* __restrict__ v, long vs, const T* __restrict__ zi, long zis,
+                    const T* __restrict__ zf, long zfs, const float* __restrict__ bi,
+                    const float* __restrict__ bf, float cap, float k_scale,
+                    const T* __restrict__ gate, long gs, const float* __restrict__ nw, float eps,
+                    float* __restrict__ state, float* __restrict__ mstate,
+                    const int* __restrict__ pos, const int* __restrict__ seq,
+                    T* __restrict__ out, int H, int D, int Dv, int lanes, int vec) {
+    extern __shared__ float osm[];                        // Dv + 1 read-outs
+    __shared__ float red[MD_THREADS / WAVE];
+    const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x;
+    const int slot = seq[b], p = pos[b];
+    T* op = out + ((long)b * H + h) * Dv;
+    if (slot < 0 || p < 0) {                              // uniform
+        for (int c = tid; c < Dv; c += MD_THREADS) stf<T>(op + c, 0.f);
+        return;
+    }
+    float i, f;
+    mlstm_gate_(ldf<T>(zi + b * zis + h) + bi[h], ldf<T>(zf + b * zfs + h) + bf[h], cap, i, f);
+    float m = p > 0 ? mstate[(long)slot * H + h] : 0.f;
+    const float kept = f + m;
+    m = fmaxf(kept, i);
+    const float a = p > 0 ? expf(kept - m) : 0.f, w = expf(i - m);
+    const int li = tid % lanes;
+    float kr[4], qr[4];
+    int dd[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+        dd[e] = vec ? li * 4 + e : li + e * lanes;
+        const bool ok = dd[e] < D;
+        kr[e] = ok ? ldf<T>(k + b * ks + (long)h * D + dd[e]) * k_scale * w : 0.f;
+        qr[e] = ok ? ldf<T>(q + b * qs + (long)h * D + dd[e]) : 0.f;
+    }
+    float* sp = state + ((long)slot * H + h) * (long)(Dv + 1) * D;
+    const int rpp = MD_THREADS / lanes;                   // rows per pass
+    constexpr int U = 4;                                  // passes in flight
+    for (int r0 = tid / lanes; r0 - tid / lanes <= Dv; r0 += rpp * U) {
+        float s[U][4], vv[U];
+#pragma unroll
+        for (int x = 0; x < U; ++x) {
+            const int r = r0 + x * rpp;
+            vv[x] = 0.f;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) s[x][e] = 0.f;
+            if (r > Dv) continue;
+            vv[x] = r == Dv ? 1.f : ldf<T>(v + b * vs + (long)h * Dv + r);
+            if (p <= 0) continue;                         // a sequence starts from zero
+            if (vec) {
+                if (li * 4 < D) {
+                    const float4 t = *reinterpret_cast<const float4*>(sp + (long)r * D + li * 4);
+                    s[x][0] = t.x; s[x][1] = t.y; s[x][2] = t.z; s[x][3] = t.w;
+                }
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) if (dd[e] < D) s[x][e] = sp[(long)r * D + dd[e]];
+            }
+        }
+#pragma unroll
+        for (int x = 0; x < U; ++x) {
+            const int r = r0 + x * rpp;
+            float acc = 0.f;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                s[x][e] = a * s[x][e] + kr[e] * vv[x];
+                acc += s[x][e] * qr[e];
+            }
+            for (int o = lanes / 2; o > 0; o >>= 1) acc += __shfl_xor(acc, o, WAVE);
+            if (r > Dv) continue;
+            if (li == 0) osm[r] = acc;
+            if (vec) {
+                if (li * 4 < D)
+                    *reinterpret_cast<float4*>(sp + (long)r * D + li * 4) =
+                        make_float4(s[x][0], s[x][1], s[x][2], s[x][3]);
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) if (dd[e] < D) sp[(long)r * D + dd[e]] = s[x][e];
+            }
+        }
+    }
+    __syncthreads();
+    if (tid == 0) mstate[(long)slot * H + h] = m;         // all have read it
+    const float inv = 1.f / (fmaxf(fabsf(osm[Dv]), expf(-m)) + 1e-6f);
+    float ss = 0.f;
+    for (int c = tid; c < Dv; c += MD_THREADS) { const float x = osm[c] * inv; ss += x * x; }
+    ss = wave_sum(ss);
+    if ((tid & (WAVE - 1)) == 0) red[tid / WAVE] = ss;
+    __syncthreads();
+    float tot = 0.f;
+#pragma unroll
+    for (int x = 0; x < MD_THREADS / WAVE; ++x) tot += red[x];
+    const float nrm = inv / sqrtf(tot / Dv + eps);
+    const T* gp = gate + b * gs + (long)h * Dv;
+    for (int c = tid; c < Dv; c += MD_THREADS)
+        stf<T>(op + c, osm[c] * nrm * nw[h * Dv + c] * sigmoidf_(ldf<T>(gp + c)));
+}
+
+// Long bf16 rows in chunks of GC_N tokens on the matrix cores. G_t is the running sum
+// of log a inside a chunk; all exponents are differences G_t - G_s (s <= t) and never
+// positive.
+//   mlstm_chunk_state_kernel  E = sum_s w_s exp(G_end - G_s) k_s v_s^T (and the n row),
+//                             the factor folded into the keys, three bf16 terms
+//   gla_chunk_link_kernel     start states S_c (two bf16 terms), the carried state
+//   mlstm_chunk_out_kernel    A_ts = (q_t k_s) w_s exp(G_t - G_s), o_t = exp(G_t) q_t S_c
+//                             + sum_s A_ts v_s; n_t q_t from S_c's last row and the sums
+//                             of A's rows; division, norm, weight, sigmoid gate
+// Decays are one number per token and head, so they multiply the scores and the
+// accumulators in fp32 and the products take q, k and v as they are.
+
+// exclusive use of one wave: running sum of log a over the chunk's tokens (lane = token;
+// tokens past the last add nothing)
+DEV float chunk_decay_sum_(const float* __restrict__ ld, long tok0, int H, int h, int cnt,
+                           int lane) {
+    float g = lane < cnt ? ld[(tok0 + lane) * H + h] : 0.f;
+#pragma unroll
+    for (int o = 1; o < WAVE; o <<= 1) {
+        const float x = __shfl_up(g, o, WAVE);
+        if (lane >= o) g += x;
+    }
+    return g;
+}
+
+template <int DP, int NT>
+__global__ void __launch_bounds__(256)
+mlstm_chunk_state_kernel(const bf16* __restrict__ k, long ks, const bf16* __restrict__ v, long vs,
+                         const float* __restrict__ ld, const float* __restrict__ wt,
+                         float k_scale, const int* __restrict__ seq,
+                         const int* __restrict__ nvalid, float* __restrict__ ws,
+                         float* __restrict__ wdec, int S, int H, int D, int Dv, int nc) {
+    __shared__ __attribute__((aligned(16))) uint16_t kt[3][DP * GC_VS];
+    __shared__ __attribute__((aligned(16))) uint16_t vt[NT * 16 * GC_VS];
+    __shared__ float cf[GC_N];                            // w_s exp(G_end - G_s) k_scale
+    __shared__ float tot[4][DP];
+    const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+    const int lr = lane & 15, lg = lane >> 4;
+    const int c = blockIdx.x % nc, d0 = blockIdx.x / nc * DP, h = blockIdx.y, b = blockIdx.z;
+    const int n = seq[b] < 0 ? 0 : nvalid[b];
+    const int cnt = min(GC_N, n - c * GC_N);
+    if (cnt <= 0) return;                                 // uniform
+    const long tok0 = (long)b * S + c * GC_N;
+    const int Dn = min(DP, D - d0);                       // this workgroup's key channels
+    const bf16* kp = k + (long)h * D + d0;
+    static_assert(4 * DP <= 256, "one (channel, 16 tokens) task per thread");
+    uint4 vr[NT / 2];
+    gc_load_rows_<NT * 2>(v + tok0 * vs + (long)h * Dv, vs, cnt, Dv, vr, tid);
+    const int d = tid % DP, sb = tid / DP;
+    float kv[16];
+    if (sb < 4) {
+        const int dc = min(d, Dn - 1);
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            const int m = sb * 16 + i;
+            const float kk = ldf<bf16>(kp + (tok0 + min(m, cnt - 1)) * ks + dc);
+            kv[i] = m < cnt && d < Dn ? kk : 0.f;
+        }
+    }
+    if (wv == 0) {
+        const float g = chunk_decay_sum_(ld, tok0, H, h, cnt, lane);
+        const float end = __shfl(g, WAVE - 1, WAVE);
+        cf[lane] = lane < cnt ? wt[(tok0 + lane) * H + h] * k_scale * expf(end - g) : 0.f;
+        if (lane == 0 && d0 == 0) wdec[((long)b * nc + c) * H + h] = expf(end);
+    }
+    gc_store_vt_<NT * 2>(vr, vt, tid);
+    __syncthreads();
+    if (sb < 4) {
+        float ns = 0.f;
+        bf16x8_t t0[2], t1[2], t2[2];                     // the three terms of 16 tokens
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            const float x = kv[i] * cf[sb * 16 + i];
+            ns += x;
+            const __bf16 a0 = (__bf16)x;
+            const float r1 = x - (float)a0;
+            const __bf16 a1 = (__bf16)r1;
+            t0[i >> 3][i & 7] = a0;
+            t1[i >> 3][i & 7] = a1;
+            t2[i >> 3][i & 7] = (__bf16)(r1 - (float)a1);
+        }
+        tot[sb][d] = ns;
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+            const int at = d * GC_VS + sb * 16 + u * 8;
+            *reinterpret_cast<bf16x8_t*>(kt[0] + at) = t0[u];
+            *reinterpret_cast<bf16x8_t*>(kt[1] + at) = t1[u];
+            *reinterpret_cast<bf16x8_t*>(kt[2] + at) = t2[u];
+        }
+    }
+    __syncthreads();
+    float* wp = ws + (((long)b * nc + c) * H + h) * (long)(Dv + 1) * D + d0;
+    if (tid < Dn) wp[(long)Dv * D + tid] = tot[0][tid] + tot[1][tid] + tot[2][tid] + tot[3][tid];
+    constexpr int DT = DP / 16;
+    for (int tile = wv; tile < DT * NT; tile += 4) {
+        const int dt = tile % DT, nt = tile / DT;
+        if (nt * 16 >= Dv || dt * 16 >= Dn) continue;
+        f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk) {
+            const bf16x8_t va = *reinterpret_cast<const bf16x8_t*>(
+                vt + (nt * 16 + lr) * GC_VS + kk * 32 + lg * 8);
+#pragma unroll
+            for (int e = 2; e >= 0; --e) {                // small terms first
+                const bf16x8_t kb = *reinterpret_cast<const bf16x8_t*>(
+                    kt[e] + (dt * 16 + lr) * GC_VS + kk * 32 + lg * 8);
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va, kb, acc, 0, 0, 0);
+            }
+        }
+        const int dd = dt * 16 + lr;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int nn = nt * 16 + lg * 4 + r;
+            if (nn < Dv && dd < Dn) wp[(long)nn * D + dd] = acc[r];
+        }
+    }
+}
+
+// two words of packed (high | low) bf16 terms each -> a vector of high and one of low terms
+DEV void unpack_terms_(const uint4 s0, const uint4 s1, bf16x8_t& hi, bf16x8_t& lo) {
+    const uint4 hv = make_uint4(
+        (s0.x >> 16) | (s0.y & 0xffff0000u), (s0.z >> 16) | (s0.w & 0xffff0000u),
+        (s1.x >> 16) | (s1.y & 0xffff0000u), (s1.z >> 16) | (s1.w & 0xffff0000u));
+    const uint4 lv = make_uint4(
+        (s0.x & 0xffffu) | (s0.y << 16), (s0.z & 0xffffu) | (s0.w << 16),
+        (s1.x & 0xffffu) | (s1.y << 16), (s1.z & 0xffffu) | (s1.w << 16));
+    hi = __builtin_bit_cast(bf16x8_t, hv);
+    lo = __builtin_bit_cast(bf16x8_t, lv);
+}
+
+// Workgroup = (chunk, head). Wave w makes the scores of tokens 16 w .. and leaves them
+// in LDS (two bf16 terms); then it owns value tiles w * NT/4 .. for all 64 tokens, so a
+// start state's rows are read by one wave only.
+template <int DP, int NT>
+__global__ void __launch_bounds__(256, 2)
+mlstm_chunk_out_kernel(const bf16* __restrict__ q, long qs, const bf16* __restrict__ k, long ks,
+                       const bf16* __restrict__ v, long vs, const float* __restrict__ ld,
+                       const float* __restrict__ wt, const float* __restrict__ mx, float k_scale,
+                       const bf16* __restrict__ gate, long gs, const float* __restrict__ nw,
+                       float eps, const int* __restrict__ seq, const int* __restrict__ nvalid,
+                       const float* __restrict__ ws, bf16* __restrict__ out, int S, int H, int D,
+                       int Dv, int nc) {
+    constexpr int KS = DP + 8, KK = DP / 32, NTW = NT / 4, OS = NT * 16 + 4;
+    constexpr int QK = 2 * GC_N * KS * 2 > GC_N * OS * 4 ? 2 * GC_N * KS * 2 : GC_N * OS * 4;
+    extern __shared__ __attribute__((aligned(16))) char smc[];
+    uint16_t* ql = reinterpret_cast<uint16_t*>(smc);      // GC_N * KS, then kl: the same
+    uint16_t* kl = ql + GC_N * KS;
+    float* ol = reinterpret_cast<float*>(smc);            // GC_N * OS, over q and k in the end
+    uint16_t* vt = reinterpret_cast<uint16_t*>(smc + QK); // NT * 16 * GC_VS
+    uint16_t* ah = vt + NT * 16 * GC_VS;                  // GC_N * GC_VS, rows = queries
+    uint16_t* al = ah + GC_N * GC_VS;
+    float* gl = reinterpret_cast<float*>(al + GC_N * GC_VS);   // G_t in base 2
+    float* wl = gl + GC_N;                                // w_s k_scale
+    float* iv = wl + GC_N;                                // 1 / normalizer
+    float (*part)[GC_N] = reinterpret_cast<float (*)[GC_N]>(iv + GC_N);   // 4 x GC_N
+    const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+    const int lr = lane & 15, lg = lane >> 4;
+    const int c = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+    const int n = seq[b] < 0 ? 0 : nvalid[b];
+    const int cnt = min(GC_N, n - c * GC_N);
+    if (cnt <= 0) return;                                 // uniform
+    const long tok0 = (long)b * S + c * GC_N;
+    uint4 qr[DP / 32], kr[DP / 32], vr[NT / 2];
+    gc_load_rows_<DP / 8>(q + tok0 * qs + (long)h * D, qs, cnt, D, qr, tid);
+    gc_load_rows_<DP / 8>(k + tok0 * ks + (long)h * D, ks, cnt, D, kr, tid);
+    gc_load_rows_<NT * 2>(v + tok0 * vs + (long)h * Dv, vs, cnt, Dv, vr, tid);
+    // the start state: this wave's value rows, and this lane's share of the n row
+    const float* sp = ws + (((long)b * nc + c) * H + h) * (long)(Dv + 1) * D;
+    uint4 sr[NTW][KK][2], nr[KK][2];
+#pragma unroll
+    for (int kk = 0; kk < KK; ++kk) {
+        const int d = kk * 32 + lg * 8;
+#pragma unroll
+        for (int i = 0; i < NTW; ++i) {
+            const int row = (w * NTW + i) * 16 + lr;
+            sr[i][kk][0] = sr[i][kk][1] = make_uint4(0, 0, 0, 0);
+            if (row < Dv && d < D) {
+                const float* rp = sp + (long)row * D + d;
+                sr[i][kk][0] = *reinterpret_cast<const uint4*>(rp);
+                sr[i][kk][1] = *reinterpret_cast<const uint4*>(rp + 4);
+            }
+        }
+        nr[kk][0] = nr[kk][1] = make_uint4(0, 0, 0, 0);
+        if (d < D) {
+            const float* rp = sp + (long)Dv * D + d;
+            nr[kk][0] = *reinterpret_cast<const uint4*>(rp);
+            nr[kk][1] = *reinterpret_cast<const uint4*>(rp + 4);
+        }
+    }
+    if (w == 0) {
+        gl[lane] = chunk_decay_sum_(ld, tok0, H, h, cnt, lane) * 1.4426950408889634f;
+        wl[lane] = lane < cnt ? wt[(tok0 + lane) * H + h] * k_scale : 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < DP / 32; ++i) {
+        const int x = tid + i * 256;
+        const int at = (x % GC_N) * KS + (x / GC_N) * 8;
+        *reinterpret_cast<uint4*>(ql + at) = qr[i];
+        *reinterpret_cast<uint4*>(kl + at) = kr[i];
+    }
+    gc_store_vt_<NT * 2>(vr, vt, tid);
+    __syncthreads();
+    // ---- scores of tokens 16 w + lr (a lane: keys j*16 + lg*4 .. +3)
+    {
+        const int t = w * 16 + lr;
+        const float gt = gl[t];
+        bf16x8_t qf[KK];
+        float nq = 0.f;
+#pragma unroll
+        for (int kk = 0; kk < KK; ++kk) {
+            qf[kk] = *reinterpret_cast<const bf16x8_t*>(ql + t * KS + kk * 32 + lg * 8);
+            bf16x8_t hi, lo;
+            unpack_terms_(nr[kk][0], nr[kk][1], hi, lo);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) nq += (float)qf[kk][e] * ((float)hi[e] + (float)lo[e]);
+        }
+        nq *= exp2_(gt);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            if (j > (w | 1)) continue;                    // blocks no product reads
+            f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
+            if (j <= w)
+#pragma unroll
+                for (int kk = 0; kk < KK; ++kk) {
+                    const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(
+                        kl + (j * 16 + lr) * KS + kk * 32 + lg * 8);
+                    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[kk], acc, 0, 0, 0);
+                }
+            union { __bf16 x[4]; uint2 u; } ph, pl;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int s = j * 16 + lg * 4 + r;
+                const float a = s <= t ? acc[r] * wl[s] * exp2_(gt - gl[s]) : 0.f;
+                nq += a;
+                split_bf16_(a, ph.x[r], pl.x[r]);
+            }
+            *reinterpret_cast<uint2*>(ah + t * GC_VS + j * 16 + lg * 4) = ph.u;
+            *reinterpret_cast<uint2*>(al + t * GC_VS + j * 16 + lg * 4) = pl.u;
+        }
+        nq += __shfl_xor(nq, 16, WAVE);
+        nq += __shfl_xor(nq, 32, WAVE);
+        if (lg == 0) {
+            const float m = mx[(tok0 + min(t, cnt - 1)) * H + h];
+            iv[t] = 1.f / (fmaxf(fabsf(nq), expf(-m)) + 1e-6f);
+        }
+    }
+    __syncthreads();
+    // ---- o = exp(G_t) q S + A v for this wave's value tiles, divided
+    f32x4_t o[4][NTW];
+#pragma unroll
+    for (int tb = 0; tb < 4; ++tb) {
+        bf16x8_t qf[KK];
+#pragma unroll
+        for (int kk = 0; kk < KK; ++kk)
+            qf[kk] = *reinterpret_cast<const bf16x8_t*>(ql + (tb * 16 + lr) * KS + kk * 32 + lg * 8);
+        const float4 g4 = *reinterpret_cast<const float4*>(gl + tb * 16 + lg * 4);
+        const float eg[4] = {exp2_(g4.x), exp2_(g4.y), exp2_(g4.z), exp2_(g4.w)};
+#pragma unroll
+        for (int i = 0; i < NTW; ++i) {
+            f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int kk = 0; kk < KK; ++kk) {
+                bf16x8_t hi, lo;
+                unpack_terms_(sr[i][kk][0], sr[i][kk][1], hi, lo);
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[kk], lo, acc, 0, 0, 0);
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[kk], hi, acc, 0, 0, 0);
+            }
+#pragma unroll
+            for (int r = 0; r < 4; ++r) acc[r] *= eg[r];
+#pragma unroll
+            for (int pr = 0; pr < 2; ++pr) {
+                if (pr * 2 > tb) continue;
+                const bf16x8_t vb = *reinterpret_cast<const bf16x8_t*>(
+                    vt + ((w * NTW + i) * 16 + lr) * GC_VS + pr * 32 + lg * 8);
+                const bf16x8_t pl = *reinterpret_cast<const bf16x8_t*>(
+                    al + (tb * 16 + lr) * GC_VS + pr * 32 + lg * 8);
+                const bf16x8_t ph = *reinterpret_cast<const bf16x8_t*>(
+                    ah + (tb * 16 + lr) * GC_VS + pr * 32 + lg * 8);
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pl, vb, acc, 0, 0, 0);
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ph, vb, acc, 0, 0, 0);
+            }
+            o[tb][i] = acc;
+        }
+    }
+#pragma unroll
+    for (int tb = 0; tb < 4; ++tb)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int t = tb * 16 + lg * 4 + r;
+            const float inv = iv[t];
+            float ss = 0.f;
+#pragma unroll
+            for (int i = 0; i < NTW; ++i) { o[tb][i][r] *= inv; ss += o[tb][i][r] * o[tb][i][r]; }
+            ss += __shfl_xor(ss, 1, WAVE);                // channels past Dv are zero
+            ss += __shfl_xor(ss, 2, WAVE);
+            ss += __shfl_xor(ss, 4, WAVE);
+            ss += __shfl_xor(ss, 8, WAVE);
+            if (lr == 0) part[w][t] = ss;
+        }
+    __syncthreads();                                      // q and k are no longer read
+#pragma unroll
+    for (int tb = 0; tb < 4; ++tb)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+#pragma unroll
+            for (int i = 0; i < NTW; ++i)
+                ol[(tb * 16 + lg * 4 + r) * OS + (w * NTW + i) * 16 + lr] = o[tb][i][r];
+    __syncthreads();
+    const int D8 = Dv / 8;
+    for (int x = tid; x < cnt * D8; x += 256) {
+        const int t = x / D8, ch = (x % D8) * 8;
+        const float inv = 1.f / sqrtf((part[0][t] + part[1][t] + part[2][t] + part[3][t]) / Dv + eps);
+        float ov[8], gv[8];
+        load8<float>(ol + t * OS + ch, ov);
+        load8<bf16>(gate + (tok0 + t) * gs + (long)h * Dv + ch, gv);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ov[e] *= inv * nw[h * Dv + ch + e] * sigmoidf_(gv[e]);
+        store8<bf16>(out + (tok0 + t) * (long)(H * Dv) + (long)h * Dv + ch, ov);
+    }
+}
+
 static inline int grid_for(long total, int block, int cap = 8192) {
     long g = (total + block - 1) / block;
     if (g < 1) g = 1;
@@ -3695,11 +4533,13 @@ int nx_decay_scan(const void* q, long qs, const void* k, long ks, const void* v,
                   const float* a_log, const float* head_decay, float k_scale, const float* skip,
                   float* state, const int* pos, const int* seq, const int* nvalid, float* out,
                   int B, int S, int H, int G, int D, int Dv, float* ws, float* wdec, int nseg,
-                  int seglen, int channel, hipStream_t st) {
+                  int seglen, int channel, const float* wgt, int ones, hipStream_t st) {
     if ((long)B * S <= 0) return 0;
     if (D <= 0 || Dv <= 0 || G <= 0 || H % G != 0 || D > 256) return -1;
     if ((dt == nullptr) == (head_decay == nullptr)) return -2;
-    if (dt && !channel && (!dt_bias || !a_log)) return -2;
+    if (dt && !channel && !wgt && (!dt_bias || !a_log)) return -2;
+    if (wgt && (!dt || dt_bf16 || channel)) return -2;
+    if (ones < 0 || ones > 1 || (ones && (Dv < 2 || skip))) return -2;
     if (channel && (!dt || dt_bf16 || a_log || skip)) return -2;
     if (H > 65535 || B > 65535) return -3;
     // the kernel reads state rows 16 bytes at a time when dim % 4 == 0
@@ -3711,7 +4551,7 @@ int nx_decay_scan(const void* q, long qs, const void* k, long ks, const void* v,
 #define DSK(T, TD, RV, MD, CHV) decay_scan_kernel<T, TD, RV, MD, CHV><<<grid, block, 0, st>>>( \
         (const T*)q, qs, (const T*)k, ks, (const T*)v, vs, (const TD*)dt, dts, dt_bias, a_log, \
         head_decay, k_scale, skip, state, pos, seq, nvalid, out, S, H, G, D, Dv, ws, wdec, nseg, \
-        seglen)
+        seglen, wgt, ones)
 #define DSR(T, TD, MD, CHV) do { if (D <= 16) DSK(T, TD, 1, MD, CHV); \
         else if (D <= 32) DSK(T, TD, 2, MD, CHV); \
         else if (D <= 64) DSK(T, TD, 4, MD, CHV); else if (D <= 128) DSK(T, TD, 8, MD, CHV); \
@@ -3811,8 +4651,8 @@ int nx_group_gated_norm(const float* y, const void* gate, long gs, int gate_bf16
 }
 
 int nx_group_router(const float* logits, long ls, int E, int extra, int top, int ngroups,
-                    int keep, float scale, int normalize, const float* corr, float* dense,
-                    int* idx, float* wts, long T, hipStream_t st) {
+                    int keep, float scale, int normalize, const float* corr, int sig, int gtwo,
+                    float norm_eps, float* dense, int* idx, float* wts, long T, hipStream_t st) {
     if (T <= 0) return 0;
     if (E <= 0 || top <= 0 || top > E || top > WAVE || ngroups <= 0 || E % ngroups != 0 ||
         keep <= 0 || keep > ngroups || (long)top > (long)(E / ngroups) * keep) return -1;
@@ -3820,14 +4660,15 @@ int nx_group_router(const float* logits, long ls, int E, int extra, int top, int
     if (sh > 60 * 1024) return -2;
     dim3 grid((unsigned)((T + RT_WAVES - 1) / RT_WAVES)), block(RT_WAVES * WAVE);
     group_router_kernel<<<grid, block, sh, st>>>(logits, ls, E, extra, top, ngroups, keep, scale,
-                                                 normalize, corr, dense, idx, wts, T);
+                                                 normalize, corr, sig, gtwo, norm_eps, dense, idx,
+                                                 wts, T);
     return (int)hipGetLastError();
 }
 
 int nx_router_fused(const void* x, long xs, int x_bf16, const float* w, int W, int E, int extra,
                     int top, int ngroups, int keep, float scale, int normalize, const float* corr,
-                    const float* bias, float* dense, int* idx, float* wts, long T,
-                    hipStream_t st) {
+                    const float* bias, int sig, int gtwo, float norm_eps, float* dense, int* idx,
+                    float* wts, long T, hipStream_t st) {
     if (T <= 0) return 0;
     if (E <= 0 || top <= 0 || top > E || top > WAVE || ngroups <= 0 || E % ngroups != 0 ||
         keep <= 0 || keep > ngroups || (long)top > (long)(E / ngroups) * keep || W <= 0) return -1;
@@ -3839,10 +4680,10 @@ int nx_router_fused(const void* x, long xs, int x_bf16, const float* w, int W, i
     dim3 grid((unsigned)T), block(RT_WAVES * WAVE);
     if (x_bf16) router_fused_kernel<bf16><<<grid, block, sh, st>>>(
         (const bf16*)x, xs, w, W, vec, E, extra, top, ngroups, keep, scale, normalize, corr, bias,
-        dense, idx, wts);
+        sig, gtwo, norm_eps, dense, idx, wts);
     else router_fused_kernel<float><<<grid, block, sh, st>>>(
         (const float*)x, xs, w, W, vec, E, extra, top, ngroups, keep, scale, normalize, corr, bias,
-        dense, idx, wts);
+        sig, gtwo, norm_eps, dense, idx, wts);
     return (int)hipGetLastError();
 }
 
@@ -3878,27 +4719,22 @@ int nx_act_scale(const void* x, int is_bf16, const float* gates, int gcols, int 
     return (int)hipGetLastError();
 }
 
-int nx_clamped_glu_scale(const void* x, int is_bf16, const float* gates, long gs, int ff, int E,
-                         float limit, float slimit, float alpha, void* out, long rows, int C,
-                         hipStream_t st) {
+int nx_glu_scale(const void* x, int is_bf16, const float* gates, long gs, int ff, int E, int act,
+                 float limit, float slimit, float alpha, void* out, long rows, int C,
+                 hipStream_t st) {
     if (rows * C <= 0) return 0;
-    if (E < 0 || (E > 0 && (ff <= 0 || !gates)) || (long)E * ff > C) return -1;
+    if (E < 0 || (E > 0 && (ff <= 0 || !gates)) || (long)E * ff > C || act < 0 || act > 1) return -1;
     if (E == 0) ff = 8;
     const bool vec = (C % 8) == 0 && (ff % 8) == 0 && ((uintptr_t)x % 16) == 0 &&
                      ((uintptr_t)out % 16) == 0;
-    if (vec) {
-        dim3 grid(grid_for(rows * (C / 8), 256)), block(256);
-        if (is_bf16) clamped_glu_scale_vec_kernel<bf16><<<grid, block, 0, st>>>(
-            (const bf16*)x, gates, gs, ff, E, limit, slimit, alpha, (bf16*)out, rows, C);
-        else clamped_glu_scale_vec_kernel<float><<<grid, block, 0, st>>>(
-            (const float*)x, gates, gs, ff, E, limit, slimit, alpha, (float*)out, rows, C);
-    } else {
-        dim3 grid(grid_for(rows * C, 256)), block(256);
-        if (is_bf16) clamped_glu_scale_kernel<bf16><<<grid, block, 0, st>>>(
-            (const bf16*)x, gates, gs, ff, E, limit, slimit, alpha, (bf16*)out, rows, C);
-        else clamped_glu_scale_kernel<float><<<grid, block, 0, st>>>(
-            (const float*)x, gates, gs, ff, E, limit, slimit, alpha, (float*)out, rows, C);
-    }
+    dim3 grid(grid_for(vec ? rows * (C / 8) : rows * C, 256)), block(256);
+#define GS(T, A) do { if (vec) glu_scale_vec_kernel<T, A><<<grid, block, 0, st>>>( \
+        (const T*)x, gates, gs, ff, E, limit, slimit, alpha, (T*)out, rows, C); \
+    else glu_scale_kernel<T, A><<<grid, block, 0, st>>>( \
+        (const T*)x, gates, gs, ff, E, limit, slimit, alpha, (T*)out, rows, C); } while (0)
+    if (is_bf16) { if (act) GS(bf16, 1); else GS(bf16, 0); }
+    else { if (act) GS(float, 1); else GS(float, 0); }
+#undef GS
     return (int)hipGetLastError();
 }
 
@@ -4004,6 +4840,155 @@ int nx_head_product(const void* a, const void* w, void* out, int T, int H, int K
     dim3 grid((N + 15) / 16, H, (T + 63) / 64), block(256);
     head_product_kernel<<<grid, block, 0, st>>>((const bf16*)a, (const bf16*)w, (bf16*)out, T, H,
                                                 K, N);
+    return (int)hipGetLastError();
+}
+
+int nx_hyper_step(const float* xin, long xrow, long xstr, const void* y, int is_bf16,
+                  const float* mix, const float* wout, float* xout, const float* win,
+                  const float* nw, float eps, void* hout, float* uout, float* scratch, long rows,
+                  int NS, int C, hipStream_t st) {
+    if (rows <= 0) return 0;
+    if (C <= 0 || NS <= 0 || !xin || (y && (!mix || !wout)) || (nw ? !hout : !uout)) return -1;
+    dim3 grid((unsigned)rows), block(LN_THREADS);
+    const bool vec = (C % 4) == 0 && (xrow % 4) == 0 && (xstr % 4) == 0 && NS <= 4 &&
+                     C <= LN_THREADS * 32 &&
+                     (((uintptr_t)xin | (uintptr_t)xout | (uintptr_t)y | (uintptr_t)nw |
+                       (uintptr_t)hout | (uintptr_t)uout) % 16) == 0;
+    if (!vec && ((y && xout == xin) || (nw && !scratch))) return -2;
+#define HSV(T, N, V) hyper_step_vec_kernel<T, N, V><<<grid, block, 0, st>>>( \
+        xin, xrow, xstr, (const T*)y, mix, wout, xout, win, nw, eps, (T*)hout, uout, C)
+#define HSN(T, N) do { if (C <= LN_THREADS * 4) HSV(T, N, 1); else if (C <= LN_THREADS * 8) HSV(T, N, 2); \
+        else if (C <= LN_THREADS * 16) HSV(T, N, 4); else HSV(T, N, 8); } while (0)
+#define HS(T) do { if (!vec) hyper_step_kernel<T><<<grid, block, 0, st>>>( \
+            xin, xrow, xstr, (const T*)y, mix, wout, xout, win, nw, eps, (T*)hout, uout, scratch, \
+            NS, C); \
+        else if (NS == 1) HSN(T, 1); else if (NS == 2) HSN(T, 2); else if (NS == 3) HSN(T, 3); \
+        else HSN(T, 4); } while (0)
+    if (is_bf16) HS(bf16); else HS(float);
+#undef HS
+#undef HSN
+#undef HSV
+    return (int)hipGetLastError();
+}
+
+int nx_qkv_rows(const void* q, long qs, const void* k, long ks, const void* v, long vs,
+                const void* vf, long vfs, const float* lam, int is_bf16, const int* pos,
+                const int* slots, const float* inv_freq, int half, int unorm, float eps, void* qo,
+                void* kc, void* vc, long nslots, long ntok, int H, int G, int D, int Dv,
+                hipStream_t st) {
+    if (ntok <= 0) return 0;
+    if (H <= 0 || G <= 0 || D <= 0 || Dv <= 0 || half < 0 || 2 * half > D || half > HN_MAXC / 2 ||
+        (half > 0 && !inv_freq) || (vf && !lam)) return -1;
+    const int vecn = is_bf16 ? 8 : 4;
+    const bool vec = (D % 8) == 0 && D <= 8 * WAVE && (half % 8) == 0 && ((G * Dv) % 8) == 0 &&
+                     (qs % vecn) == 0 && (ks % vecn) == 0 && (vs % vecn) == 0 && (vfs % vecn) == 0 &&
+                     (((uintptr_t)q | (uintptr_t)k | (uintptr_t)v | (uintptr_t)vf | (uintptr_t)qo |
+                       (uintptr_t)kc | (uintptr_t)vc) % 16) == 0;
+    int lanes = 1;
+    while (lanes * 8 < D) lanes *= 2;
+    dim3 grid((unsigned)ntok), block(256);
+#define QK(T) do { if (vec) qkv_rows_vec_kernel<T><<<grid, block, 0, st>>>( \
+            (const T*)q, qs, (const T*)k, ks, (const T*)v, vs, (const T*)vf, vfs, lam, pos, slots, \
+            inv_freq, half, unorm, eps, (T*)qo, (T*)kc, (T*)vc, nslots, H, G, D, Dv, lanes); \
+        else qkv_rows_kernel<T><<<grid, block, 0, st>>>( \
+            (const T*)q, qs, (const T*)k, ks, (const T*)v, vs, (const T*)vf, vfs, lam, pos, slots, \
+            inv_freq, half, unorm, eps, (T*)qo, (T*)kc, (T*)vc, nslots, H, G, D, Dv); } while (0)
+    if (is_bf16) QK(bf16); else QK(float);
+#undef QK
+    return (int)hipGetLastError();
+}
+
+int nx_mlstm_gates(const void* zi, long zis, const void* zf, long zfs, int is_bf16,
+                   const float* bi, const float* bf, float cap, float* mstate, const int* pos,
+                   const int* seq, const int* nvalid, float* ld, float* wt, float* mx, int B,
+                   int S, int H, hipStream_t st) {
+    if ((long)B * S <= 0) return 0;
+    if (H <= 0 || B > 65535 || !bi || !bf || !(cap > 0.f)) return -1;
+    dim3 grid(H, B), block(MG_THREADS);
+#define MG(T) mlstm_gates_kernel<T><<<grid, block, 0, st>>>( \
+        (const T*)zi, zis, (const T*)zf, zfs, bi, bf, cap, mstate, pos, seq, nvalid, ld, wt, mx, S, H)
+    if (is_bf16) MG(bf16); else MG(float);
+#undef MG
+    return (int)hipGetLastError();
+}
+
+int nx_mlstm_readout(const float* o, const float* mx, const void* gate, long gs, int is_bf16,
+                     const float* nw, float eps, const int* pos, void* out, long rows, int H,
+                     int Dv, hipStream_t st) {
+    if (rows <= 0) return 0;
+    if (H <= 0 || Dv <= 0 || !nw) return -1;
+    dim3 grid((unsigned)((rows * H + 3) / 4)), block(4 * WAVE);
+    if (is_bf16) mlstm_readout_kernel<bf16><<<grid, block, 0, st>>>(
+        o, mx, (const bf16*)gate, gs, nw, eps, pos, (bf16*)out, rows, H, Dv);
+    else mlstm_readout_kernel<float><<<grid, block, 0, st>>>(
+        o, mx, (const float*)gate, gs, nw, eps, pos, (float*)out, rows, H, Dv);
+    return (int)hipGetLastError();
+}
+
+// single-token steps; key channels up to 256
+int nx_mlstm_decode(const void* q, long qs, const void* k, long ks, const void* v, long vs,
+                    const void* zi, long zis, const void* zf, long zfs, int is_bf16,
+                    const float* bi, const float* bf, float cap, float k_scale, const void* gate,
+                    long gs, const float* nw, float eps, float* state, float* mstate,
+                    const int* pos, const int* seq, void* out, int B, int H, int D, int Dv,
+                    hipStream_t st) {
+    if (B <= 0) return 0;
+    if (H <= 0 || D <= 0 || D > 4 * WAVE || Dv <= 0 || Dv > 8192 || B > 65535 || !bi || !bf ||
+        !nw || !(cap > 0.f)) return -1;
+    const int vec = (D % 4) == 0 && ((uintptr_t)state % 16) == 0;
+    int lanes = 1;
+    while (lanes * 4 < D) lanes *= 2;
+    dim3 grid(H, B), block(MD_THREADS);
+    const size_t sh = (size_t)(Dv + 1) * sizeof(float);
+#define MDK(T) mlstm_decode_kernel<T><<<grid, block, sh, st>>>( \
+        (const T*)q, qs, (const T*)k, ks, (const T*)v, vs, (const T*)zi, zis, (const T*)zf, zfs, \
+        bi, bf, cap, k_scale, (const T*)gate, gs, nw, eps, state, mstate, pos, seq, (T*)out, H, D, \
+        Dv, lanes, vec)
+    if (is_bf16) MDK(bf16); else MDK(float);
+#undef MDK
+    return (int)hipGetLastError();
+}
+
+// chunked form: bf16 q/k/v/gate/out, D and Dv multiples of 8 up to 128; ws holds
+// (B, chunks, H, Dv + 1, D), wdec (B, chunks, H)
+int nx_mlstm_chunked(const void* q, long qs, const void* k, long ks, const void* v, long vs,
+                     const float* ld, const float* wt, const float* mx, float k_scale,
+                     const void* gate, long gs, const float* nw, float eps, float* state,
+                     const int* pos, const int* seq, const int* nvalid, float* ws, float* wdec,
+                     void* out, int B, int S, int H, int D, int Dv, hipStream_t st) {
+    if ((long)B * S <= 0) return 0;
+    if (D <= 0 || Dv <= 0 || D > 128 || Dv > 128 || (D % 8) || (Dv % 8)) return -1;
+    if ((qs % 8) || (ks % 8) || (vs % 8) || (gs % 8) ||
+        (((uintptr_t)q | (uintptr_t)k | (uintptr_t)v | (uintptr_t)gate | (uintptr_t)ws |
+          (uintptr_t)out) % 16) || !gate || !nw) return -2;
+    const int nc = (S + GC_N - 1) / GC_N;
+    if (H > 65535 || B > 65535) return -3;
+    dim3 grid(nc, H, B), block(256);
+    const long per_head = (long)(Dv + 1) * D;
+#define MC(DPV, NT) do { \
+        constexpr int DPB = DPV < 64 ? DPV : 64; \
+        constexpr size_t qk = 2 * GC_N * (DPV + 8) * 2 > GC_N * (NT * 16 + 4) * 4 \
+            ? 2 * GC_N * (DPV + 8) * 2 : GC_N * (NT * 16 + 4) * 4; \
+        const size_t lsh = qk + (size_t)(NT * 16 + 2 * GC_N) * GC_VS * 2 + 7 * GC_N * 4; \
+        static bool attr_set = false; \
+        if (!attr_set) { \
+            if (hipFuncSetAttribute((const void*)mlstm_chunk_out_kernel<DPV, NT>, \
+                    hipFuncAttributeMaxDynamicSharedMemorySize, (int)lsh) != hipSuccess) return -5; \
+            attr_set = true; \
+        } \
+        dim3 gst(nc * ((D + DPB - 1) / DPB), H, B); \
+        mlstm_chunk_state_kernel<DPB, NT><<<gst, block, 0, st>>>( \
+            (const bf16*)k, ks, (const bf16*)v, vs, ld, wt, k_scale, seq, nvalid, ws, wdec, S, H, \
+            D, Dv, nc); \
+        gla_chunk_link_kernel<<<grid_for((long)B * H * per_head, 256), 256, 0, st>>>( \
+            ws, wdec, state, pos, seq, nvalid, B, S, H, 1, per_head, nc); \
+        mlstm_chunk_out_kernel<DPV, NT><<<grid, block, lsh, st>>>( \
+            (const bf16*)q, qs, (const bf16*)k, ks, (const bf16*)v, vs, ld, wt, mx, k_scale, \
+            (const bf16*)gate, gs, nw, eps, seq, nvalid, ws, (bf16*)out, S, H, D, Dv, nc); } while (0)
+#define MCN(DPV) do { if (Dv <= 64) MC(DPV, 4); else MC(DPV, 8); } while (0)
+    if (D <= 32) MCN(32); else if (D <= 64) MCN(64); else MCN(128);
+#undef MCN
+#undef MC
     return (int)hipGetLastError();
 }
 

@@ -498,7 +498,7 @@ def low_rank_decay(low, weight, bias, tau: float):
 
 def decay_scan(q, k, v, state, positions, seq_ids, dim: int, vdim: int,
                dt=None, dt_bias=None, a_log=None, head_decay=None,
-               k_scale: float = 1.0, skip=None, log_decay=None):
+               k_scale: float = 1.0, skip=None, log_decay=None, weight=None, ones: bool = False):
     """Linear recurrence with a decay per head and matrix state, carried in ``state`` (slots, H, vdim, dim) fp32 (stored transposed):
 
         S_t = a_t S_{t-1} + k_t (w_t v_t)^T ;  o_t = S_t^T q_t (+ skip_h v_t)
@@ -508,7 +508,10 @@ def decay_scan(q, k, v, state, positions, seq_ids, dim: int, vdim: int,
     exp(-exp(a_log) w_t) (selective state spaces: k = B, q = C, v = x); or
     ``head_decay`` (H,): a_t = head_decay, w_t = 1 (retention); or
     ``log_decay`` (B,S,H*dim): a decay per head and KEY CHANNEL, S_t =
-    diag(exp(log_decay_t)) S_{t-1} + k_t v_t^T (gated linear attention). q, k
+    diag(exp(log_decay_t)) S_{t-1} + k_t v_t^T (gated linear attention); or
+    ``log_decay`` and ``weight`` (B,S,H) each: a_t = exp(log_decay_t), w_t =
+    weight_t. ``ones`` appends a value channel that is always one (state and
+    output have one more row per head). q, k
     (B,S,G*dim) are shared by H/G consecutive heads, v (B,S,H*vdim); k is
     multiplied by ``k_scale``. Returns fp32 (B,S,H*vdim)."""
     B, S = positions.shape
@@ -519,7 +522,12 @@ def decay_scan(q, k, v, state, positions, seq_ids, dim: int, vdim: int,
     qf = q.float().reshape(B, S, G, D).repeat_interleave(rep, dim=2)
     kf = (k.float() * k_scale).reshape(B, S, G, D).repeat_interleave(rep, dim=2)
     vf = v.float().reshape(B, S, H, Dv)
-    if dt is not None:
+    if ones:
+        vf = torch.cat([vf, torch.ones_like(vf[..., :1])], dim=-1)
+        Dv = Dv + 1
+    if weight is not None:
+        a, w = torch.exp(log_decay.float()), weight.float()
+    elif dt is not None:
         w = torch.nn.functional.softplus(dt.float() + dt_bias.float(), threshold=20.0)
         a = torch.exp(-torch.exp(a_log.float()) * w)
     elif log_decay is not None:
@@ -547,6 +555,69 @@ def decay_scan(q, k, v, state, positions, seq_ids, dim: int, vdim: int,
     return out.reshape(B, S, H * Dv)
 
 
+def mlstm_gates(i_gate, f_gate, i_bias, f_bias, gate_cap: float):
+    """Log input and log forget gates (fp32) from their projections."""
+    i = gate_cap * torch.tanh((i_gate.float() + i_bias.float()) / gate_cap)
+    f = torch.nn.functional.logsigmoid(
+        gate_cap * torch.tanh((f_gate.float() + f_bias.float()) / gate_cap))
+    return i, f
+
+
+def mlstm(q, k, v, i_gate, f_gate, gate, i_bias, f_bias, gate_cap: float, norm_weight, eps: float,
+          state, max_state, positions, seq_ids, dim: int, vdim: int):
+    """Matrix memory with exponential gates: per head, with log gates i, f of
+    :func:`mlstm_gates` and a running maximum m from 0,
+
+        m_t = max(f_t + m_{t-1}, i_t) ; a_t = exp(f_t + m_{t-1} - m_t)
+        S_t = a_t S_{t-1} + exp(i_t - m_t) k_t v_t^T ; n_t likewise with k alone
+        o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6)
+
+    (q scaled by dim^-1/2; it rides on k here), then an RMS norm per head, the
+    weight (H*vdim) and sigmoid(gate). ``state`` (slots, H, vdim + 1, dim)
+    holds S transposed and n as its last row, ``max_state`` (slots, H) m."""
+    B, S = positions.shape
+    H = v.shape[-1] // vdim
+    i, f = mlstm_gates(i_gate, f_gate, i_bias, f_bias, gate_cap)
+    log_a, w = torch.zeros_like(f), torch.zeros_like(f)
+    mx = torch.zeros_like(f)
+    n_valid, p0s = _row_extent(positions)
+    for b in range(B):
+        slot, n = int(seq_ids[b]), int(n_valid[b])
+        if slot < 0 or n == 0:
+            continue
+        m = max_state[slot].clone() if int(p0s[b]) > 0 else torch.zeros(H, device=v.device)
+        for t in range(n):
+            kept = f[b, t] + m
+            m = torch.maximum(kept, i[b, t])
+            log_a[b, t], w[b, t], mx[b, t] = kept - m, torch.exp(i[b, t] - m), m
+        max_state[slot] = m
+    o = decay_scan(q, k, v, state, positions, seq_ids, dim, vdim, k_scale=dim ** -0.5,
+                   log_decay=log_a, weight=w, ones=True).view(B, S, H, vdim + 1)
+    den = torch.maximum(o[..., vdim].abs(), torch.exp(-mx)) + 1e-6
+    o = o[..., :vdim] / den.unsqueeze(-1)
+    o = o * torch.rsqrt((o * o).mean(-1, keepdim=True) + eps)
+    o = o.reshape(B, S, H * vdim) * norm_weight.float() * torch.sigmoid(gate.float())
+    return o.to(gate.dtype)
+
+
+def hyper_step(streams, y, mix, w_out, w_in):
+    """Parallel residual streams: (new streams (B,S,n,C), sum_t w_in[t] x_t)
+    with x_t = sum_s mix[s, t] streams_s + w_out[t] y; ``streams`` (B,S,C)
+    stands for n equal ones, ``y`` None changes nothing, ``w_in`` None sums."""
+    n = mix.shape[0]
+    if streams.dim() == 3:
+        if y is None:
+            tot = float(n) if w_in is None else w_in.float().sum()
+            return streams, streams * tot
+        streams = streams.unsqueeze(2).expand(-1, -1, n, -1)
+    if y is not None:
+        streams = torch.einsum("bqsc,st->bqtc", streams, mix.float()) \
+            + w_out.float().view(1, 1, n, 1) * y.float().unsqueeze(2)
+    if w_in is None:
+        return streams, streams.sum(2)
+    return streams, (streams * w_in.float().view(1, 1, n, 1)).sum(2)
+
+
 def group_gated_norm(y, gate, weight, eps: float, groups: int, gate_first: bool,
                      out_dtype=torch.float32):
     """RMS norm of (.., C) rows in ``groups`` equal parts (each part by its
@@ -569,12 +640,13 @@ def group_gated_norm(y, gate, weight, eps: float, groups: int, gate_first: bool,
 
 def group_limited_router(logits, num_experts: int, top_k: int, n_groups: int,
                          keep_groups: int, scale: float, normalize: bool = False,
-                         correction=None):
-    """Softmax over the first ``num_experts`` columns of fp32 ``logits``
+                         correction=None, score: str = "softmax", group_top: int = 1,
+                         norm_eps: float = 0.0):
+    """Softmax (or, ``score`` = sigmoid, the sigmoids) of the first ``num_experts`` columns of fp32 ``logits``
     (T, E + extra); experts form ``n_groups`` groups of neighbours, a group
-    scores as its best expert and only experts of the ``keep_groups`` best
-    groups compete for the ``top_k`` places. Weights are the chosen experts'
-    softmax scores times ``scale`` (divided by their sum first when
+    scores as the sum of its ``group_top`` best experts and only experts of
+    the ``keep_groups`` best groups compete for the ``top_k`` places. Weights are the chosen experts'
+    scores times ``scale`` (divided by their sum + ``norm_eps`` first when
     ``normalize``). ``correction`` (E,) is added to the scores for the choice
     only (the weights stay the scores). Extra columns are per-token sigmoid
     gates. Returns
@@ -583,11 +655,11 @@ def group_limited_router(logits, num_experts: int, top_k: int, n_groups: int,
     T = logits.shape[0]
     E = num_experts
     lf = logits.float()
-    s = torch.softmax(lf[:, :E], dim=-1)
+    s = torch.sigmoid(lf[:, :E]) if score == "sigmoid" else torch.softmax(lf[:, :E], dim=-1)
     cand = s if correction is None else s + correction.float()
     if n_groups > 1 and keep_groups < n_groups:
         per = E // n_groups
-        gs = s.view(T, n_groups, per).max(-1).values
+        gs = cand.view(T, n_groups, per).topk(min(group_top, per), dim=-1).values.sum(-1)
         best = gs.topk(keep_groups, dim=-1).indices
         gmask = torch.zeros_like(gs, dtype=torch.bool).scatter(1, best, True)
         cand = torch.where(gmask.repeat_interleave(per, dim=1), cand,
@@ -595,7 +667,7 @@ def group_limited_router(logits, num_experts: int, top_k: int, n_groups: int,
     idx = cand.topk(top_k, dim=-1).indices
     w = s.gather(1, idx)
     if normalize:
-        w = w / w.sum(-1, keepdim=True)
+        w = w / (w.sum(-1, keepdim=True) + norm_eps)
     w = w * scale
     dense = torch.zeros_like(lf)
     dense[:, :E] = torch.zeros_like(s).scatter(1, idx, w)
@@ -622,6 +694,18 @@ def clamped_glu_scale(hid, gates, expert_ff: int, num_experts: int, limit: float
         out[:, :ne] = clamped_glu(g[:, :ne], u[:, :ne], limit, alpha) * gates.float()[:, cols]
     if C > ne:
         out[:, ne:] = clamped_glu(g[:, ne:], u[:, ne:], shared_limit, alpha)
+    return out.to(out_dtype)
+
+
+def silu_glu_scale(hid, gates, expert_ff: int, num_experts: int, out_dtype):
+    """silu(gate) * up of stacked experts in the layout of
+    :func:`clamped_glu_scale`, times the token's routing weights."""
+    C = hid.shape[1] // 2
+    ne = num_experts * expert_ff
+    out = torch.nn.functional.silu(hid.float()[:, :C]) * hid.float()[:, C:]
+    if ne:
+        cols = torch.arange(ne, device=hid.device) // expert_ff
+        out[:, :ne] *= gates.float()[:, cols]
     return out.to(out_dtype)
 
 

@@ -636,24 +636,36 @@ def low_rank_decay(low, weight, bias, tau: float):
 
 def decay_scan(q, k, v, state, step: StepLayout, dim: int, vdim: int, dt=None,
                dt_bias=None, a_log=None, head_decay=None, k_scale: float = 1.0, skip=None,
-               log_decay=None):
+               log_decay=None, weight=None, ones: bool = False):
     """Decayed linear recurrence with matrix state (see ref.decay_scan):
     selective state spaces (``dt``/``dt_bias``/``a_log``), fixed per-head
-    decays (``head_decay``) or a decay per key channel (its logarithm
-    ``log_decay`` (B,S,H*dim) fp32). q, k (B,S,G*dim), v (B,S,H*vdim) may be column
+    decays (``head_decay``), a decay per key channel (its logarithm
+    ``log_decay`` (B,S,H*dim) fp32) or, with ``weight`` (B,S,H) fp32, given
+    log decays (B,S,H) and write weights per head and token. q, k (B,S,G*dim),
+    v (B,S,H*vdim) may be column
     slices of wider tensors; ``state`` (slots, H, vdim, dim) fp32 is read
-    (unless the row starts at position 0) and advanced. Returns fp32."""
+    (unless the row starts at position 0) and advanced. With ``ones`` the
+    state has one more row per head, of a value channel that is always one,
+    and so has the output. Returns fp32."""
     assert sum(x is not None for x in (dt, head_decay, log_decay)) == 1
+    assert weight is None or log_decay is not None
+    ones = int(bool(ones))
     if v.is_cuda:
         lib = _load()
         B, S = v.shape[0], v.shape[1]
         H = v.shape[-1] // vdim
         G = q.shape[-1] // dim
         assert q.dtype == k.dtype == v.dtype and state.dtype == torch.float32
-        assert state.is_contiguous() and tuple(state.shape[1:]) == (H, vdim, dim)
+        rows = vdim + ones
+        assert state.is_contiguous() and tuple(state.shape[1:]) == (H, rows, dim)
         assert H % G == 0 and q.shape[-1] == G * dim and k.shape[-1] == G * dim
-        out = torch.empty(B, S, H * vdim, dtype=torch.float32, device=v.device)
-        channel, dch = log_decay is not None, 1
+        out = torch.empty(B, S, H * rows, dtype=torch.float32, device=v.device)
+        channel, dch = log_decay is not None and weight is None, 1
+        if weight is not None:
+            assert log_decay.dtype == weight.dtype == torch.float32
+            assert tuple(log_decay.shape) == tuple(weight.shape) == (B, S, H)
+            assert log_decay.is_contiguous() and weight.is_contiguous()
+            dt = log_decay
         if channel:
             assert G == H and skip is None and log_decay.shape[-1] == H * dim
             assert log_decay.dtype == torch.float32
@@ -661,7 +673,7 @@ def decay_scan(q, k, v, state, step: StepLayout, dim: int, vdim: int, dt=None,
         # a long row with few (row, head, channel block) workgroups is cut into
         # segments that scan side by side (two passes joined by a short serial
         # link over the segments' end states)
-        groups = B * H * ((vdim + 15) // 16)
+        groups = B * H * ((rows + 15) // 16)
         nseg, seglen, ws, wdec = 1, S, None, None
         if S >= 256 and groups < 1024:
             nseg = 1
@@ -669,7 +681,7 @@ def decay_scan(q, k, v, state, step: StepLayout, dim: int, vdim: int, dt=None,
                 nseg *= 2
             if nseg > 1:
                 seglen = ((S + nseg - 1) // nseg + 15) // 16 * 16
-                ws = torch.empty(B * nseg * H * vdim * dim, dtype=torch.float32, device=v.device)
+                ws = torch.empty(B * nseg * H * rows * dim, dtype=torch.float32, device=v.device)
                 wdec = torch.empty(B * nseg * H * dch, dtype=torch.float32, device=v.device)
         _check(lib.nx_decay_scan(
             _p(q), ctypes.c_long(_rows_view(q)), _p(k), ctypes.c_long(_rows_view(k)),
@@ -681,12 +693,13 @@ def decay_scan(q, k, v, state, step: StepLayout, dim: int, vdim: int, dt=None,
             _p(None if head_decay is None else _f32(head_decay)),
             ctypes.c_float(k_scale), _p(None if skip is None else _f32(skip)),
             _p(state), _p(step.positions), _p(step.seq_ids), _p(step.nvalid), _p(out),
-            B, S, H, G, dim, vdim, _p(ws), _p(wdec), nseg, seglen, int(channel),
-            _stream()), "decay_scan")
+            B, S, H, G, dim, rows, _p(ws), _p(wdec), nseg, seglen, int(channel),
+            _p(weight), ones, _stream()), "decay_scan")
         return out
     return ref.decay_scan(q, k, v, state, step.positions, step.seq_ids, dim, vdim,
                           dt=dt, dt_bias=dt_bias, a_log=a_log, head_decay=head_decay,
-                          k_scale=k_scale, skip=skip, log_decay=log_decay)
+                          k_scale=k_scale, skip=skip, log_decay=log_decay, weight=weight,
+                          ones=bool(ones))
 
 
 CHUNKED_GLA_MIN_TOKENS = 96
@@ -747,13 +760,82 @@ def group_gated_norm(y, gate, weight, eps: float, groups: int, gate_first: bool,
     return ref.group_gated_norm(y, gate, weight, eps, groups, gate_first, out_dtype)
 
 
+CHUNKED_MLSTM_MIN_TOKENS = 64
+
+
+def mlstm(q, k, v, i_gate, f_gate, gate, i_bias, f_bias, gate_cap: float, norm_weight, eps: float,
+          state, max_state, step: StepLayout, dim: int, vdim: int):
+    """Matrix memory with exponential gates and its gated read-out norm (see
+    ref.mlstm). q, k (B,S,H*dim), v, gate (B,S,H*vdim), i_gate, f_gate
+    (B,S,H): raw projections, column slices of one GEMM output are fine;
+    ``state`` (slots, H, vdim + 1, dim) and ``max_state`` (slots, H) fp32 are
+    read (unless the row starts at position 0) and advanced. Returns
+    (B,S,H*vdim) in the gate's dtype. Single-token steps are one launch; long
+    bf16 rows run in chunks on the matrix cores; everything else is gates,
+    scan and read-out."""
+    B, S = v.shape[0], v.shape[1]
+    H = v.shape[-1] // vdim
+    k_scale = dim ** -0.5
+    if not v.is_cuda:
+        return ref.mlstm(q, k, v, i_gate, f_gate, gate, i_bias, f_bias, gate_cap, norm_weight, eps,
+                         state, max_state, step.positions, step.seq_ids, dim, vdim)
+    lib = _load()
+    assert q.dtype == k.dtype == v.dtype == gate.dtype == i_gate.dtype == f_gate.dtype
+    assert q.shape[-1] == k.shape[-1] == H * dim and gate.shape[-1] == H * vdim
+    assert i_gate.shape[-1] == f_gate.shape[-1] == i_bias.numel() == f_bias.numel() == H
+    assert state.dtype == max_state.dtype == torch.float32 and norm_weight.numel() == H * vdim
+    assert state.is_contiguous() and tuple(state.shape[1:]) == (H, vdim + 1, dim)
+    assert max_state.is_contiguous() and tuple(max_state.shape[1:]) == (H,)
+    bi, bf, nw = _f32(i_bias), _f32(f_bias), _f32(norm_weight)
+
+    def rows(t):
+        return _p(t), ctypes.c_long(_rows_view(t))
+
+    if S == 1 and dim <= 256:
+        out = torch.empty(B, S, H * vdim, dtype=gate.dtype, device=v.device)
+        _check(lib.nx_mlstm_decode(
+            *rows(q), *rows(k), *rows(v), *rows(i_gate), *rows(f_gate), _is_bf16(v), _p(bi), _p(bf),
+            ctypes.c_float(gate_cap), ctypes.c_float(k_scale), *rows(gate), _p(nw),
+            ctypes.c_float(eps), _p(state), _p(max_state), _p(step.positions), _p(step.seq_ids),
+            _p(out), B, H, dim, vdim, _stream()), "mlstm_decode")
+        return out
+    log_a, w, mx = torch.empty(3, B, S, H, dtype=torch.float32, device=v.device).unbind(0)
+    _check(lib.nx_mlstm_gates(
+        *rows(i_gate), *rows(f_gate), _is_bf16(i_gate), _p(bi), _p(bf), ctypes.c_float(gate_cap),
+        _p(max_state), _p(step.positions), _p(step.seq_ids), _p(step.nvalid), _p(log_a), _p(w),
+        _p(mx), B, S, H, _stream()), "mlstm_gates")
+    if S >= CHUNKED_MLSTM_MIN_TOKENS and dim <= 128 and vdim <= 128 and dim % 8 == 0 and \
+            vdim % 8 == 0 and v.dtype == torch.bfloat16 and \
+            all(_rows_view(t) % 8 == 0 and t.data_ptr() % 16 == 0 for t in (q, k, v, gate)):
+        nc = (S + 63) // 64
+        ws = torch.empty(B * nc * H * (vdim + 1) * dim, dtype=torch.float32, device=v.device)
+        wdec = torch.empty(B * nc * H, dtype=torch.float32, device=v.device)
+        out = torch.empty(B, S, H * vdim, dtype=torch.bfloat16, device=v.device)
+        _check(lib.nx_mlstm_chunked(
+            *rows(q), *rows(k), *rows(v), _p(log_a), _p(w), _p(mx), ctypes.c_float(k_scale),
+            *rows(gate), _p(nw), ctypes.c_float(eps), _p(state), _p(step.positions),
+            _p(step.seq_ids), _p(step.nvalid), _p(ws), _p(wdec), _p(out), B, S, H, dim, vdim,
+            _stream()), "mlstm_chunked")
+        return out
+    o = decay_scan(q, k, v, state, step, dim, vdim, k_scale=k_scale, log_decay=log_a, weight=w,
+                   ones=True)
+    out = torch.empty(B, S, H * vdim, dtype=gate.dtype, device=v.device)
+    _check(lib.nx_mlstm_readout(
+        _p(o), _p(mx), *rows(gate), _is_bf16(gate), _p(nw), ctypes.c_float(eps),
+        _p(step.positions), _p(out), ctypes.c_long(B * S), H, vdim, _stream()), "mlstm_readout")
+    return out
+
+
 def group_limited_router(logits, num_experts: int, top_k: int, n_groups: int = 1,
                          keep_groups: int = 1, scale: float = 1.0, normalize: bool = False,
-                         correction=None):
+                         correction=None, score: str = "softmax", group_top: int = 1,
+                         norm_eps: float = 0.0):
     """Group-limited top-k routing on fp32 logits (T, E + extra) (see
     ref.group_limited_router; ``correction`` (E,) shifts the scores for the
-    choice only): returns (dense (T, E + extra) weights with
+    choice only; ``score``: softmax or sigmoid; a group scores as the sum of
+    its ``group_top`` (1 or 2) best): returns (dense (T, E + extra) weights with
     sigmoid gates in the extra columns, idx (T, top_k) int32, weights)."""
+    assert score in ("softmax", "sigmoid") and group_top in (1, 2)
     if logits.is_cuda:
         lib = _load()
         T, C = logits.shape
@@ -766,12 +848,13 @@ def group_limited_router(logits, num_experts: int, top_k: int, n_groups: int = 1
         _check(lib.nx_group_router(
             _p(logits), ctypes.c_long(logits.stride(0)), E, C - E, top_k, max(n_groups, 1),
             max(min(keep_groups, n_groups), 1), ctypes.c_float(scale), int(normalize),
-            _p(None if correction is None else _f32(correction)),
+            _p(None if correction is None else _f32(correction)), int(score == "sigmoid"),
+            int(group_top == 2), ctypes.c_float(norm_eps),
             _p(dense), _p(idx), _p(wts), ctypes.c_long(T), _stream()), "group_limited_router")
         return dense, idx, wts
     return ref.group_limited_router(logits, num_experts, top_k, max(n_groups, 1),
                                     max(min(keep_groups, n_groups), 1), scale, normalize,
-                                    correction)
+                                    correction, score, group_top, norm_eps)
 
 
 FUSED_ROUTER_MAX_TOKENS = 512
@@ -779,12 +862,14 @@ FUSED_ROUTER_MAX_TOKENS = 512
 
 def route_tokens(x, weight, num_experts: int, top_k: int, n_groups: int = 1,
                  keep_groups: int = 1, scale: float = 1.0, normalize: bool = False,
-                 correction=None, bias=None):
+                 correction=None, bias=None, score: str = "softmax", group_top: int = 1,
+                 norm_eps: float = 0.0):
     """Router product and selection: fp32 logits ``x.float() @ weight.T + bias``
     (x (T, hidden) in any dtype, weight (E + extra, hidden) fp32), then
     :func:`group_limited_router`. Steps of few tokens do both in one launch;
     larger ones take the library product first."""
     T = x.shape[0]
+    assert score in ("softmax", "sigmoid") and group_top in (1, 2)
     if x.is_cuda and 0 < T <= FUSED_ROUTER_MAX_TOKENS and x.stride(-1) == 1:
         lib = _load()
         E, C = num_experts, weight.shape[0]
@@ -797,12 +882,13 @@ def route_tokens(x, weight, num_experts: int, top_k: int, n_groups: int = 1,
             _p(x), ctypes.c_long(x.stride(0)), _is_bf16(x), _p(weight), weight.shape[1], E, C - E,
             top_k, max(n_groups, 1), max(min(keep_groups, n_groups), 1), ctypes.c_float(scale),
             int(normalize), _p(None if correction is None else _f32(correction)),
-            _p(None if bias is None else _f32(bias)),
-            _p(dense), _p(idx), _p(wts), ctypes.c_long(T), _stream()), "route_tokens")
+            _p(None if bias is None else _f32(bias)), int(score == "sigmoid"),
+            int(group_top == 2), ctypes.c_float(norm_eps), _p(dense), _p(idx), _p(wts), ctypes.c_long(T), _stream()), "route_tokens")
         return dense, idx, wts
     logits = torch.nn.functional.linear(x.float(), weight, bias)
     return group_limited_router(logits, num_experts, top_k, n_groups, keep_groups, scale,
-                                normalize, correction=correction)
+                                normalize, correction=correction, score=score,
+                                group_top=group_top, norm_eps=norm_eps)
 
 
 def latent_row_write(x, norm_weight, eps: float, inv_freq, step: StepLayout, k_cache,
@@ -875,25 +961,37 @@ def clamped_glu_scale(hid, gates, expert_ff: int, num_experts: int, limit: float
     hid (T, 2*C) = [gate | up] of C = E*ff + shared columns -> (T, C), an
     expert's columns times the token's routing weight ``gates[t, e]`` (fp32,
     (T, >= E), row-strided), the shared columns with their own clamp."""
-    out_dtype = out_dtype or hid.dtype
     if hid.is_cuda:
-        lib = _load()
-        T, C2 = hid.shape
-        C = C2 // 2
-        assert hid.is_contiguous() and out_dtype == hid.dtype and C2 == 2 * C
-        assert num_experts * expert_ff <= C
-        if num_experts:
-            assert gates.dtype == torch.float32 and gates.stride(1) == 1
-            assert gates.shape[0] == T and gates.shape[1] >= num_experts
-        out = torch.empty(T, C, dtype=out_dtype, device=hid.device)
-        _check(lib.nx_clamped_glu_scale(
-            _p(hid), _is_bf16(hid), _p(gates if num_experts else None),
-            ctypes.c_long(gates.stride(0) if num_experts else 0), expert_ff, num_experts,
-            ctypes.c_float(limit), ctypes.c_float(shared_limit), ctypes.c_float(alpha),
-            _p(out), ctypes.c_long(T), C, _stream()), "clamped_glu_scale")
-        return out
+        return _glu_scale(hid, gates, expert_ff, num_experts, 0, limit, shared_limit, alpha,
+                          out_dtype)
     return ref.clamped_glu_scale(hid, gates, expert_ff, num_experts, limit, shared_limit,
-                                 alpha, out_dtype)
+                                 alpha, out_dtype or hid.dtype)
+
+
+def silu_glu_scale(hid, gates, expert_ff: int, num_experts: int, out_dtype=None):
+    """silu(gate) * up of stacked experts, times the token's routing weight (see
+    :func:`clamped_glu_scale` for the layout)."""
+    if hid.is_cuda:
+        return _glu_scale(hid, gates, expert_ff, num_experts, 1, 0.0, 0.0, 0.0, out_dtype)
+    return ref.silu_glu_scale(hid, gates, expert_ff, num_experts, out_dtype or hid.dtype)
+
+
+def _glu_scale(hid, gates, expert_ff, num_experts, act, limit, shared_limit, alpha, out_dtype):
+    lib = _load()
+    T, C2 = hid.shape
+    C = C2 // 2
+    assert hid.is_contiguous() and out_dtype in (None, hid.dtype) and C2 == 2 * C
+    assert num_experts * expert_ff <= C
+    if num_experts:
+        assert gates.dtype == torch.float32 and gates.stride(1) == 1
+        assert gates.shape[0] == T and gates.shape[1] >= num_experts
+    out = torch.empty(T, C, dtype=hid.dtype, device=hid.device)
+    _check(lib.nx_glu_scale(
+        _p(hid), _is_bf16(hid), _p(gates if num_experts else None),
+        ctypes.c_long(gates.stride(0) if num_experts else 0), expert_ff, num_experts, act,
+        ctypes.c_float(limit), ctypes.c_float(shared_limit), ctypes.c_float(alpha),
+        _p(out), ctypes.c_long(T), C, _stream()), "glu_scale")
+    return out
 
 
 def sigmoid_gate_(y, gate):
@@ -1010,3 +1108,102 @@ def token_gate_proj(h, weight, ids, table, offset: int):
             ctypes.c_long(ids.numel()), C, _stream()), "token_gate_proj")
         return out
     return token_gate(torch.nn.functional.linear(h, weight), ids, table, offset)
+
+
+def hyper_step(streams, y, mix, w_out, w_in, norm_weight, eps: float, out_dtype,
+               keep: bool = True):
+    """One step of a residual kept as parallel streams (fp32): stream t becomes
+    sum_s mix[s, t] streams_s + w_out[t] * y, then their weighted sum
+    u = sum_t w_in[t] x_t is normed for the next sublayer (layer norm with a
+    weight, fp32 statistics). ``streams`` (B,S,n,C), or (B,S,C) when all of
+    them still equal one row; ``y`` None reads the streams without changing
+    them; ``w_in`` None is the plain sum and ``norm_weight`` None returns u
+    itself in fp32. Returns (streams, the normed u in ``out_dtype``);
+    ``streams`` is updated in place where it can be, and not made anew
+    without ``keep``."""
+    n = mix.shape[0]
+    B, S, C = streams.shape[0], streams.shape[1], streams.shape[-1]
+    shared = streams.dim() == 3
+    if streams.is_cuda:
+        lib = _load()
+        assert streams.dtype == torch.float32 and streams.is_contiguous()
+        assert shared or streams.shape[2] == n
+        assert tuple(mix.shape) == (n, n) and w_out.numel() == n
+        assert w_in is None or w_in.numel() == n
+        keep = keep and y is not None
+        vec = n <= 4 and C % 4 == 0 and C <= 8192
+        if y is not None:
+            y = y.contiguous()
+            assert y.numel() == B * S * C
+        new = streams
+        if keep and (shared or not vec):
+            new = torch.empty(B, S, n, C, dtype=torch.float32, device=streams.device)
+        dt = y.dtype if y is not None else out_dtype
+        assert norm_weight is None or out_dtype == dt
+        h = torch.empty(B, S, C, dtype=torch.float32 if norm_weight is None else out_dtype,
+                        device=streams.device)
+        scratch = None
+        if norm_weight is not None and not vec:
+            scratch = torch.empty(B * S * C, dtype=torch.float32, device=streams.device)
+        _check(lib.nx_hyper_step(
+            _p(streams), ctypes.c_long(C if shared else n * C), ctypes.c_long(0 if shared else C),
+            _p(y), int(dt == torch.bfloat16), _p(_f32(mix)), _p(_f32(w_out)),
+            _p(new if keep else None), _p(None if w_in is None else _f32(w_in)),
+            _p(None if norm_weight is None else _f32(norm_weight)), ctypes.c_float(eps),
+            _p(None if norm_weight is None else h), _p(h if norm_weight is None else None),
+            _p(scratch), ctypes.c_long(B * S), n, C, _stream()), "hyper_step")
+        return new, h
+    new, u = ref.hyper_step(streams, y, mix, w_out, w_in)
+    if norm_weight is not None:
+        u = ref.layer_norm(u, norm_weight, eps, out_dtype)
+    return new, u
+
+
+def attention_rows(q, k, v, step: StepLayout, inv_freq, unit_norm: bool, eps: float, k_cache,
+                   v_cache, slot_mapping, v_first=None, v_lambda=None):
+    """Query, key and value rows of a step in one launch: q (B,S,H*D) and k
+    (B,S,G*D) rotated (half-split pairs of the first 2*len(inv_freq)
+    channels, fp32 angles; None = not) and, with ``unit_norm``, divided by
+    their root mean square per head; keys and values (B,S,G*Dv) scattered into
+    the paged caches (blocks, block, G, D*) at ``slot_mapping``; with
+    ``v_first`` (same shape as v) the values are (1 - lambda) v + lambda
+    v_first, ``v_lambda`` a one-element fp32 tensor. Column slices of a fused
+    projection are fine. Returns the queries, dense."""
+    B, S = q.shape[0], q.shape[1]
+    G, D = k_cache.shape[2], k_cache.shape[3]
+    Dv = v_cache.shape[3]
+    H = q.shape[-1] // D
+    assert k.shape[-1] == G * D and v.shape[-1] == G * Dv and q.shape[-1] == H * D
+    assert v_first is None or (v_first.shape == v.shape and v_lambda is not None)
+    if q.is_cuda:
+        lib = _load()
+        assert q.dtype == k.dtype == v.dtype == k_cache.dtype == v_cache.dtype
+        assert k_cache.is_contiguous() and v_cache.is_contiguous()
+        half = 0 if inv_freq is None else inv_freq.numel()
+        if v_first is not None:
+            assert v_first.dtype == v.dtype and v_lambda.dtype == torch.float32
+            assert v_lambda.numel() == 1
+        out = torch.empty(B, S, H * D, dtype=q.dtype, device=q.device)
+        _check(lib.nx_qkv_rows(
+            _p(q), ctypes.c_long(_rows_view(q)), _p(k), ctypes.c_long(_rows_view(k)),
+            _p(v), ctypes.c_long(_rows_view(v)), _p(v_first),
+            ctypes.c_long(0 if v_first is None else _rows_view(v_first)),
+            _p(v_lambda if v_first is not None else None), _is_bf16(q), _p(step.positions),
+            _p(step.i32(slot_mapping)), _p(_f32(inv_freq) if half else None), half,
+            int(bool(unit_norm)), ctypes.c_float(eps), _p(out), _p(k_cache), _p(v_cache),
+            ctypes.c_long(k_cache.shape[0] * k_cache.shape[1]), ctypes.c_long(B * S), H, G, D, Dv,
+            _stream()), "attention_rows")
+        return out
+
+    def rows(x, n):
+        x = ref.head_norm_rotate(x.reshape(B, S, n, D), step.positions, None, 0.0, inv_freq)
+        if unit_norm:
+            x = x * torch.rsqrt((x * x).mean(-1, keepdim=True) + eps)
+        return x.to(q.dtype)
+
+    if v_first is not None:
+        lam = v_lambda.float().reshape(())
+        v = ((1.0 - lam) * v.float() + lam * v_first.float()).to(v.dtype)
+    ref.paged_kv_write(k_cache, v_cache, rows(k, G).view(B * S, G, D), v.reshape(B * S, G, Dv),
+                       slot_mapping)
+    return rows(q, H).view(B, S, H * D)

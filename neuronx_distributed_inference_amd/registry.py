@@ -86,6 +86,11 @@ _REGISTRY: Dict[str, Tuple[str, str, str]] = {
         "RisutarInferenceConfig",
         "RisutarForCausalLM",
     ),
+    "sitidra": (
+        "neuronx_distributed_inference_amd.models.sitidra.modeling_sitidra",
+        "SitidraInferenceConfig",
+        "SitidraForCausalLM",
+    ),
     "soputar": (
         "neuronx_distributed_inference_amd.models.soputar.modeling_soputar",
         "SoputarInferenceConfig",
