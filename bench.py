@@ -75,11 +75,13 @@ def parse_args():
                         "parallel, retention, routed experts; Tamilix: chunk-local slope "
                         "attention, windowed gated latent attention, identity-routed "
                         "experts; Risutar: latent attention, gated linear attention, "
-                        "routed gelu experts) beside Llama at equal "
+                        "routed gelu experts; Sitidra: parallel residual streams, "
+                        "chunk-local rotary attention, matrix memory with exponential "
+                        "gates, routed silu experts) beside Llama at equal "
                         "width/depth/ff/vocab")
-    p.add_argument("--hybrid-models", default="llama,nabelix,soputar,kuterax,tamilix,risutar",
+    p.add_argument("--hybrid-models", default="llama,nabelix,soputar,kuterax,tamilix,risutar,sitidra",
                    help="comma-separated subset of llama,nabelix,soputar,kuterax,tamilix,"
-                        "risutar for --hybrid")
+                        "risutar,sitidra for --hybrid")
     p.add_argument("--hybrid-sizes", default="2048,4096",
                    help="comma-separated layer widths for --hybrid")
     p.add_argument("--hybrid-layers", type=int, default=4)
@@ -124,6 +126,9 @@ def run_hybrid_bench(args):
     )
     from neuronx_distributed_inference_amd.models.risutar.modeling_risutar import (
         RisutarForCausalLM, RisutarInferenceConfig,
+    )
+    from neuronx_distributed_inference_amd.models.sitidra.modeling_sitidra import (
+        SitidraForCausalLM, SitidraInferenceConfig,
     )
 
     dtype = "bfloat16" if on_gpu else "float32"
@@ -265,6 +270,27 @@ def run_hybrid_bench(args):
                 embedding={"bigram": {"buckets": 65536, "mul_prev": 40503, "mul_cur": 9973}},
                 token_side={"dim": 64}, postln_alpha=(2.0 * L) ** 0.25, norm={"eps": 1e-5})
             cls = RisutarForCausalLM
+        elif kind == "sitidra":
+            # the design's layer mix, repeated to depth L: attention and matrix-memory
+            # layers in turn on four residual streams, blocks of 1024 positions, values
+            # blended, every layer with routed experts: four of sixteen of ff/8 (in four
+            # groups of which two stay) plus a shared expert of ff/2
+            moe = {"kind": "moe", "expert": {"ff": ff // 8}, "shared": {"ff": ff // 2},
+                   "router": {"experts": 16, "top": 4, "groups": {"count": 4, "keep": 2},
+                              "scale": 2.0}}
+            pair = [
+                {"type": "attention", "mlp": moe, "mixer": {
+                    "heads": H, "kv_heads": G, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                    "mask": {"size": 1024}, "rot": {"base": 10000.0, "dims": 128},
+                    "v_mix": True}},
+                {"type": "mlstm", "mlp": moe, "mixer": {
+                    "heads": H, "dim": 128, "vdim": 128, "gate_cap": 15.0}},
+            ]
+            cfg = SitidraInferenceConfig(
+                neuron_config=ec, architecture="Sitidra", width=width, vocab=V,
+                layers=[json.loads(json.dumps(pair[i % 2])) for i in range(L)], streams=4,
+                norm={"eps": 1e-5}, logit_softcap=30.0)
+            cls = SitidraForCausalLM
         else:
             layer = {"type": "parallel", "mlp": {"kind": "dense", "ff": ff}, "mixer": {
                 "left": {"heads": H, "kv_heads": G, "dim": 128, "vdim": 128,
@@ -292,7 +318,8 @@ def run_hybrid_bench(args):
         return m
 
     for width in [int(x) for x in args.hybrid_sizes.split(",")]:
-        for kind in [k for k in ("llama", "nabelix", "soputar", "kuterax", "tamilix", "risutar")
+        for kind in [k for k in ("llama", "nabelix", "soputar", "kuterax", "tamilix", "risutar",
+                                  "sitidra")
                      if k in args.hybrid_models.split(",")]:
             with torch.inference_mode():
                 # ---- prefill: one prompt, three timed repetitions

@@ -3591,16 +3591,18 @@ qkv_rows_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, long 
 // state of a head is (Dv + 1) rows of D key channels: a row per value channel, then n
 // (the row of a value channel that is always one). Both exponents are never positive.
 DEV void mlstm_gate_(float zi, float zf, float cap, float& i, float& f) {
-    i = cap * tanhf(zi / cap);
     const float x = cap * tanhf(zf / cap);
+    i = cap * tanhf(zi / cap);
     f = fminf(x, 0.f) - log1pf(expf(-fabsf(x)));
 }
 
 #define MG_THREADS 512
+#define MG_KEEP 8
 // One workgroup per (row, head): log a, w and m of every token of the step, and the
 // carried m. A thread owns consecutive tokens; (sum of f, running maximum from minus
 // infinity) pairs of the threads' spans are combined by a scan, then every thread
-// walks its span from its true start.
+// walks its span from its true start. Spans of up to MG_KEEP tokens keep their gates
+// in registers, longer ones make them again.
 template <typename T>
 __global__ void __launch_bounds__(MG_THREADS)
 mlstm_gates_kernel(const T* __restrict__ zi, long zis, const T* __restrict__ zf, long zfs,
@@ -3619,12 +3621,30 @@ mlstm_gates_kernel(const T* __restrict__ zi, long zis, const T* __restrict__ zf,
     const float bih = bi[h], bfh = bf[h];
     const long tok0 = (long)b * S;
     float F = 0.f, M = -INFINITY;
-    for (int t = t0; t < t1; ++t) {
-        float i, f;
-        mlstm_gate_(ldf<T>(zi + (tok0 + t) * zis + h) + bih,
-                    ldf<T>(zf + (tok0 + t) * zfs + h) + bfh, cap, i, f);
-        F += f;
-        M = fmaxf(M + f, i);
+    float ik[MG_KEEP], fk[MG_KEEP];
+    const bool kept_all = per <= MG_KEEP;                 // uniform
+    if (kept_all) {
+#pragma unroll
+        for (int x = 0; x < MG_KEEP; ++x) {               // loads in flight together
+            const long tk = tok0 + min(t0 + x, n - 1);
+            ik[x] = ldf<T>(zi + tk * zis + h) + bih;
+            fk[x] = ldf<T>(zf + tk * zfs + h) + bfh;
+        }
+#pragma unroll
+        for (int x = 0; x < MG_KEEP; ++x) {
+            if (x >= t1 - t0) continue;
+            mlstm_gate_(ik[x], fk[x], cap, ik[x], fk[x]);
+            F += fk[x];
+            M = fmaxf(M + fk[x], ik[x]);
+        }
+    } else {
+        for (int t = t0; t < t1; ++t) {
+            float i, f;
+            mlstm_gate_(ldf<T>(zi + (tok0 + t) * zis + h) + bih,
+                        ldf<T>(zf + (tok0 + t) * zfs + h) + bfh, cap, i, f);
+            F += f;
+            M = fmaxf(M + f, i);
+        }
     }
     float pf = F, pm = M;                                 // inclusive over the wave
 #pragma unroll
@@ -3638,16 +3658,25 @@ mlstm_gates_kernel(const T* __restrict__ zi, long zis, const T* __restrict__ zf,
     for (int x = 0; x < wv; ++x) m = fmaxf(m + wf[x], wm[x]);
     const float ef = __shfl_up(pf, 1, WAVE), em = __shfl_up(pm, 1, WAVE);
     if (lane > 0) m = fmaxf(m + ef, em);
-    for (int t = t0; t < t1; ++t) {
-        float i, f;
-        mlstm_gate_(ldf<T>(zi + (tok0 + t) * zis + h) + bih,
-                    ldf<T>(zf + (tok0 + t) * zfs + h) + bfh, cap, i, f);
+    auto step = [&](int t, float i, float f) {
         const float kept = f + m;
         m = fmaxf(kept, i);
         const long at = (tok0 + t) * H + h;
         ld[at] = kept - m;
         wt[at] = expf(i - m);
         mx[at] = m;
+    };
+    if (kept_all) {
+#pragma unroll
+        for (int x = 0; x < MG_KEEP; ++x)
+            if (x < t1 - t0) step(t0 + x, ik[x], fk[x]);
+    } else {
+        for (int t = t0; t < t1; ++t) {
+            float i, f;
+            mlstm_gate_(ldf<T>(zi + (tok0 + t) * zis + h) + bih,
+                        ldf<T>(zf + (tok0 + t) * zfs + h) + bfh, cap, i, f);
+            step(t, i, f);
+        }
     }
     __syncthreads();                                      // every thread has read the carried m
     if (t1 == n && t0 < n) mstate[(long)slot * H + h] = m;

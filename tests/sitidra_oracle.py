@@ -240,5 +240,6 @@ def forward(cfg, weights, tokens, collect=None):
         if collect is not None:
             collect.append(xs.sum(1))
     x = layer_norm(xs.sum(1), _w(weights, "final.norm"), cfg["norm"]["eps"])
-    cap = cfg["logit_softcap"]
-    return cap * torch.tanh(x @ _w(weights, "head").T / cap)
+    logits = x @ _w(weights, "head").T
+    cap = cfg.get("logit_softcap")
+    return cap * torch.tanh(logits / cap) if cap else logits
