@@ -525,6 +525,39 @@ def test_the_running_maximum_starts_at_zero(device):
     assert abs(mx.item() + 0.6931) < 1e-3                # f of the first token, not its i
 
 
+@pytest.mark.parametrize("device,dtype", [
+    ("cpu", F32), pytest.param("cuda", F32, marks=pytest.mark.gpu),
+    pytest.param("cuda", BF16, marks=pytest.mark.gpu)])
+def test_the_denominators_constant(device, dtype):
+    """Large gates (exp(-m) far below 1e-6) and a query orthogonal to the
+    normalizer: the constant 1e-6 is what divides, and with values this small
+    next to the norm's eps it shows. The first two tokens write, the rest read."""
+    H, D, Dv, T, eps, cap = 1, 8, 16, 128, 1e-4, 16.0
+    torch.manual_seed(14)
+    k = torch.zeros(T, D)
+    k[0, 0] = k[1, 1] = 1.0
+    q = torch.zeros(T, D)
+    q[:, 0], q[:, 1] = 1.0, -1.0
+    v = (torch.randn(T, Dv) * 3e-8).to(dtype).float()
+    z = torch.full((T, H), 64.0)
+    i, f = oracle.mlstm_gates(z.double(), z.double(), cap)
+    o, (_, _, m) = oracle.mlstm_scan(q.double().view(T, H, D) * D ** -0.5, k.double().view(T, H, D),
+                                     v.double().view(T, H, Dv), i, f)
+    assert torch.exp(-m).item() < 2e-7
+    want = oracle.rms(o, eps).view(T, Dv) * 0.5
+    for cuts in ([T], [64, 62, 1, 1], [2] * 3 + [T - 6], [1] * 6 + [T - 6]):
+        mem, mx = torch.zeros(1, H, Dv + 1, D, device=device), torch.zeros(1, H, device=device)
+        got, at = [], 0
+        zero, one = torch.zeros(H, device=device), torch.ones(H * Dv, device=device)
+        for n in cuts:
+            st = step_of(torch.arange(at, at + n).view(1, n), [0], device)
+            part = [t[None, at:at + n].to(device, dtype) for t in (q, k, v, z, z, torch.zeros(T, Dv))]
+            got.append(seqmix.mlstm(*part, zero, zero, cap, one, eps, mem, mx, st, D, Dv)[0].cpu())
+            at += n
+        assert want[1:].abs().mean() > 0.05
+        close(torch.cat(got), want, 2e-3, 0.05)
+
+
 @pytest.mark.gpu
 @pytest.mark.parametrize("H,D,Dv,T,cuts", [
     (2, 64, 48, 300, [300]), (3, 128, 128, 700, [700]), (2, 32, 64, 520, [257, 1, 262]),
