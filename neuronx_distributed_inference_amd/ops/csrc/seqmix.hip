@@ -1931,17 +1931,17 @@ head_norm_rope_kernel(const TIn* __restrict__ x, long xt, long xh, TOut* __restr
 
 // ----------------------------------------------------- decayed linear recurrence
 // S_t = a_t S_{t-1} + k_t (w_t v_t)^T, o_t = S_t^T q_t (+ skip_h v_t), one scalar
-// decay per head and token, or (CH) one per key channel: S_t = diag(a_t) S_{t-1} +
+// decay per head and token, or (KIND 1) one per key channel: S_t = diag(a_t) S_{t-1} +
 // k_t v_t^T. Workgroup = (row, head, 16 value channels); the 16
 // lanes of a channel split its key rows (lane p owns rows p*R .. p*R+R-1), the
 // state sits in registers for the whole step and is read/written once. Tokens
 // are staged through LDS in chunks of DS_TC (q, k, v, decay, step size), so
 // global loads are coalesced and the serial loop reads only LDS.
 // Decay: selective (dt projection + dt_bias, a_log: w = softplus(dt + bias),
-// a = exp(-exp(a_log) w)), fixed per head (head_decay: a = decay, w = 1), or given
-// (wgt: a = exp(dt), w = wgt, both per head and token). CH takes
-// `dt` (H*D wide, fp32) as the decays' logarithms. `ones`: the last of the Dv value
-// channels is not read but one (a normalizer row).
+// a = exp(-exp(a_log) w)) or fixed per head (head_decay: a = decay, w = 1). KIND 1 takes
+// `dt` (H*D wide, fp32) as the decays' logarithms. KIND 2: both are given per head and
+// token, a = exp(dt), w = wgt, and the last of the Dv value channels is not read but one
+// (a normalizer row).
 //
 // Long rows with few workgroups are cut into `nseg` segments of `seglen`
 // tokens that run side by side; the recurrence is linear in the state, so
@@ -1955,7 +1955,7 @@ head_norm_rope_kernel(const TIn* __restrict__ x, long xt, long xh, TOut* __restr
 // MODE 0 is the plain single pass (decode steps, short portions, full batches).
 #define DS_TC 16
 
-template <typename T, typename TD, int R, int MODE, bool CH>
+template <typename T, typename TD, int R, int MODE, int KIND>
 __global__ void __launch_bounds__(256)
 decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, long ks,
                   const T* __restrict__ v, long vs, const TD* __restrict__ dt, long dts,
@@ -1965,8 +1965,9 @@ decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, lon
                   const int* __restrict__ pos, const int* __restrict__ seq,
                   const int* __restrict__ nvalid, float* __restrict__ out, int S, int H, int G,
                   int D, int Dv, float* __restrict__ ws, float* __restrict__ wdec, int nseg,
-                  int seglen, const float* __restrict__ wgt, int ones) {
+                  int seglen, const float* __restrict__ wgt) {
     constexpr int DP = 16 * R;
+    constexpr bool CH = KIND == 1;
     __shared__ __attribute__((aligned(16))) float sd[CH ? DS_TC : 1][CH ? DP : 4];
     __shared__ __attribute__((aligned(16))) float sq[MODE == 1 ? 1 : DS_TC][DP], sk[DS_TC][DP];
     __shared__ float sv[DS_TC][16], sa[DS_TC], sw[DS_TC];
@@ -2033,13 +2034,13 @@ decay_scan_kernel(const T* __restrict__ q, long qs, const T* __restrict__ k, lon
             const int tt = tid >> 4, cc = tid & 15;       // 256 = DS_TC * 16
             float vv = 0.f;
             if (tt < cnt && c0 + cc < Dv)
-                vv = ones && c0 + cc == Dv - 1 ? 1.f
-                    : ldf<T>(v + ((long)b * S + t0 + tt) * vs + (long)h * (Dv - ones) + c0 + cc);
+                vv = KIND == 2 && c0 + cc == Dv - 1 ? 1.f
+                    : ldf<T>(v + ((long)b * S + t0 + tt) * vs + (long)h * (Dv - (KIND == 2)) + c0 + cc);
             sv[tt][cc] = vv;
         }
         if (!CH && tid < cnt) {
             float a, w = 1.f;
-            if (wgt) {
+            if constexpr (KIND == 2) {
                 const long tok = (long)b * S + t0 + tid;
                 w = wgt[tok * H + h];
                 a = expf(ldf<TD>(dt + tok * dts + h));
@@ -4562,14 +4563,13 @@ int nx_decay_scan(const void* q, long qs, const void* k, long ks, const void* v,
                   const float* a_log, const float* head_decay, float k_scale, const float* skip,
                   float* state, const int* pos, const int* seq, const int* nvalid, float* out,
                   int B, int S, int H, int G, int D, int Dv, float* ws, float* wdec, int nseg,
-                  int seglen, int channel, const float* wgt, int ones, hipStream_t st) {
+                  int seglen, int kind, const float* wgt, hipStream_t st) {
     if ((long)B * S <= 0) return 0;
     if (D <= 0 || Dv <= 0 || G <= 0 || H % G != 0 || D > 256) return -1;
     if ((dt == nullptr) == (head_decay == nullptr)) return -2;
-    if (dt && !channel && !wgt && (!dt_bias || !a_log)) return -2;
-    if (wgt && (!dt || dt_bf16 || channel)) return -2;
-    if (ones < 0 || ones > 1 || (ones && (Dv < 2 || skip))) return -2;
-    if (channel && (!dt || dt_bf16 || a_log || skip)) return -2;
+    if (dt && kind == 0 && (!dt_bias || !a_log)) return -2;
+    if (kind != 0 && (!dt || dt_bf16 || a_log || skip)) return -2;
+    if (kind < 0 || kind > 2 || (kind == 2 && (!wgt || Dv < 2))) return -2;
     if (H > 65535 || B > 65535) return -3;
     // the kernel reads state rows 16 bytes at a time when dim % 4 == 0
     if (((uintptr_t)state % 16) != 0 || ((uintptr_t)ws % 16) != 0) return -5;
@@ -4580,23 +4580,24 @@ int nx_decay_scan(const void* q, long qs, const void* k, long ks, const void* v,
 #define DSK(T, TD, RV, MD, CHV) decay_scan_kernel<T, TD, RV, MD, CHV><<<grid, block, 0, st>>>( \
         (const T*)q, qs, (const T*)k, ks, (const T*)v, vs, (const TD*)dt, dts, dt_bias, a_log, \
         head_decay, k_scale, skip, state, pos, seq, nvalid, out, S, H, G, D, Dv, ws, wdec, nseg, \
-        seglen, wgt, ones)
+        seglen, wgt)
 #define DSR(T, TD, MD, CHV) do { if (D <= 16) DSK(T, TD, 1, MD, CHV); \
         else if (D <= 32) DSK(T, TD, 2, MD, CHV); \
         else if (D <= 64) DSK(T, TD, 4, MD, CHV); else if (D <= 128) DSK(T, TD, 8, MD, CHV); \
         else DSK(T, TD, 16, MD, CHV); } while (0)
 #define DST(MD) do { \
-        if (in_bf16) { if (dt_bf16) DSR(bf16, bf16, MD, false); else DSR(bf16, float, MD, false); } \
-        else { if (dt_bf16) DSR(float, bf16, MD, false); else DSR(float, float, MD, false); } } while (0)
-#define DSC(MD) do { if (!channel) DST(MD); else if (in_bf16) DSR(bf16, float, MD, true); \
-        else DSR(float, float, MD, true); } while (0)
+        if (in_bf16) { if (dt_bf16) DSR(bf16, bf16, MD, 0); else DSR(bf16, float, MD, 0); } \
+        else { if (dt_bf16) DSR(float, bf16, MD, 0); else DSR(float, float, MD, 0); } } while (0)
+#define DSC(MD) do { if (kind == 0) DST(MD); \
+        else if (kind == 1) { if (in_bf16) DSR(bf16, float, MD, 1); else DSR(float, float, MD, 1); } \
+        else { if (in_bf16) DSR(bf16, float, MD, 2); else DSR(float, float, MD, 2); } } while (0)
     if (nseg == 1) {
         DSC(0);
     } else {
         DSC(1);
         const long per_head = (long)Dv * D;
         decay_scan_link_kernel<<<grid_for((long)B * H * per_head, 256), 256, 0, st>>>(
-            ws, wdec, state, pos, seq, nvalid, B, S, H, per_head, nseg, channel ? D : 1);
+            ws, wdec, state, pos, seq, nvalid, B, S, H, per_head, nseg, kind == 1 ? D : 1);
         DSC(2);
     }
 #undef DSC

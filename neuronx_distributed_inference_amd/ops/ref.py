@@ -498,7 +498,7 @@ def low_rank_decay(low, weight, bias, tau: float):
 
 def decay_scan(q, k, v, state, positions, seq_ids, dim: int, vdim: int,
                dt=None, dt_bias=None, a_log=None, head_decay=None,
-               k_scale: float = 1.0, skip=None, log_decay=None, weight=None, ones: bool = False):
+               k_scale: float = 1.0, skip=None, log_decay=None, weight=None):
     """Linear recurrence with a decay per head and matrix state, carried in ``state`` (slots, H, vdim, dim) fp32 (stored transposed):
 
         S_t = a_t S_{t-1} + k_t (w_t v_t)^T ;  o_t = S_t^T q_t (+ skip_h v_t)
@@ -510,7 +510,7 @@ def decay_scan(q, k, v, state, positions, seq_ids, dim: int, vdim: int,
     ``log_decay`` (B,S,H*dim): a decay per head and KEY CHANNEL, S_t =
     diag(exp(log_decay_t)) S_{t-1} + k_t v_t^T (gated linear attention); or
     ``log_decay`` and ``weight`` (B,S,H) each: a_t = exp(log_decay_t), w_t =
-    weight_t. ``ones`` appends a value channel that is always one (state and
+    weight_t, with a value channel that is always one appended (state and
     output have one more row per head). q, k
     (B,S,G*dim) are shared by H/G consecutive heads, v (B,S,H*vdim); k is
     multiplied by ``k_scale``. Returns fp32 (B,S,H*vdim)."""
@@ -522,7 +522,7 @@ def decay_scan(q, k, v, state, positions, seq_ids, dim: int, vdim: int,
     qf = q.float().reshape(B, S, G, D).repeat_interleave(rep, dim=2)
     kf = (k.float() * k_scale).reshape(B, S, G, D).repeat_interleave(rep, dim=2)
     vf = v.float().reshape(B, S, H, Dv)
-    if ones:
+    if weight is not None:
         vf = torch.cat([vf, torch.ones_like(vf[..., :1])], dim=-1)
         Dv = Dv + 1
     if weight is not None:
@@ -592,7 +592,7 @@ def mlstm(q, k, v, i_gate, f_gate, gate, i_bias, f_bias, gate_cap: float, norm_w
             log_a[b, t], w[b, t], mx[b, t] = kept - m, torch.exp(i[b, t] - m), m
         max_state[slot] = m
     o = decay_scan(q, k, v, state, positions, seq_ids, dim, vdim, k_scale=dim ** -0.5,
-                   log_decay=log_a, weight=w, ones=True).view(B, S, H, vdim + 1)
+                   log_decay=log_a, weight=w).view(B, S, H, vdim + 1)
     den = torch.maximum(o[..., vdim].abs(), torch.exp(-mx)) + 1e-6
     o = o[..., :vdim] / den.unsqueeze(-1)
     o = o * torch.rsqrt((o * o).mean(-1, keepdim=True) + eps)

@@ -636,27 +636,26 @@ def low_rank_decay(low, weight, bias, tau: float):
 
 def decay_scan(q, k, v, state, step: StepLayout, dim: int, vdim: int, dt=None,
                dt_bias=None, a_log=None, head_decay=None, k_scale: float = 1.0, skip=None,
-               log_decay=None, weight=None, ones: bool = False):
+               log_decay=None, weight=None):
     """Decayed linear recurrence with matrix state (see ref.decay_scan):
     selective state spaces (``dt``/``dt_bias``/``a_log``), fixed per-head
     decays (``head_decay``), a decay per key channel (its logarithm
     ``log_decay`` (B,S,H*dim) fp32) or, with ``weight`` (B,S,H) fp32, given
-    log decays (B,S,H) and write weights per head and token. q, k (B,S,G*dim),
-    v (B,S,H*vdim) may be column
-    slices of wider tensors; ``state`` (slots, H, vdim, dim) fp32 is read
-    (unless the row starts at position 0) and advanced. With ``ones`` the
-    state has one more row per head, of a value channel that is always one,
-    and so has the output. Returns fp32."""
+    log decays (B,S,H) and write weights per head and token; the state then
+    has one more row per head, of a value channel that is always one (a
+    normalizer), and so has the output. q, k (B,S,G*dim), v (B,S,H*vdim) may
+    be column slices of wider tensors; ``state`` (slots, H, vdim [+ 1], dim)
+    fp32 is read (unless the row starts at position 0) and advanced. Returns
+    fp32."""
     assert sum(x is not None for x in (dt, head_decay, log_decay)) == 1
     assert weight is None or log_decay is not None
-    ones = int(bool(ones))
     if v.is_cuda:
         lib = _load()
         B, S = v.shape[0], v.shape[1]
         H = v.shape[-1] // vdim
         G = q.shape[-1] // dim
         assert q.dtype == k.dtype == v.dtype and state.dtype == torch.float32
-        rows = vdim + ones
+        rows = vdim + int(weight is not None)
         assert state.is_contiguous() and tuple(state.shape[1:]) == (H, rows, dim)
         assert H % G == 0 and q.shape[-1] == G * dim and k.shape[-1] == G * dim
         out = torch.empty(B, S, H * rows, dtype=torch.float32, device=v.device)
@@ -693,13 +692,12 @@ def decay_scan(q, k, v, state, step: StepLayout, dim: int, vdim: int, dt=None,
             _p(None if head_decay is None else _f32(head_decay)),
             ctypes.c_float(k_scale), _p(None if skip is None else _f32(skip)),
             _p(state), _p(step.positions), _p(step.seq_ids), _p(step.nvalid), _p(out),
-            B, S, H, G, dim, rows, _p(ws), _p(wdec), nseg, seglen, int(channel),
-            _p(weight), ones, _stream()), "decay_scan")
+            B, S, H, G, dim, rows, _p(ws), _p(wdec), nseg, seglen,
+            2 if weight is not None else int(channel), _p(weight), _stream()), "decay_scan")
         return out
     return ref.decay_scan(q, k, v, state, step.positions, step.seq_ids, dim, vdim,
                           dt=dt, dt_bias=dt_bias, a_log=a_log, head_decay=head_decay,
-                          k_scale=k_scale, skip=skip, log_decay=log_decay, weight=weight,
-                          ones=bool(ones))
+                          k_scale=k_scale, skip=skip, log_decay=log_decay, weight=weight)
 
 
 CHUNKED_GLA_MIN_TOKENS = 96
@@ -817,8 +815,7 @@ def mlstm(q, k, v, i_gate, f_gate, gate, i_bias, f_bias, gate_cap: float, norm_w
             _p(step.seq_ids), _p(step.nvalid), _p(ws), _p(wdec), _p(out), B, S, H, dim, vdim,
             _stream()), "mlstm_chunked")
         return out
-    o = decay_scan(q, k, v, state, step, dim, vdim, k_scale=k_scale, log_decay=log_a, weight=w,
-                   ones=True)
+    o = decay_scan(q, k, v, state, step, dim, vdim, k_scale=k_scale, log_decay=log_a, weight=w)
     out = torch.empty(B, S, H * vdim, dtype=gate.dtype, device=v.device)
     _check(lib.nx_mlstm_readout(
         _p(o), _p(mx), *rows(gate), _is_bf16(gate), _p(nw), ctypes.c_float(eps),
