@@ -3,8 +3,10 @@
 // short causal convolutions with a carried tail, paged KV scatter with distinct
 // K/V head sizes, interleaved rotary positions, paged softmax attention with
 // optional sliding window / always-visible first tokens / log-distance penalty /
-// query temperature / tanh score cap / softmax sink, the gated delta-rule
-// linear recurrence, and gated feed-forward activations.
+// query temperature / tanh score cap / softmax sink, linear recurrences with matrix
+// state (gated delta rule, decayed scans, chunked gated linear attention, matrix memory
+// with exponential gates), parallel residual streams, routers, and gated feed-forward
+// activations.
 //
 // Built as a plain C-ABI shared library (no torch headers): the Python side
 // passes raw device pointers and the current HIP stream, so the kernels are
